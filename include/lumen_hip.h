@@ -389,6 +389,102 @@ int lumen_decoder_layer_decode_f32(lumen_decoder_layer *layer, lumen_kv_cache *c
                                    const float *input_norm_dev, const float *post_norm_dev, const float *q_norm_dev,
                                    const float *k_norm_dev, const float *x_dev, float *y_dev);
 
+/* ------------------------------------------------- layered hybrid decoder
+ * A decoder-only model whose layers differ in their sequence mixer (no counterpart in the reference; beside
+ * lumen_llama_*, with the same loader, sampler, turn loop, decode graph and products).  x = embed[token] * embed_scale;
+ * a layer is x += residual_mult * mixer(norm1(x)), then x += residual_mult * ff(norm2(x)); norms are RMS norms whose
+ * stored weight has norm_offset added (1: weights stored around zero); logits = head final_norm(x).
+ * With loop_times > 0 layers [loop_start, loop_stop) run loop_times times in a row on the same weights, each pass with
+ * its own state; before pass t, x = W_in [x; x0] + step[t], x0 being the embedding output.
+ * Mixers (h: the mixer's input; tensors "l<i>.mix.<name>"):
+ *   WINDOW_ATTENTION  q, k, v, g projections; RMSNorm of the whole q and of the whole k (q.norm, k.norm); score =
+ *                     softcap tanh(q.k scale / softcap) (softcap 0: plain) - r1 ln(1 + r2 distance); softmax over the
+ *                     last `window` positions (0: all); times sigmoid(g); o
+ *   WKV               token-shift mixes mu.{r,k,v,g,w}; decay exp(-exp(w2 tanh(w1 .) + w0)); per head o = (S + u k v^T)^T r,
+ *                     S <- w S + k v^T; RMSNorm per head, times norm, times silu(gate); o
+ *   CHANNEL_DELTA     causal convolution (conv taps) + SiLU on q, k, v; unit q, k per head (unit_eps under the root, q also
+ *                     times dim^-1/2); decay exp(-exp(A_log) softplus(a2 a1 h + dt_bias)) per key channel; S <- g S;
+ *                     S <- S + k (sigmoid(b) (v - S^T k))^T; o = S^T q; RMSNorm per head, times norm, times sigmoid(g2 g1 h); o
+ * ff > 0: feed-forward mlp.down(PolyNorm(mlp.up(.))) with mlp.act = {a, b, c, e}: a N(z) + b N(z^2) + c N(z^3) + e.
+ * The state between steps -- rolling key / value stores of window - 1 + max_chunk positions, recurrent matrices in f32,
+ * convolution and token-shift inputs -- belongs to the model's one live sequence; lumen_hybrid_reset gives it back.
+ * Heads up to 256 wide, inner sizes up to 16384, up to 16 taps; sizes need not be multiples of anything. */
+#define LUMEN_MIXER_WINDOW_ATTENTION 0
+#define LUMEN_MIXER_WKV 1
+#define LUMEN_MIXER_CHANNEL_DELTA 2
+typedef struct lumen_hybrid lumen_hybrid;
+typedef struct {
+    int mixer;                       /* LUMEN_MIXER_* */
+    int heads, kv_heads, dim, vdim;  /* WKV: kv_heads = heads, vdim = dim */
+    int window;                      /* attention: positions a query sees, itself included; 0: all */
+    float scale, softcap;            /* attention */
+    int conv;                        /* CHANNEL_DELTA: taps of the causal convolution */
+    int rank_lo;                     /* inner size of the decay's low-rank product (WKV w1 / w2, CHANNEL_DELTA a1 / a2) */
+    int rank_hi;                     /* CHANNEL_DELTA: inner size of the gate's (g1 / g2) */
+    int ff;                          /* feed-forward width, 0: none */
+} lumen_hybrid_layer;
+typedef struct {
+    int vocab_size, width, num_layers;
+    int loop_start, loop_stop, loop_times; /* loop_times 0: no loop */
+    float embed_scale, norm_eps, norm_offset, residual_mult, unit_eps;
+    int max_seq_len;                 /* tokens a sequence may hold */
+    int max_chunk;                   /* longest piece a prompt is run in (0: 2048) */
+    int weight_dtype;                /* LUMEN_DTYPE_F32 or _BF16: storage of the matrices; arithmetic is f32 either way */
+} lumen_hybrid_config;
+int lumen_hybrid_create(lumen_ctx *ctx, const lumen_hybrid_config *cfg, const lumen_hybrid_layer *layers, lumen_hybrid **out);
+int lumen_hybrid_destroy(lumen_hybrid *model);
+/* parameters by name, as for lumen_llama_*; shapes must match exactly */
+int lumen_hybrid_num_params(const lumen_hybrid *model, int *n_out);
+int lumen_hybrid_param_info(const lumen_hybrid *model, int index, char *name, int name_len, int64_t *shape_out, int *ndim_out);
+int lumen_hybrid_set_param(lumen_hybrid *model, const char *name, const void *data_host, int dtype, const int64_t *shape, int ndim);
+int lumen_hybrid_load_safetensors(lumen_hybrid *model, const char *path, int *n_loaded_out, int *n_missing_out);
+/* the next s tokens of the live sequence, any s >= 1 (one token: the decode step).  want [n_want]: ascending places
+ * among them whose logits go to logits_host [n_want, vocab].  residual_host (or NULL) receives the residual stream after
+ * every layer run, [lumen_hybrid_num_runs, s, width]. */
+int lumen_hybrid_forward(lumen_hybrid *model, const int32_t *ids_host, int s, const int32_t *want_host, int n_want, float *logits_host,
+                         float *residual_host);
+int lumen_hybrid_decode_greedy(lumen_hybrid *model, int first_id, int n, int32_t *ids_out_host, float *logits_out_host);
+int lumen_hybrid_generate_turn(lumen_hybrid *model, const int32_t *new_tokens, int n_new, const int32_t *history, int n_history,
+                               const lumen_sampling *sampling, const int32_t *stop_ids, int n_stop, int32_t *out_ids, int out_cap, int *n_out);
+/* n greedy steps with every product and mixer launch between two HIP events.  Classes: 0 embedding, 1 loop input, 2 / 3
+ * attention projections / mixer, 4 / 5 WKV, 6 / 7 CHANNEL_DELTA, 8 output projection, 9 up, 10 down, 11 head. */
+int lumen_hybrid_decode_profile(lumen_hybrid *model, int first_id, int n, double *ms_sum_out, int *count_out, int n_classes);
+int lumen_hybrid_set_decode_mode(lumen_hybrid *model, int mode);
+int lumen_hybrid_reset(lumen_hybrid *model);
+int lumen_hybrid_len(const lumen_hybrid *model, int *len_out);
+int lumen_hybrid_num_runs(const lumen_hybrid *model, int *n_out);
+int lumen_hybrid_decode_bytes(const lumen_hybrid *model, int len, double *bytes_out);
+
+/* The mechanisms as operators, f32, rows one after the other.
+ * polynorm: z, out [rows, dim], coef {a, b, c, e}. */
+int lumen_polynorm_f32(lumen_ctx *ctx, const float *z_dev, const float *coef_dev, float *out_dev, int rows, int dim, float eps);
+/* mixes [n, s, dim]: h_t + (h_{t-1} - h_t) mu_i, h_{-1} = prev [dim]; next [dim] receives the last h */
+int lumen_token_shift_f32(lumen_ctx *ctx, const float *h_dev, const float *mu_dev, const float *prev_dev, float *next_dev, float *mixes_dev,
+                          int n, int s, int dim);
+/* a head's state is stored as [vdim][rows], rows = dim rounded up (zeros beyond dim) */
+int lumen_recurrence_state_rows(int dim, int *rows_out);
+/* r, k, v, z [s, heads, dim]; decay exp(-exp(z + bias)), bias and u [heads, dim]; state [heads, dim, rows] read and written */
+int lumen_wkv_f32(lumen_ctx *ctx, const float *r_dev, const float *k_dev, const float *v_dev, const float *z_dev, const float *bias_dev,
+                  const float *u_dev, float *state_dev, float *out_dev, int s, int heads, int dim);
+/* q, k [s, kv_heads, dim], v [s, heads, vdim], z [s, heads, dim], b [s, heads] (before the sigmoid) */
+int lumen_channel_delta_f32(lumen_ctx *ctx, const float *q_dev, const float *k_dev, const float *v_dev, const float *z_dev, const float *b_dev,
+                            const float *bias_dev, const float *a_log_dev, float *state_dev, float *out_dev, int s, int heads, int kv_heads,
+                            int dim, int vdim);
+/* qkv [s, 2 kv_heads dim + heads vdim]: convolution with taps_w [channels, taps] (last column: current token) + SiLU,
+ * unit q and k; prev / next [taps - 1, channels]: inputs before the first / up to the last token, oldest first */
+int lumen_conv_unit_f32(lumen_ctx *ctx, const float *qkv_dev, const float *taps_dev, const float *prev_dev, float *next_dev, float *q_dev,
+                        float *k_dev, float *v_dev, int s, int taps, int heads, int kv_heads, int dim, int vdim, float unit_eps, float q_scale);
+/* o [rows, heads, vdim] in place: RMS norm per head, times gain, times act(gate) (0 none, 1 sigmoid, 2 silu) */
+int lumen_head_norm_gate_f32(lumen_ctx *ctx, float *o_dev, const float *gain_dev, int gain_shared, const float *gate_dev, int gate_act, int rows,
+                             int heads, int vdim, float eps);
+/* s tokens at positions pos.. of a sequence whose last keys / values sit in k_ring [kv_heads, cap, dim rounded up to 4]
+ * and v_ring (position p in slot p mod cap; cap >= window - 1 + s), which receive the new ones.  gate, q_norm, k_norm
+ * and r1 / r2 may be NULL.  s == 1 runs the decode kernel, s > 1 the prompt kernel. */
+int lumen_window_attn_f32(lumen_ctx *ctx, const float *q_dev, const float *k_dev, const float *v_dev, const float *gate_dev,
+                          const float *q_norm_dev, const float *k_norm_dev, const float *r1_dev, const float *r2_dev, float *k_ring_dev,
+                          float *v_ring_dev, int cap, float *out_dev, int s, int pos, int heads, int kv_heads, int dim, int vdim, int window,
+                          float scale, float softcap, float norm_eps);
+
 #ifdef __cplusplus
 }
 #endif

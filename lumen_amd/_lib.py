@@ -41,6 +41,19 @@ class LlamaConfigStruct(C.Structure):
                 ("tie_embeddings", C.c_int), ("weight_dtype", C.c_int)]
 
 
+class HybridLayerStruct(C.Structure):  # lumen_hybrid_layer
+    _fields_ = [("mixer", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int),
+                ("window", C.c_int), ("scale", C.c_float), ("softcap", C.c_float), ("conv", C.c_int),
+                ("rank_lo", C.c_int), ("rank_hi", C.c_int), ("ff", C.c_int)]
+
+
+class HybridConfigStruct(C.Structure):  # lumen_hybrid_config
+    _fields_ = [("vocab_size", C.c_int), ("width", C.c_int), ("num_layers", C.c_int), ("loop_start", C.c_int),
+                ("loop_stop", C.c_int), ("loop_times", C.c_int), ("embed_scale", C.c_float), ("norm_eps", C.c_float),
+                ("norm_offset", C.c_float), ("residual_mult", C.c_float), ("unit_eps", C.c_float),
+                ("max_seq_len", C.c_int), ("max_chunk", C.c_int), ("weight_dtype", C.c_int)]
+
+
 _vp, _f, _i = C.c_void_p, C.c_float, C.c_int
 _pp = C.POINTER(C.c_void_p)
 
@@ -121,6 +134,29 @@ SIGNATURES = {
     "lumen_decoder_layer_create": (_i, [_vp, C.POINTER(LlamaConfigStruct), _pp]),
     "lumen_decoder_layer_destroy": (_i, [_vp]),
     "lumen_decoder_layer_decode_f32": (_i, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
+    "lumen_hybrid_create": (_i, [_vp, C.POINTER(HybridConfigStruct), C.POINTER(HybridLayerStruct), _pp]),
+    "lumen_hybrid_destroy": (_i, [_vp]),
+    "lumen_hybrid_num_params": (_i, [_vp, C.POINTER(_i)]),
+    "lumen_hybrid_param_info": (_i, [_vp, _i, C.c_char_p, _i, C.POINTER(C.c_int64), C.POINTER(_i)]),
+    "lumen_hybrid_set_param": (_i, [_vp, C.c_char_p, _vp, _i, C.POINTER(C.c_int64), _i]),
+    "lumen_hybrid_load_safetensors": (_i, [_vp, C.c_char_p, C.POINTER(_i), C.POINTER(_i)]),
+    "lumen_hybrid_forward": (_i, [_vp, _vp, _i, _vp, _i, _vp, _vp]),
+    "lumen_hybrid_decode_greedy": (_i, [_vp, _i, _i, _vp, _vp]),
+    "lumen_hybrid_generate_turn": (_i, [_vp, _vp, _i, _vp, _i, _vp, _vp, _i, _vp, _i, C.POINTER(_i)]),
+    "lumen_hybrid_decode_profile": (_i, [_vp, _i, _i, C.POINTER(C.c_double), C.POINTER(_i), _i]),
+    "lumen_hybrid_set_decode_mode": (_i, [_vp, _i]),
+    "lumen_hybrid_reset": (_i, [_vp]),
+    "lumen_hybrid_len": (_i, [_vp, C.POINTER(_i)]),
+    "lumen_hybrid_num_runs": (_i, [_vp, C.POINTER(_i)]),
+    "lumen_hybrid_decode_bytes": (_i, [_vp, _i, C.POINTER(C.c_double)]),
+    "lumen_polynorm_f32": (_i, [_vp, _vp, _vp, _vp, _i, _i, _f]),
+    "lumen_token_shift_f32": (_i, [_vp] * 6 + [_i] * 3),
+    "lumen_recurrence_state_rows": (_i, [_i, C.POINTER(_i)]),
+    "lumen_wkv_f32": (_i, [_vp] * 9 + [_i] * 3),
+    "lumen_channel_delta_f32": (_i, [_vp] * 10 + [_i] * 5),
+    "lumen_conv_unit_f32": (_i, [_vp] * 8 + [_i] * 6 + [_f] * 2),
+    "lumen_head_norm_gate_f32": (_i, [_vp, _vp, _vp, _i, _vp, _i, _i, _i, _i, _f]),
+    "lumen_window_attn_f32": (_i, [_vp] * 11 + [_i, _vp] + [_i] * 7 + [_f] * 3),
 }
 
 

@@ -1,6 +1,7 @@
 // Small HBM-bound kernels of the path: RMSNorm, SiLU / add / mul / SwiGLU,
 // embedding gather, greedy argmax and the tensor form of RoPE.
 #include "internal.h"
+#include "mixers.h"
 #include "wave_reduce.h"
 
 #include <cmath>
@@ -94,7 +95,7 @@ int launch_rmsnorm(lumen_ctx *ctx, const float *x, const float *w, float *out, i
 }
 
 // -------------------------------------------------------------- elementwise
-enum { OP_SILU, OP_ADD, OP_MUL, OP_SWIGLU, OP_COPY };
+enum { OP_SILU, OP_ADD, OP_MUL, OP_SWIGLU, OP_COPY, OP_TANH };
 
 template <int OP>
 __global__ __launch_bounds__(256) void ew_kernel(const float *__restrict__ a, const float *__restrict__ b,
@@ -108,6 +109,8 @@ __global__ __launch_bounds__(256) void ew_kernel(const float *__restrict__ a, co
             r = x * sig;
         } else if (OP == OP_COPY) {
             r = x;
+        } else if (OP == OP_TANH) {
+            r = tanhf(x);
         } else if (OP == OP_ADD) {
             r = x + b[i];
         } else if (OP == OP_MUL) {
@@ -136,6 +139,98 @@ int launch_add(lumen_ctx *ctx, const float *a, const float *b, float *out, size_
 int launch_mul(lumen_ctx *ctx, const float *a, const float *b, float *out, size_t n) { return launch_ew<OP_MUL>(ctx, a, b, out, n); }
 int launch_swiglu(lumen_ctx *ctx, const float *g, const float *u, float *out, size_t n) { return launch_ew<OP_SWIGLU>(ctx, g, u, out, n); }
 static int launch_copy(lumen_ctx *ctx, const float *x, float *out, size_t n) { return launch_ew<OP_COPY>(ctx, x, x, out, n); }
+
+int launch_tanh(lumen_ctx *ctx, const float *x, float *out, size_t n) { return launch_ew<OP_TANH>(ctx, x, x, out, n); }
+
+// ----------------------------------------------------- PolyNorm, token shift, row helpers
+// One workgroup per row; the row is read once for the three sums and once more (from cache) for the values.
+__global__ __launch_bounds__(256) void polynorm_kernel(const float *z, const float *__restrict__ coef, float *out, int dim,
+                                                       int stride, float eps) {
+    __shared__ float red[3][4];
+    const float *zr = z + (size_t)blockIdx.x * stride;
+    float *o = out + (size_t)blockIdx.x * stride;
+    const int tid = threadIdx.x;
+    float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+    for (int i = tid; i < dim; i += 256) {
+        const float v = zr[i], q = v * v, q2 = q * q;
+        s1 += q;
+        s2 += q2;
+        s3 = fmaf(q2, q, s3);
+    }
+    s1 = wave_sum(s1);
+    s2 = wave_sum(s2);
+    s3 = wave_sum(s3);
+    if ((tid & 63) == 0) {
+        red[0][tid >> 6] = s1;
+        red[1][tid >> 6] = s2;
+        red[2][tid >> 6] = s3;
+    }
+    __syncthreads();
+    const float n = (float)dim;
+    const float a1 = coef[0] / sqrtf(((red[0][0] + red[0][1]) + (red[0][2] + red[0][3])) / n + eps);
+    const float a2 = coef[1] / sqrtf(((red[1][0] + red[1][1]) + (red[1][2] + red[1][3])) / n + eps);
+    const float a3 = coef[2] / sqrtf(((red[2][0] + red[2][1]) + (red[2][2] + red[2][3])) / n + eps);
+    const float c3 = coef[3];
+    for (int i = tid; i < dim; i += 256) {
+        const float v = zr[i];
+        o[i] = fmaf(fmaf(fmaf(a3, v, a2), v, a1), v, c3);
+    }
+}
+
+int launch_polynorm(lumen_ctx *ctx, const float *z, const float *coef, float *out, int rows, int dim, int stride, float eps) {
+    if (rows <= 0 || dim <= 0) return LUMEN_OK;
+    hipLaunchKernelGGL(polynorm_kernel, dim3(rows), dim3(256), 0, ctx->stream, z, coef, out, dim, stride, eps);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+__global__ __launch_bounds__(256) void token_shift_kernel(const float *__restrict__ h, const float *__restrict__ mu,
+                                                          const float *__restrict__ prev, float *__restrict__ next,
+                                                          float *__restrict__ mixes, int n, int s, int dim) {
+    const int t = blockIdx.x;
+    const float *cur = h + (size_t)t * dim, *bef = t ? cur - dim : prev;
+    for (int i = threadIdx.x; i < dim; i += 256) {
+        const float c = cur[i], d = bef[i] - c;
+        for (int m = 0; m < n; ++m) mixes[((size_t)m * s + t) * dim + i] = fmaf(d, mu[(size_t)m * dim + i], c);
+        if (t == s - 1) next[i] = c;
+    }
+}
+
+int launch_token_shift(lumen_ctx *ctx, const float *h, const float *mu, const float *prev, float *next, float *mixes, int n,
+                       int s, int dim) {
+    if (s <= 0 || dim <= 0) return LUMEN_OK;
+    hipLaunchKernelGGL(token_shift_kernel, dim3(s), dim3(256), 0, ctx->stream, h, mu, prev, next, mixes, n, s, dim);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+__global__ __launch_bounds__(256) void add_steps_kernel(const float *__restrict__ base, const float *__restrict__ step,
+                                                        float *__restrict__ out, int rows, int dim) {
+    const size_t r = blockIdx.x;
+    const int t = blockIdx.y;
+    for (int i = threadIdx.x; i < dim; i += 256) out[((size_t)t * rows + r) * dim + i] = base[r * dim + i] + step[(size_t)t * dim + i];
+}
+
+int launch_add_steps(lumen_ctx *ctx, const float *base, const float *step, float *out, int times, int rows, int dim) {
+    if (times <= 0 || rows <= 0) return LUMEN_OK;
+    hipLaunchKernelGGL(add_steps_kernel, dim3(rows, times), dim3(256), 0, ctx->stream, base, step, out, rows, dim);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+__global__ __launch_bounds__(256) void gather_rows_kernel(const float *__restrict__ x, const int *__restrict__ idx,
+                                                          float *__restrict__ out, int dim) {
+    const float *src = x + (size_t)idx[blockIdx.x] * dim;
+    float *dst = out + (size_t)blockIdx.x * dim;
+    for (int i = threadIdx.x; i < dim; i += 256) dst[i] = src[i];
+}
+
+int launch_gather_rows(lumen_ctx *ctx, const float *x, const int *idx, float *out, int n, int dim) {
+    if (n <= 0) return LUMEN_OK;
+    hipLaunchKernelGGL(gather_rows_kernel, dim3(n), dim3(256), 0, ctx->stream, x, idx, out, dim);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
 
 // ---------------------------------------------------------------- embedding
 // out[t, :] = W[ids[t], :], src/layers/basic/embedding.rs:47-57.  ids were

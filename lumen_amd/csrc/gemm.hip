@@ -32,6 +32,11 @@ typedef unsigned int v2u __attribute__((ext_vector_type(2)));
 #define BK 32
 #define STAGE 4  // 16-byte pieces of A and of W per thread per slice: 128 rows x 32 k / 256 threads
 
+// residual + alpha * product (alpha = 1: the plain sum, bit for bit)
+__device__ __forceinline__ v4f scaled_add(const v4f r, float alpha, const v4f v) {
+    return v4f{fmaf(alpha, v.x, r.x), fmaf(alpha, v.y, r.y), fmaf(alpha, v.z, r.z), fmaf(alpha, v.w, r.w)};
+}
+
 __device__ __forceinline__ float silu_g(float g) {
     const float sig = 1.0f / (1.0f + expf(-g));
     return g * sig;
@@ -61,7 +66,7 @@ __device__ __forceinline__ void store_tile(const GemmArgs &a, const v16f (&acc)[
                     if (!(col & 1) && row < M && col < N) a.C[(size_t)row * (N >> 1) + (col >> 1)] = silu_g(v) * up;
                 } else if (row < M && col < N) {
                     const size_t o = (size_t)row * N + col;
-                    a.C[o] = (EPI == EPI_RESIDUAL) ? a.residual[o] + v : v;
+                    a.C[o] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, v, a.residual[o]) : v;
                 }
             }
 }
@@ -242,7 +247,7 @@ __device__ __forceinline__ void store_wave_tiles(const GemmArgs &a, const v16f (
                     if (!(col & 1) && row < M && col < N) a.C[(size_t)row * (N >> 1) + (col >> 1)] = silu_g(v) * up;
                 } else if (row < M && col < N) {
                     const size_t o = (size_t)row * N + col;
-                    a.C[o] = (EPI == EPI_RESIDUAL) ? a.residual[o] + v : v;
+                    a.C[o] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, v, a.residual[o]) : v;
                 }
             }
 }
@@ -520,7 +525,7 @@ __global__ __launch_bounds__(SK_THREADS) void gemm_skinny_kernel(GemmArgs a, int
                         for (int r = 0; r < R; ++r)
                             if (row + r < N) {
                                 const size_t o = mrow * N + row + r;
-                                a.C[o] = (EPI == EPI_RESIDUAL) ? a.residual[o] + acc[r][m] : acc[r][m];
+                                a.C[o] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, acc[r][m], a.residual[o]) : acc[r][m];
                             }
                     }
                 }
@@ -721,7 +726,7 @@ __global__ __launch_bounds__(256) void gemm_stream_kernel(GemmArgs a) {
                 if (!(col & 1) && row < M && col < N) a.C[(size_t)row * (N >> 1) + (col >> 1)] = silu_g(v) * up;
             } else if (row < M && col < N) {
                 const size_t o = (size_t)row * N + col;
-                a.C[o] = (EPI == EPI_RESIDUAL) ? a.residual[o] + v : v;
+                a.C[o] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, v, a.residual[o]) : v;
             }
         }
     STAGE_T_STORES_DONE(6);
@@ -753,7 +758,7 @@ __global__ __launch_bounds__(256) void gemm_reduce_kernel(GemmArgs a, int splits
                 a.C[2 * q] = silu_g(v.x) * v.y;
                 a.C[2 * q + 1] = silu_g(v.z) * v.w;
             } else if (EPI == EPI_RESIDUAL) {
-                *(v4 *)(a.C + 4 * q) = r4 + v;
+                *(v4 *)(a.C + 4 * q) = scaled_add(r4, a.alpha, v);
             } else {
                 *(v4 *)(a.C + 4 * q) = v;
             }
@@ -773,7 +778,7 @@ __global__ __launch_bounds__(256) void gemm_reduce_kernel(GemmArgs a, int splits
         for (size_t o = (size_t)blockIdx.x * blockDim.x + threadIdx.x; o < MN; o += stride) {
             float v = 0.f;
             for (int s = 0; s < splits; ++s) v += a.part[(size_t)s * MN + o];
-            a.C[o] = (EPI == EPI_RESIDUAL) ? a.residual[o] + v : v;
+            a.C[o] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, v, a.residual[o]) : v;
         }
     }
 }
@@ -805,7 +810,7 @@ __global__ __launch_bounds__(256) void gemm_reduce_norm_kernel(GemmArgs a, int s
 #pragma unroll
             for (int s = 0; s < GEMM_MAX_SPLITS; ++s)
                 if (s < splits) acc += pv[s];
-            v[i] = r4 + acc;
+            v[i] = scaled_add(r4, a.alpha, acc);
             *(v4 *)(a.C + base + k) = v[i];
         }
     }

@@ -105,6 +105,98 @@ __device__ __forceinline__ void stage_x(float *xs, const float *__restrict__ x, 
     __syncthreads();
 }
 
+// One sum over the workgroup for each of n values, the same in every thread; red [n][GEMV_MAX_WAVES].
+template <int NV>
+__device__ __forceinline__ void workgroup_sums(float (&v)[NV], float (*red)[GEMV_MAX_WAVES], int nwaves) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i) v[i] = wave_sum(v[i]);
+    if ((threadIdx.x & 63) == 0)
+#pragma unroll
+        for (int i = 0; i < NV; ++i) red[i][threadIdx.x >> 6] = v[i];
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        v[i] = 0.f;
+        for (int w = 0; w < nwaves; ++w) v[i] += red[i][w];
+    }
+}
+
+// The same raw staging for a prologue that is not a plain norm: calls put(k, v) for every 16-byte piece (zero beyond K).
+template <int XB, typename Put>
+__device__ __forceinline__ void stage_pieces(const float *__restrict__ x, int K, int kpad, int nwaves, Put put) {
+    const int nthreads = nwaves * 64;
+    for (int k0 = (int)threadIdx.x * 4; k0 < kpad; k0 += nthreads * 4 * XB) {
+        v4f v[XB];
+#pragma unroll
+        for (int i = 0; i < XB; ++i) {
+            const int k = k0 + i * nthreads * 4;
+            v[i] = v4f{0.f, 0.f, 0.f, 0.f};
+            if (k < K) v[i] = *(const v4f *)(x + k);
+        }
+#pragma unroll
+        for (int i = 0; i < XB; ++i) {
+            const int k = k0 + i * nthreads * 4;
+            if (k < kpad) put(k, v[i]);
+        }
+    }
+}
+
+// PolyNorm of the staged vector: one pass over x takes the sums of z^2, z^4 and z^6, a second one in LDS applies
+// ((c3 z + c2) z + c1) z + e with the inverse root mean squares folded into the coefficients.
+template <int XB>
+__device__ __forceinline__ void stage_polynorm(float *xs, const float *__restrict__ x, const float *__restrict__ coef,
+                                               float eps, int dim, int K, int kpad, int nwaves) {
+    __shared__ float red_p[3][GEMV_MAX_WAVES];
+    const float c0 = coef[0], c1 = coef[1], c2 = coef[2], c3 = coef[3];
+    float s[3] = {0.f, 0.f, 0.f};
+    stage_pieces<XB>(x, K, kpad, nwaves, [&](int k, const v4f v) {
+        *(v4f *)(xs + k) = v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const float q = v[e] * v[e], q2 = q * q;
+            s[0] += q;
+            s[1] += q2;
+            s[2] = fmaf(q2, q, s[2]);
+        }
+    });
+    workgroup_sums(s, red_p, nwaves);
+    const float n = (float)dim;
+    const float a1 = c0 / sqrtf(s[0] / n + eps), a2 = c1 / sqrtf(s[1] / n + eps), a3 = c2 / sqrtf(s[2] / n + eps);
+    for (int k = (int)threadIdx.x * 4; k < K; k += nwaves * 64 * 4) {
+        v4f v = *(const v4f *)(xs + k);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = fmaf(fmaf(fmaf(a3, v[e], a2), v[e], a1), v[e], c3);
+        *(v4f *)(xs + k) = v;
+    }
+    __syncthreads();
+}
+
+// RMSNorm and token shift: h = norm(x), then h + (h' - h) mu.  `writer`: this workgroup leaves h for the next token.
+template <int XB>
+__device__ __forceinline__ void stage_shift(float *xs, const float *__restrict__ x, const float *__restrict__ g, float eps,
+                                            const float *__restrict__ mu, const float *__restrict__ prev, float *next,
+                                            bool writer, int K, int kpad, int nwaves) {
+    __shared__ float red_s[1][GEMV_MAX_WAVES];
+    float ss[1] = {0.f};
+    stage_pieces<XB>(x, K, kpad, nwaves, [&](int k, const v4f v) {
+        *(v4f *)(xs + k) = v;
+        ss[0] += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+    });
+    workgroup_sums(ss, red_s, nwaves);
+    const float inv = 1.0f / sqrtf(ss[0] / (float)K + eps);
+    for (int k = (int)threadIdx.x * 4; k < K; k += nwaves * 64 * 4) {
+        v4f v = *(const v4f *)(xs + k);
+        const v4f gg = *(const v4f *)(g + k), pp = *(const v4f *)(prev + k), mm = *(const v4f *)(mu + k);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = v[e] * inv * gg[e];
+        if (writer) *(v4f *)(next + k) = v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = fmaf(pp[e] - v[e], mm[e], v[e]);
+        *(v4f *)(xs + k) = v;
+    }
+    __syncthreads();
+}
+
 // Latency-bound launches (every wavefront has a single unit whose loads all go out at once): the first
 // GEMV_EARLY pieces of x of a thread -- and of the norm gains -- are requested BEFORE the weights.  Loads
 // return in the order they were issued, so x queued behind the weights would arrive after them, and the
@@ -250,7 +342,10 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
     constexpr int U = 8 / R;                   // loads in flight per lane per row
     constexpr int PIECE = SWEEP * U;           // elements of a row one piece covers
     constexpr int ESZ = BF16 ? 2 : 4;
-    const int K = K_hot, N = N_hot, D = D_hot;
+    // (several products in one launch: this workgroup's rows)
+    const int seg = PRO == PRO_SHIFT ? (int)blockIdx.y : 0;
+    const int K = K_hot, D = D_hot;
+    const int N = PRO == PRO_SHIFT ? (seg == a.shift_segs - 1 ? a.shift_last_rows : a.shift_rows) : N_hot;
     const int kpad = (K + PIECE - 1) / PIECE * PIECE;  // xs is zero from K to kpad
 
     STAGE_T(0);
@@ -258,8 +353,10 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
     const int gw = blockIdx.x * nwaves + (threadIdx.x >> 6);
     const int nw = nblocks * nwaves;
     const int nunits = (N + R - 1) / R;
-    const char *Wb = (const char *)W_hot;
     const size_t row_bytes = (size_t)K * ESZ;
+    const char *Wb = (const char *)W_hot + (PRO == PRO_SHIFT ? (size_t)seg * a.shift_rows * row_bytes : 0);
+    float *y_out = a.y + (PRO == PRO_SHIFT ? (size_t)seg * a.shift_rows : 0);
+    if (PRO == PRO_SHIFT && (int)blockIdx.x * nwaves >= (N + R - 1) / R) return;  // (no unit of a short segment here)
     const int half_d = D >> 1;
 
     // row r of unit u: consecutive rows, or the RoPE pair (j, j + D/2) of one head
@@ -299,7 +396,7 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
         }
     };
 
-    constexpr bool EARLY = XB == 0 && PRO != PRO_ATTN_FOLD;
+    constexpr bool EARLY = XB == 0 && (PRO == PRO_NONE || PRO == PRO_RMSNORM);
     v4f xe[GEMV_EARLY], ge[GEMV_EARLY];
     // (with a row selector -- the first layer's gather -- the address of x needs a trip to memory itself:
     // then the weights go first)
@@ -345,6 +442,12 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
     preload(gw);
     STAGE_T(1);
     if (PRO == PRO_ATTN_FOLD) stage_attn_fold(xs, a, K, kpad, nwaves);
+    else if (PRO == PRO_POLYNORM) stage_polynorm<(XB > 0 ? XB : 1)>(xs, xin, norm_w_hot, a.eps, a.norm_dim, K, kpad, nwaves);
+    else if (PRO == PRO_SHIFT) {
+        const unsigned slot = *a.shift_step & 1u;
+        stage_shift<(XB > 0 ? XB : 1)>(xs, xin, norm_w_hot, a.eps, a.shift_mu + (size_t)seg * K, a.shift_state + (size_t)slot * K,
+                                       a.shift_state + (size_t)(slot ^ 1u) * K, seg == 0 && blockIdx.x == 0, K, kpad, nwaves);
+    }
     else if (EARLY) stage_x_early<PRO>(xs, xin, norm_w_hot, a.eps, K, kpad, nwaves, xe, ge);
     else stage_x<PRO, (XB > 0 ? XB : 1)>(xs, xin, norm_w_hot, a.eps, K, kpad, nwaves);
     STAGE_T(2);
@@ -410,7 +513,7 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
                         const int row = u * R + r;
                         if (row < N) {
                             // residual: x + y, src/ops/arithmetic.rs:48-51 via src/models/llama.rs:110,115
-                            a.y[row] = (EPI == EPI_RESIDUAL) ? (r == 0 ? pre0 : pre1) + acc[r] : acc[r];
+                            y_out[row] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, acc[r], r == 0 ? pre0 : pre1) : acc[r];
                         }
                     }
                 }
@@ -575,6 +678,10 @@ template <bool BF16, int R, int XB, bool KA>
 static void launch_pro(const GemvArgs &a, dim3 grid, int threads, size_t lds, hipStream_t s) {
     if (a.pro == PRO_ATTN_FOLD)  // o_proj only (launch_gemv checks): one row per unit, residual epilogue
         hipLaunchKernelGGL((gemv_kernel<BF16, 1, PRO_ATTN_FOLD, EPI_RESIDUAL, XB, KA>), grid, dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
+    else if (a.pro == PRO_POLYNORM)  // the down product of a feed-forward (launch_gemv checks): residual epilogue
+        hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_POLYNORM, EPI_RESIDUAL, (XB == 0 ? 1 : XB), KA>), grid, dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
+    else if (a.pro == PRO_SHIFT)  // token-shift products (launch_gemv checks): plain store
+        hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_SHIFT, EPI_STORE, (XB == 0 ? 1 : XB), KA>), dim3(grid.x, a.shift_segs), dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
     else if (a.pro == PRO_RMSNORM)
         launch_epi<BF16, R, PRO_RMSNORM, XB, KA>(a, grid, threads, lds, s);
     else
@@ -645,7 +752,7 @@ GemvPick gemv_pick(int num_cus, int N, int K, int w_bf16, int pro, int epi, bool
     // at a time from three pieces per thread on.
     const int x_pieces = (kpad + p.threads * 4 - 1) / (p.threads * 4);
     const int nunits = (N + p.R - 1) / p.R;
-    const bool early_x = pro != PRO_ATTN_FOLD && x_pieces <= GEMV_EARLY && kpad / piece <= 2 &&
+    const bool early_x = (pro == PRO_NONE || pro == PRO_RMSNORM) && x_pieces <= GEMV_EARLY && kpad / piece <= 2 &&
                          nunits <= p.blocks * (p.threads / 64);
     p.xb = early_x ? 0 : x_pieces > 2 ? 4 : 1;
     p.ka = K % piece == 0;  // whole pieces: no clamped load positions
@@ -684,6 +791,13 @@ int launch_gemv(lumen_ctx *ctx, const GemvArgs &a) {
             LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over attention partials: one row per unit, residual epilogue, at most %d slices (got %d)",
                        GEMV_FOLD_MAX_SLICES, a.attn_nslices);
     }
+    if (a.pro == PRO_POLYNORM && (a.epi != EPI_RESIDUAL || !a.norm_w || a.norm_dim <= 0))
+        LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over a PolyNorm input: residual epilogue, four coefficients and the element count");
+    if (a.pro == PRO_SHIFT &&
+        (a.epi != EPI_STORE || !a.norm_w || !a.shift_mu || !a.shift_state || !a.shift_step || a.shift_segs < 1 || a.row_sel ||
+         a.shift_rows != a.N || a.shift_last_rows < 1 || a.shift_last_rows > a.N ||
+         ((((uintptr_t)a.shift_mu | (uintptr_t)a.shift_state | (uintptr_t)a.norm_w) & 15) != 0)))
+        LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over token-shift mixes: store epilogue, mixes, state and segment sizes");
     if ((a.epi == EPI_SWIGLU || a.epi == EPI_ROPE_QKV) && (a.N & 1))
         LUMEN_FAIL(LUMEN_ERR_SHAPE, "paired-row epilogue needs an even row count, got %d", a.N);
     if (a.epi == EPI_ARGMAX) {

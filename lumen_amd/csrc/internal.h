@@ -94,7 +94,11 @@ struct lumen_kv_cache {
 // ---------------------------------------------------------------- launchers
 // Every launcher validates nothing: callers check shapes first.
 
-enum GemvPro { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_ATTN_FOLD = 2 };
+// PRO_POLYNORM: x is the vector z of a feed-forward and enters the product as a N(z) + b N(z^2) + c N(z^3) + e (powers
+// element by element, N divides by the root mean square over norm_dim elements); norm_w = {a, b, c, e}.
+// PRO_SHIFT: RMSNorm, then the token-shift mix h + (h' - h) mu of h with the previous token's h'; gridDim.y products
+// at once, each with a mix of its own (GemvArgs::shift_*).
+enum GemvPro { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_ATTN_FOLD = 2, PRO_POLYNORM = 3, PRO_SHIFT = 4 };
 enum GemvEpi { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ARGMAX = 3, EPI_ROPE_QKV = 4 };
 
 struct GemvArgs {
@@ -107,6 +111,15 @@ struct GemvArgs {
     const float *norm_w;  // PRO_RMSNORM: gain [K]
     float eps;
     const float *residual;  // EPI_RESIDUAL: [N]
+    float alpha = 1.0f;     // EPI_RESIDUAL: y = residual + alpha * (W x)
+    int norm_dim;           // PRO_POLYNORM: elements the mean is taken over (0: K)
+    // PRO_SHIFT: W holds shift_segs matrices one after the other, shift_rows rows each but shift_last_rows in the last;
+    // segment s reads the mix of shift_mu [shift_segs][K].  h' is slot (*shift_step & 1) of shift_state [2][K]; the
+    // other slot receives this token's h.
+    const float *shift_mu;
+    float *shift_state;
+    const unsigned *shift_step;
+    int shift_segs, shift_rows, shift_last_rows;
     // x (and, with residual_sel, the residual) is row *row_sel of a [rows, row_stride] table:
     // the embedding gather folded into the first layer's GEMVs
     const int *row_sel;
@@ -161,6 +174,7 @@ struct GemmArgs {
     int w_bf16;
     int epi;
     const float *residual;  // [M, N]
+    float alpha = 1.0f;     // EPI_RESIDUAL: C = residual + alpha * (A W^T)
     float *part;            // split-K partial tiles [splits, M, N] (set by the launcher)
     // optional, with EPI_RESIDUAL: the RMSNorm of the finished rows as well, norm_out [M, N] = (C * inv_rms) * norm_w
     // (src/layers/norm/rms_norm.rs:45-58): where K is split the pass that adds the splits takes it along (one

@@ -9,6 +9,7 @@
 // replayed per token; greedy generation never returns to the host between
 // tokens.
 #include "internal.h"
+#include "model_common.h"
 
 #include <algorithm>
 #include <cmath>
@@ -299,7 +300,7 @@ extern "C" int lumen_llama_create(lumen_ctx *ctx, const lumen_llama_config *cfg,
 }
 
 // ----------------------------------------------------------- parameter upload
-static void f32_to_bf16_host(const float *src, uint16_t *dst, size_t n) {
+void f32_to_bf16_host(const float *src, uint16_t *dst, size_t n) {
     for (size_t i = 0; i < n; ++i) {
         uint32_t u;
         memcpy(&u, src + i, 4);
@@ -312,7 +313,7 @@ static void f32_to_bf16_host(const float *src, uint16_t *dst, size_t n) {
     }
 }
 
-static void bf16_to_f32_host(const uint16_t *src, float *dst, size_t n) {
+void bf16_to_f32_host(const uint16_t *src, float *dst, size_t n) {
     for (size_t i = 0; i < n; ++i) {
         const uint32_t u = (uint32_t)src[i] << 16;  // half::bf16::to_f32, src/loader.rs:58
         memcpy(dst + i, &u, 4);
@@ -677,25 +678,7 @@ static int ensure_decode_graph(lumen_llama *m) {
     if (m->graph_exec) return LUMEN_OK;
     m->graph_expect_short = expect_short_cache(m);
     m->graph_slices = chain_plan_key(m);
-    hipStream_t s = m->ctx->stream;
-    HIP_TRY(hipStreamSynchronize(s));
-    HIP_TRY(hipStreamBeginCapture(s, hipStreamCaptureModeThreadLocal));
-    const int rc = enqueue_decode_step(m);
-    hipGraph_t g = nullptr;
-    const hipError_t e = hipStreamEndCapture(s, &g);
-    if (rc != LUMEN_OK) {
-        if (g) hipGraphDestroy(g);
-        return rc;
-    }
-    if (e != hipSuccess) LUMEN_FAIL(LUMEN_ERR_HIP, "hipStreamEndCapture failed: %s", hipGetErrorString(e));
-    const hipError_t ei = hipGraphInstantiate(&m->graph_exec, g, nullptr, nullptr, 0);
-    if (ei != hipSuccess) {
-        hipGraphDestroy(g);
-        m->graph_exec = nullptr;
-        LUMEN_FAIL(LUMEN_ERR_HIP, "hipGraphInstantiate failed: %s", hipGetErrorString(ei));
-    }
-    m->graph = g;
-    return LUMEN_OK;
+    return record_graph(m->ctx->stream, [&]() { return enqueue_decode_step(m); }, &m->graph, &m->graph_exec);
 }
 
 // one decode step: a graph replay, or the same launches one by one

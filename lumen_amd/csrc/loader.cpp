@@ -21,9 +21,8 @@
 #include <string>
 #include <vector>
 
-#include "../../include/lumen_hip.h"
+#include "model_common.h"
 
-void lumen_set_error(const char *fmt, ...);
 // names of the model's parameters in the order of LlamaModel::named_parameters and their shapes
 int lumen_llama_param_list(const lumen_llama *m, std::vector<std::string> &names, std::vector<std::vector<int64_t>> &shapes);
 
@@ -243,23 +242,14 @@ extern "C" int lumen_safetensors_find(const char *path, const char *name, int *d
     return LUMEN_OK;
 }
 
-extern "C" int lumen_llama_load_safetensors(lumen_llama *m, const char *path, int *n_loaded_out, int *n_missing_out) {
-    if (n_loaded_out) *n_loaded_out = 0;
-    if (n_missing_out) *n_missing_out = 0;
-    if (!m || !path) {
-        lumen_set_error("llama_load_safetensors: null argument");
-        return LUMEN_ERR_INVALID;
-    }
+int load_safetensors_into(const char *path, const std::vector<std::string> &names, const std::vector<std::vector<int64_t>> &shapes,
+                          const std::function<int(const char *, const void *, int, const int64_t *, int)> &set_param,
+                          int *n_loaded_out, int *n_missing_out) {
     Mapping map;
     std::map<std::string, Entry> entries;
     const unsigned char *data = nullptr;
     uint64_t data_len = 0;
     int rc = open_safetensors(path, map, entries, data, data_len);
-    if (rc != LUMEN_OK) return rc;
-
-    std::vector<std::string> names;
-    std::vector<std::vector<int64_t>> shapes;
-    rc = lumen_llama_param_list(m, names, shapes);
     if (rc != LUMEN_OK) return rc;
     int loaded = 0, missing = 0;
     for (size_t i = 0; i < names.size(); ++i) {
@@ -294,11 +284,29 @@ extern "C" int lumen_llama_load_safetensors(lumen_llama *m, const char *path, in
                             (unsigned long long)((en.end - en.begin) / esz), (unsigned long long)want);
             return LUMEN_ERR_SHAPE;
         }
-        rc = lumen_llama_set_param(m, names[i].c_str(), data + en.begin, dtype, shapes[i].data(), (int)shapes[i].size());
+        rc = set_param(names[i].c_str(), data + en.begin, dtype, shapes[i].data(), (int)shapes[i].size());
         if (rc != LUMEN_OK) return rc;
         ++loaded;
     }
     if (n_loaded_out) *n_loaded_out = loaded;
     if (n_missing_out) *n_missing_out = missing;
     return LUMEN_OK;
+}
+
+extern "C" int lumen_llama_load_safetensors(lumen_llama *m, const char *path, int *n_loaded_out, int *n_missing_out) {
+    if (n_loaded_out) *n_loaded_out = 0;
+    if (n_missing_out) *n_missing_out = 0;
+    if (!m || !path) {
+        lumen_set_error("llama_load_safetensors: null argument");
+        return LUMEN_ERR_INVALID;
+    }
+    std::vector<std::string> names;
+    std::vector<std::vector<int64_t>> shapes;
+    const int rc = lumen_llama_param_list(m, names, shapes);
+    if (rc != LUMEN_OK) return rc;
+    return load_safetensors_into(path, names, shapes,
+                                 [m](const char *n, const void *d, int t, const int64_t *sh, int nd) {
+                                     return lumen_llama_set_param(m, n, d, t, sh, nd);
+                                 },
+                                 n_loaded_out, n_missing_out);
 }

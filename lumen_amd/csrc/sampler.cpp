@@ -11,9 +11,7 @@
 #include <cstdint>
 #include <vector>
 
-#include "../../include/lumen_hip.h"
-
-void lumen_set_error(const char *fmt, ...);
+#include "model_common.h"
 
 // splitmix64: state += golden gamma, output mixed; the top 24 bits make a float in [0, 1)
 extern "C" float lumen_rand01(uint64_t *state) {
@@ -98,41 +96,36 @@ extern "C" int lumen_sample_top_p_f32(const float *logits, int n, float temperat
 // One turn of the chat loop, main.rs:325-378, without the tokenizer: the caller passes the new
 // tokens of the turn and the tokens already in the cache; text-based stops (:364-366) are the
 // caller's business.
-extern "C" int lumen_llama_generate_turn(lumen_llama *m, const int32_t *new_tokens, int n_new, const int32_t *history,
-                                         int n_history, const lumen_sampling *sp, const int32_t *stop_ids, int n_stop,
-                                         int32_t *out_ids, int out_cap, int *n_out) {
+int generate_turn(const TurnModel &m, const int32_t *new_tokens, int n_new, const int32_t *history, int n_history,
+                  const lumen_sampling *sp, const int32_t *stop_ids, int n_stop, int32_t *out_ids, int out_cap, int *n_out) {
     if (n_out) *n_out = 0;
-    if (!m || !new_tokens || !sp || !out_ids || !n_out || (n_history > 0 && !history) || (n_stop > 0 && !stop_ids)) {
-        lumen_set_error("llama_generate_turn: null argument");
+    if (!new_tokens || !sp || !out_ids || !n_out || (n_history > 0 && !history) || (n_stop > 0 && !stop_ids)) {
+        lumen_set_error("generate_turn: null argument");
         return LUMEN_ERR_INVALID;
     }
     if (n_new <= 0) {
-        lumen_set_error("llama_generate_turn: empty turn");
+        lumen_set_error("generate_turn: empty turn");
         return LUMEN_ERR_SHAPE;
     }
-    lumen_llama_config cfg;
-    int rc = lumen_llama_get_config(m, &cfg);
-    if (rc != LUMEN_OK) return rc;
     int cur = 0;
-    rc = lumen_llama_kv_len(m, &cur);
+    int rc = m.len(&cur);
     if (rc != LUMEN_OK) return rc;
-    if (cur + n_new + 8 >= cfg.max_seq_len) {  // :266: the reference resets and rebuilds the prompt here
+    if (cur + n_new + 8 >= m.max_len) {  // :266: the reference resets and rebuilds the prompt here
         lumen_set_error("KV cache overflow: len=%d + %d new tokens + 8 >= max_seq=%d (reset and start a first turn)", cur,
-                        n_new, cfg.max_seq_len);
+                        n_new, m.max_len);
         return LUMEN_ERR_KV_OVERFLOW;
     }
     std::vector<int32_t> all(history, history + (n_history > 0 ? n_history : 0));
     all.insert(all.end(), new_tokens, new_tokens + n_new);
-    std::vector<float> ids(n_new), logits((size_t)cfg.vocab_size);
-    for (int i = 0; i < n_new; ++i) ids[i] = (float)new_tokens[i];  // tensor_from_token_ids, :143-152
-    rc = lumen_llama_forward(m, ids.data(), n_new, logits.data(), 0);
+    std::vector<float> logits((size_t)m.vocab);
+    rc = m.forward(new_tokens, n_new, logits.data());
     if (rc != LUMEN_OK) return rc;
     uint64_t state = sp->seed;
     const int window = sp->recent_window > 0 ? sp->recent_window : 0;
     for (int g = 0; g < sp->max_gen && *n_out < out_cap; ++g) {
         const size_t start = all.size() > (size_t)window ? all.size() - (size_t)window : 0;  // :337-338
         int32_t next = 0;
-        rc = lumen_sample_top_p_f32(logits.data(), cfg.vocab_size, sp->temperature, sp->top_p, sp->repetition_penalty,
+        rc = lumen_sample_top_p_f32(logits.data(), m.vocab, sp->temperature, sp->top_p, sp->repetition_penalty,
                                     all.data() + start, (int)(all.size() - start), lumen_rand01(&state), &next);
         if (rc != LUMEN_OK) return rc;
         bool stop = false;
@@ -140,12 +133,33 @@ extern "C" int lumen_llama_generate_turn(lumen_llama *m, const int32_t *new_toke
         if (stop) break;  // :348-350
         all.push_back(next);
         out_ids[(*n_out)++] = next;
-        const float one = (float)next;
-        rc = lumen_llama_forward(m, &one, 1, logits.data(), 0);  // :361-367
+        rc = m.forward(&next, 1, logits.data());  // :361-367
         if (rc != LUMEN_OK) return rc;
-        rc = lumen_llama_kv_len(m, &cur);
+        rc = m.len(&cur);
         if (rc != LUMEN_OK) return rc;
-        if (cur + 2 >= cfg.max_seq_len) break;  // :370-372
+        if (cur + 2 >= m.max_len) break;  // :370-372
     }
     return LUMEN_OK;
+}
+
+extern "C" int lumen_llama_generate_turn(lumen_llama *m, const int32_t *new_tokens, int n_new, const int32_t *history,
+                                         int n_history, const lumen_sampling *sp, const int32_t *stop_ids, int n_stop,
+                                         int32_t *out_ids, int out_cap, int *n_out) {
+    if (n_out) *n_out = 0;
+    if (!m) {
+        lumen_set_error("llama_generate_turn: null argument");
+        return LUMEN_ERR_INVALID;
+    }
+    lumen_llama_config cfg;
+    const int rc = lumen_llama_get_config(m, &cfg);
+    if (rc != LUMEN_OK) return rc;
+    TurnModel t;
+    t.vocab = cfg.vocab_size;
+    t.max_len = cfg.max_seq_len;
+    t.forward = [m](const int32_t *ids, int n, float *logits) {
+        std::vector<float> f(ids, ids + n);  // tensor_from_token_ids, main.rs:143-152
+        return lumen_llama_forward(m, f.data(), n, logits, 0);
+    };
+    t.len = [m](int *n) { return lumen_llama_kv_len(m, n); };
+    return generate_turn(t, new_tokens, n_new, history, n_history, sp, stop_ids, n_stop, out_ids, out_cap, n_out);
 }

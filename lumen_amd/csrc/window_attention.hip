@@ -1,0 +1,391 @@
+// Causal attention over a sliding window with shaped scores (soft cap, logarithmic distance bias), RMSNorm of the whole
+// query and key projections in front and an element-wise output gate behind.  Keys and values live in a ring of `cap`
+// positions (slot = position mod cap): what a window can still see is never overwritten, and memory does not grow
+// with the sequence.  All arithmetic is f32.
+#include "mixers.h"
+#include "wave_reduce.h"
+
+typedef float v4f __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ float shaped_score(float dot, float scale, float softcap, float r1, float r2, int dist) {
+    float s = dot * scale;
+    if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+    return s - r1 * logf(1.0f + r2 * (float)dist);
+}
+
+__device__ __forceinline__ float gate_w(float z, int act) {
+    const float sig = 1.0f / (1.0f + expf(-z));
+    return act == GATE_SIGMOID ? sig : act == GATE_SILU ? z * sig : 1.0f;
+}
+
+// ------------------------------------------------------------------ decode
+#define WD_THREADS 512
+#define WD_WAVES (WD_THREADS / 64)
+
+int window_attn_slices(int window) { return (window + WINDOW_SLICE_KEYS - 1) / WINDOW_SLICE_KEYS; }
+
+// One workgroup per (query head, slice of up to 512 keys).  Scores: a key belongs to a row of 16 lanes, 16-byte loads;
+// thread k then shapes score k; the value rows are walked by groups of 16, 32 or 64 lanes whose sums meet in LDS.
+// DB: 64-float blocks of a key row, LV: lanes per value row.
+template <int DB, int LV>
+__global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArgs a) {
+    constexpr int GROUPS = WD_THREADS / LV;
+    constexpr int KEYS = WINDOW_SLICE_KEYS / (WD_WAVES * 4);  // keys of a row of 16 lanes
+    constexpr int U = DB == 1 ? 8 : DB == 2 ? 4 : 2;          // key rows in flight
+    __shared__ __align__(16) float qs[DB * 64], kn[DB * 64], vn[LV * 4];
+    __shared__ float sc[WINDOW_SLICE_KEYS];
+    __shared__ __align__(16) float ctx[GROUPS][LV * 4];
+    __shared__ float red[2][WD_WAVES], red_m[WD_WAVES], red_l[WD_WAVES];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, i16 = lane & 15;
+    const int h = blockIdx.x, slice = blockIdx.y, rep = a.heads / a.kv_heads, hk = h / rep, D = a.dim, Dv = a.vdim;
+    const int pos = *a.pos_dev;
+    const int lo = max(0, pos - a.window + 1) + slice * WINDOW_SLICE_KEYS;  // first key of the slice
+    const int n = min(WINDOW_SLICE_KEYS, pos + 1 - lo);
+    if (n <= 0) return;
+    const bool has_new = lo + n - 1 == pos;
+    const float *kr = a.k_ring + (size_t)hk * a.cap * a.dpad, *vr = a.v_ring + (size_t)hk * a.cap * a.vpad;
+
+    const int row0 = wave * 4 + (lane >> 4);  // this row's keys: row0, row0 + 32, ...
+    v4f kb[U][DB];
+    auto fetch = [&](int i0) {
+#pragma unroll
+        for (int i = 0; i < U; ++i) {
+            const int key = min(row0 + (i0 + i) * (WD_WAVES * 4), n - 1);
+            const float *p = kr + (size_t)((lo + key) % a.cap) * a.dpad;
+#pragma unroll
+            for (int b = 0; b < DB; ++b) {
+                const int d = b * 64 + i16 * 4;
+                kb[i][b] = v4f{0.f, 0.f, 0.f, 0.f};
+                if (d < a.dpad) kb[i][b] = *(const v4f *)(p + d);
+            }
+        }
+    };
+    fetch(0);
+
+    // queries and the new key, normalised over all heads together
+    float sq = 0.f, sk = 0.f;
+    if (a.q_norm_w)
+        for (int i = tid; i < a.heads * D; i += WD_THREADS) sq = fmaf(a.q[i], a.q[i], sq);
+    if (a.k_norm_w && has_new)
+        for (int i = tid; i < a.kv_heads * D; i += WD_THREADS) sk = fmaf(a.k[i], a.k[i], sk);
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if (lane == 0) {
+        red[0][wave] = sq;
+        red[1][wave] = sk;
+    }
+    __syncthreads();
+    sq = sk = 0.f;
+#pragma unroll
+    for (int w = 0; w < WD_WAVES; ++w) {
+        sq += red[0][w];
+        sk += red[1][w];
+    }
+    const float iq = 1.0f / sqrtf(sq / (float)(a.heads * D) + a.norm_eps);
+    const float ik = 1.0f / sqrtf(sk / (float)(a.kv_heads * D) + a.norm_eps);
+    const bool writer = has_new && h % rep == 0;
+    const size_t slot = (size_t)(pos % a.cap);
+    for (int d = tid; d < DB * 64; d += WD_THREADS) {
+        float q = 0.f, k = 0.f;
+        if (d < D) {
+            q = a.q[h * D + d];
+            if (a.q_norm_w) q = q * iq * a.q_norm_w[h * D + d];
+            if (has_new) {
+                k = a.k[hk * D + d];
+                if (a.k_norm_w) k = k * ik * a.k_norm_w[hk * D + d];
+            }
+        }
+        qs[d] = q;
+        kn[d] = k;
+        if (writer && d < a.dpad) a.k_ring[((size_t)hk * a.cap + slot) * a.dpad + d] = k;
+    }
+    for (int d = tid; d < LV * 4; d += WD_THREADS) {
+        const float v = has_new && d < Dv ? a.v[hk * Dv + d] : 0.f;
+        vn[d] = v;
+        if (writer && d < a.vpad) a.v_ring[((size_t)hk * a.cap + slot) * a.vpad + d] = v;
+    }
+    __syncthreads();
+
+    v4f q4[DB];
+#pragma unroll
+    for (int b = 0; b < DB; ++b) q4[b] = *(const v4f *)(qs + b * 64 + i16 * 4);
+    for (int i0 = 0; i0 < KEYS; i0 += U) {
+        if (i0 * (WD_WAVES * 4) >= n) break;  // (uniform)
+        if (i0) fetch(i0);
+#pragma unroll
+        for (int i = 0; i < U; ++i) {
+            const int key = row0 + (i0 + i) * (WD_WAVES * 4);
+            const bool is_new = lo + key == pos;
+            float s = 0.f;
+#pragma unroll
+            for (int b = 0; b < DB; ++b) {
+                v4f k4 = kb[i][b];
+                if (is_new) k4 = *(const v4f *)(kn + b * 64 + i16 * 4);
+                s = fmaf(q4[b].x, k4.x, s);
+                s = fmaf(q4[b].y, k4.y, s);
+                s = fmaf(q4[b].z, k4.z, s);
+                s = fmaf(q4[b].w, k4.w, s);
+            }
+            s = row16_sum(s);
+            if (i16 == 0 && key < n) sc[key] = s;
+        }
+    }
+    __syncthreads();
+    const float r1 = a.r1 ? a.r1[h] : 0.f, r2 = a.r1 ? a.r2[h] : 0.f;
+    float s = -INFINITY;
+    if (tid < n) s = shaped_score(sc[tid], a.scale, a.softcap, r1, r2, pos - lo - tid);
+    float m = wave_max(s);
+    if (lane == 0) red_m[wave] = m;
+    __syncthreads();
+    m = red_m[0];
+#pragma unroll
+    for (int w = 1; w < WD_WAVES; ++w) m = fmaxf(m, red_m[w]);
+    const float p = tid < n ? expf(s - m) : 0.f;
+    sc[tid] = p;
+    float l = wave_sum(p);
+    if (lane == 0) red_l[wave] = l;
+    __syncthreads();
+    l = 0.f;
+#pragma unroll
+    for (int w = 0; w < WD_WAVES; ++w) l += red_l[w];
+
+    const int grp = tid / LV, d4 = (tid % LV) * 4;
+    v4f acc = {0.f, 0.f, 0.f, 0.f};
+    const bool col_ok = d4 < a.vpad;
+#pragma unroll 8
+    for (int key = grp; key < n; key += GROUPS) {
+        v4f v4 = {0.f, 0.f, 0.f, 0.f};
+        if (lo + key == pos) v4 = *(const v4f *)(vn + d4);
+        else if (col_ok) v4 = *(const v4f *)(vr + (size_t)((lo + key) % a.cap) * a.vpad + d4);
+        const float w = sc[key];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[e] = fmaf(w, v4[e], acc[e]);
+    }
+    *(v4f *)(&ctx[grp][d4]) = acc;
+    __syncthreads();
+    for (int d = tid; d < Dv; d += WD_THREADS) {
+        float o = 0.f;
+#pragma unroll 8
+        for (int g = 0; g < GROUPS; ++g) o += ctx[g][d];
+        if (a.slices > 1) a.part[((size_t)h * a.slices + slice) * (Dv + 2) + d] = o;
+        else a.out[h * Dv + d] = o / l * (a.gate ? gate_w(a.gate[h * Dv + d], a.gate_act) : 1.0f);
+    }
+    if (a.slices > 1 && tid == 0) {
+        float *pp = a.part + ((size_t)h * a.slices + slice) * (Dv + 2) + Dv;
+        pp[0] = m;
+        pp[1] = l;
+    }
+}
+
+// Adds the slices of a head in slice order: one workgroup per head.
+__global__ __launch_bounds__(256) void window_merge_kernel(WindowAttnArgs a) {
+    const int h = blockIdx.x, Dv = a.vdim, pos = *a.pos_dev;
+    const int used = (min(a.window, pos + 1) + WINDOW_SLICE_KEYS - 1) / WINDOW_SLICE_KEYS;
+    const float *part = a.part + (size_t)h * a.slices * (Dv + 2);
+    float m = -INFINITY;
+    for (int s = 0; s < used; ++s) m = fmaxf(m, part[(size_t)s * (Dv + 2) + Dv]);
+    float l = 0.f;
+    for (int s = 0; s < used; ++s) l = fmaf(part[(size_t)s * (Dv + 2) + Dv + 1], expf(part[(size_t)s * (Dv + 2) + Dv] - m), l);
+    for (int d = threadIdx.x; d < Dv; d += 256) {
+        float o = 0.f;
+        for (int s = 0; s < used; ++s) o = fmaf(part[(size_t)s * (Dv + 2) + d], expf(part[(size_t)s * (Dv + 2) + Dv] - m), o);
+        a.out[h * Dv + d] = o / l * (a.gate ? gate_w(a.gate[h * Dv + d], a.gate_act) : 1.0f);
+    }
+}
+
+int launch_window_attn_decode(lumen_ctx *ctx, const WindowAttnArgs &a) {
+    const dim3 grid(a.heads, a.slices), block(WD_THREADS);
+    const int db = a.dim <= 64 ? 1 : a.dim <= 128 ? 2 : 4, lv = a.vdim <= 64 ? 16 : a.vdim <= 128 ? 32 : 64;
+    note_kernel(ctx, "window_decode_kernel<%d, %d>", db, lv);
+#define WD_LAUNCH(DB)                                                                                              \
+    do {                                                                                                           \
+        if (lv == 16) hipLaunchKernelGGL((window_decode_kernel<DB, 16>), grid, block, 0, ctx->stream, a);          \
+        else if (lv == 32) hipLaunchKernelGGL((window_decode_kernel<DB, 32>), grid, block, 0, ctx->stream, a);     \
+        else hipLaunchKernelGGL((window_decode_kernel<DB, 64>), grid, block, 0, ctx->stream, a);                   \
+    } while (0)
+    if (db == 1) WD_LAUNCH(1);
+    else if (db == 2) WD_LAUNCH(2);
+    else WD_LAUNCH(4);
+#undef WD_LAUNCH
+    if (a.slices > 1) hipLaunchKernelGGL(window_merge_kernel, dim3(a.heads), dim3(256), 0, ctx->stream, a);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+// ------------------------------------------------------------------ prompt
+// One workgroup per token: norms over all heads, queries out, key and value into the ring.
+__global__ __launch_bounds__(256) void window_append_kernel(WindowAttnArgs a) {
+    __shared__ float red[2][4];
+    const int t = blockIdx.x, tid = threadIdx.x;
+    const float *q = a.q + (size_t)t * a.stride, *k = a.k + (size_t)t * a.stride, *v = a.v + (size_t)t * a.stride;
+    const int nq = a.heads * a.dim, nk = a.kv_heads * a.dim;
+    float sq = 0.f, sk = 0.f;
+    for (int i = tid; i < nq; i += 256) sq = fmaf(q[i], q[i], sq);
+    for (int i = tid; i < nk; i += 256) sk = fmaf(k[i], k[i], sk);
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if ((tid & 63) == 0) {
+        red[0][tid >> 6] = sq;
+        red[1][tid >> 6] = sk;
+    }
+    __syncthreads();
+    sq = (red[0][0] + red[0][1]) + (red[0][2] + red[0][3]);
+    sk = (red[1][0] + red[1][1]) + (red[1][2] + red[1][3]);
+    const float iq = 1.0f / sqrtf(sq / (float)nq + a.norm_eps), ik = 1.0f / sqrtf(sk / (float)nk + a.norm_eps);
+    for (int i = tid; i < nq; i += 256) a.qn[(size_t)t * nq + i] = a.q_norm_w ? q[i] * iq * a.q_norm_w[i] : q[i];
+    const size_t slot = (size_t)((a.pos + t) % a.cap);
+    for (int i = tid; i < a.kv_heads * a.dpad; i += 256) {
+        const int g = i / a.dpad, d = i % a.dpad;
+        float x = 0.f;
+        if (d < a.dim) {
+            x = k[g * a.dim + d];
+            if (a.k_norm_w) x = x * ik * a.k_norm_w[g * a.dim + d];
+        }
+        a.k_ring[((size_t)g * a.cap + slot) * a.dpad + d] = x;
+    }
+    for (int i = tid; i < a.kv_heads * a.vpad; i += 256) {
+        const int g = i / a.vpad, d = i % a.vpad;
+        a.v_ring[((size_t)g * a.cap + slot) * a.vpad + d] = d < a.vdim ? v[g * a.vdim + d] : 0.f;
+    }
+}
+
+// Online-softmax attention on the f32 matrix instruction.  A workgroup takes 64 queries of one head, a wavefront 16 of
+// them; keys come in tiles of 32 through LDS.  Everything is transposed so that a lane owns one query: S^T = K Q^T (a
+// lane (c, g) ends up with the scores of query c against keys 4 g + r), the weights of step r are then the B operand of
+// O^T += V^T P^T as they stand, and the rescale factor is a scalar of the lane.  NB: 16-channel blocks the registers
+// are laid out for.
+#define WP_Q 64
+#define WP_K 32
+template <int NB>
+__global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, int nd, int nv) {
+    LUMEN_DYNAMIC_LDS(float, lds);
+    const int kld = nd * 16 + 4, vld = nv * 16 + 4;
+    float *ks = lds, *vs = lds + WP_K * kld;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int h = blockIdx.y, hk = h / (a.heads / a.kv_heads), D = a.dim, Dv = a.vdim;
+    const int t0 = blockIdx.x * WP_Q, tw = t0 + wave * 16, t = tw + c;  // first token of the workgroup / wavefront, own token
+    const int last = min(t0 + WP_Q, a.s) - 1;
+    const int i = a.pos + t;  // own position
+    const float r1 = a.r1 ? a.r1[h] : 0.f, r2 = a.r1 ? a.r2[h] : 0.f;
+    const float *kr = a.k_ring + (size_t)hk * a.cap * a.dpad, *vr = a.v_ring + (size_t)hk * a.cap * a.vpad;
+
+    v4f qf[NB], acc[NB];
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+        qf[b] = v4f{0.f, 0.f, 0.f, 0.f};
+        acc[b] = v4f{0.f, 0.f, 0.f, 0.f};
+        if (b < nd && t < a.s) {
+            const float *p = a.qn + ((size_t)t * a.heads + h) * D;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int d = b * 16 + g * 4 + e;
+                if (d < D) qf[b][e] = p[d];
+            }
+        }
+    }
+    float m = -INFINITY, l = 0.f;
+    const int j_first = max(0, a.pos + t0 - a.window + 1), j_last = a.pos + last;
+    const int w_first = max(0, a.pos + tw - a.window + 1), w_last = a.pos + min(tw + 15, a.s - 1);  // of this wavefront
+    for (int j0 = j_first; j0 <= j_last; j0 += WP_K) {
+        __syncthreads();
+        for (int e = tid; e < WP_K * nd * 4; e += 256) {
+            const int row = e / (nd * 4), d = (e % (nd * 4)) * 4;
+            v4f v = {0.f, 0.f, 0.f, 0.f};
+            if (j0 + row <= j_last && d < a.dpad) v = *(const v4f *)(kr + (size_t)((j0 + row) % a.cap) * a.dpad + d);
+            *(v4f *)(ks + row * kld + d) = v;
+        }
+        for (int e = tid; e < WP_K * nv * 4; e += 256) {
+            const int row = e / (nv * 4), d = (e % (nv * 4)) * 4;
+            v4f v = {0.f, 0.f, 0.f, 0.f};
+            if (j0 + row <= j_last && d < a.vpad) v = *(const v4f *)(vr + (size_t)((j0 + row) % a.cap) * a.vpad + d);
+            *(v4f *)(vs + row * vld + d) = v;
+        }
+        __syncthreads();
+        if (tw >= a.s || j0 > w_last || j0 + WP_K - 1 < w_first) continue;  // (uniform in the wavefront)
+        v4f sc[2];
+#pragma unroll
+        for (int u = 0; u < 2; ++u) sc[u] = v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+            if (b < nd) {
+                v4f kf[2];
+#pragma unroll
+                for (int u = 0; u < 2; ++u) kf[u] = *(const v4f *)(ks + (u * 16 + c) * kld + b * 16 + g * 4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+#pragma unroll
+                    for (int u = 0; u < 2; ++u) sc[u] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[u][e], qf[b][e], sc[u], 0, 0, 0);
+            }
+        float mx = m;
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int dist = i - (j0 + u * 16 + g * 4 + r);
+                sc[u][r] = dist >= 0 && dist < a.window ? shaped_score(sc[u][r], a.scale, a.softcap, r1, r2, dist) : -INFINITY;
+                mx = fmaxf(mx, sc[u][r]);
+            }
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        const float base = mx > -INFINITY ? mx : 0.f;  // (a query that has seen nothing yet keeps zero weights)
+        const float f = expf(m - base);
+        m = mx;
+        l *= f;
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                sc[u][r] = expf(sc[u][r] - base);
+                l += sc[u][r];
+            }
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+            if (b < nv) {
+                acc[b] *= f;
+#pragma unroll
+                for (int u = 0; u < 2; ++u)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(vs[(u * 16 + g * 4 + r) * vld + b * 16 + c], sc[u][r], acc[b], 0, 0, 0);
+            }
+    }
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    if (t >= a.s) return;
+    const float inv = 1.0f / l;
+    float *o = a.out + (size_t)t * a.out_stride + (size_t)h * Dv;
+    const float *gp = a.gate ? a.gate + (size_t)t * a.stride + (size_t)h * Dv : nullptr;
+#pragma unroll
+    for (int b = 0; b < NB; ++b)
+        if (b < nv) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int d = b * 16 + g * 4 + r;
+                if (d < Dv) o[d] = acc[b][r] * inv * (gp ? gate_w(gp[d], a.gate_act) : 1.0f);
+            }
+        }
+}
+
+int launch_window_attn_prefill(lumen_ctx *ctx, const WindowAttnArgs &a) {
+    if (a.s <= 0) return LUMEN_OK;
+    hipLaunchKernelGGL(window_append_kernel, dim3(a.s), dim3(256), 0, ctx->stream, a);
+    LUMEN_CHECK_LAUNCH();
+    const int nd = (a.dim + 15) / 16, nv = (a.vdim + 15) / 16;
+    const size_t lds = (size_t)WP_K * ((nd + nv) * 16 + 8) * sizeof(float);
+    const dim3 grid((a.s + WP_Q - 1) / WP_Q, a.heads);
+    const int nb = nd > nv ? nd : nv;
+#define WP_LAUNCH(NB)                                                                                                         \
+    do {                                                                                                                      \
+        if (lds > 64 * 1024)                                                                                                  \
+            HIP_TRY(hipFuncSetAttribute((const void *)window_prefill_kernel<NB>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); \
+        hipLaunchKernelGGL(window_prefill_kernel<NB>, grid, dim3(256), lds, ctx->stream, a, nd, nv);                          \
+    } while (0)
+    if (nb <= 4) WP_LAUNCH(4);
+    else if (nb <= 8) WP_LAUNCH(8);
+    else WP_LAUNCH(16);
+#undef WP_LAUNCH
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+LUMEN_DEFINE_WARM(window_attention)

@@ -42,44 +42,51 @@ class LlamaConfig:
         return dict(self.__dict__)
 
 
-class LlamaModel:
-    """llama.rs:129-280.  Caches live inside the model (init_kv_caches(1) happens at construction);
-    init_kv_caches / reset_kv_caches keep the reference's call shape."""
+class DecoderModel:
+    """What every model of this package offers its callers -- the turn loop, the command line, the trace runner --
+    over the C ABI's model functions, whose names differ in the prefix ABI only: parameters by name, a safetensors
+    file, step / generate_turn / decode_greedy on the one live sequence, reset."""
 
-    def __init__(self, config, ctx=None):
-        if isinstance(config, dict):
-            config = LlamaConfig.from_dict(config)
-        self.config = config
-        self.ctx = ctx or default_ctx()
-        c = _lib.LlamaConfigStruct(
-            config.vocab_size, config.hidden_size, config.intermediate_size, config.num_hidden_layers,
-            config.num_attention_heads, config.num_key_value_heads, config.rms_norm_eps, config.max_seq_len,
-            config.rope_theta, config.head_dim or 0, int(config.qk_norm), int(config.tie_embeddings),
-            _lib.DTYPE_BF16 if config.weight_dtype == "bf16" else _lib.DTYPE_F32)
-        h = C.c_void_p()
-        check(lib.lumen_llama_create(self.ctx.handle, C.byref(c), C.byref(h)))
-        self.handle = h
+    ABI = None           # e.g. "lumen_llama_"
+    vocab_size = None    # attributes of every model
+    handle = None
+
+    def _call(self, name, *args):
+        check(getattr(lib, self.ABI + name)(self.handle, *args))
 
     def __del__(self):
         h, self.handle = getattr(self, "handle", None), None
         if h:
-            lib.lumen_llama_destroy(h)
+            getattr(lib, self.ABI + "destroy")(h)
 
     # -- weights ------------------------------------------------------------
     def set_param(self, name, array):
-        """One tensor by HF name (llama.rs:218-279); f32 arrays or bf16 bits as uint16 (loader.rs:32-68)."""
+        """One tensor by its name; f32 arrays or bf16 bits as uint16 (loader.rs:32-68)."""
         a = np.ascontiguousarray(array)
         dtype = _lib.DTYPE_BF16 if a.dtype == np.uint16 else _lib.DTYPE_F32
         if dtype == _lib.DTYPE_F32 and a.dtype != np.float32:
             a = a.astype(np.float32)
         shape = (C.c_int64 * a.ndim)(*a.shape)
-        check(lib.lumen_llama_set_param(self.handle, name.encode(), a.ctypes.data, dtype, shape, a.ndim))
+        self._call("set_param", name.encode(), a.ctypes.data, dtype, shape, a.ndim)
+
+    def load_params(self, named):
+        for name, a in (named.items() if hasattr(named, "items") else named):
+            self.set_param(name, a)
 
     def load_safetensors(self, path):
         """ModelLoader::load_llama_weights (loader.rs:10-80): returns (tensors set, parameters the file lacks)."""
         loaded, missing = C.c_int(), C.c_int()
-        check(lib.lumen_llama_load_safetensors(self.handle, str(path).encode(), C.byref(loaded), C.byref(missing)))
+        self._call("load_safetensors", str(path).encode(), C.byref(loaded), C.byref(missing))
         return loaded.value, missing.value
+
+    # -- the live sequence ----------------------------------------------------
+    def reset(self):
+        """Gives back what the live sequence holds; the next step starts another one."""
+        self._call("reset")
+
+    def step(self, token_ids, want):
+        """The next tokens of the live sequence; logits [len(want), vocab] at the ascending places `want` among them."""
+        raise NotImplementedError
 
     def generate_turn(self, new_tokens, history=(), temperature=0.8, top_p=0.9, repetition_penalty=1.05,
                       recent_window=96, max_gen=200, seed=0, stop_ids=()):
@@ -91,15 +98,62 @@ class LlamaModel:
         sp = _lib.SamplingStruct(temperature, top_p, repetition_penalty, recent_window, max_gen, seed)
         out = np.zeros(max(max_gen, 1), np.int32)
         n = C.c_int()
-        check(lib.lumen_llama_generate_turn(self.handle, new.ctypes.data, new.size, hist.ctypes.data, hist.size,
-                                            C.byref(sp), stops.ctypes.data, stops.size, out.ctypes.data, out.size,
-                                            C.byref(n)))
+        self._call("generate_turn", new.ctypes.data, new.size, hist.ctypes.data, hist.size, C.byref(sp),
+                   stops.ctypes.data, stops.size, out.ctypes.data, out.size, C.byref(n))
         return out[:n.value].copy()
 
-    def load_params(self, named):
-        for name, a in (named.items() if hasattr(named, "items") else named):
-            self.set_param(name, a)
+    def decode_greedy(self, first_id, n, want_logits=False):
+        """The generation loop of main.rs:340-378 with greedy picks, entirely on the GPU."""
+        ids = np.empty(n, np.int32)
+        logits = np.empty((n, self.vocab_size), np.float32) if want_logits else None
+        self._call("decode_greedy", int(first_id), n, ids.ctypes.data, logits.ctypes.data if want_logits else None)
+        return (ids, logits) if want_logits else ids
 
+    DECODE_MODES = {"eager": _lib.DECODE_EAGER, "graph": _lib.DECODE_GRAPH, "persistent": _lib.DECODE_PERSISTENT}
+
+    def set_decode_mode(self, mode):
+        """'graph' (HIP graph replay per token) or 'eager' (kernel by kernel); 'persistent' is refused
+        (the library holds no such kernel)."""
+        self._call("set_decode_mode", self.DECODE_MODES[mode])
+
+    KERNEL_CLASSES = ()
+
+    def decode_profile(self, first_id, n):
+        """n greedy steps with every launch bracketed by HIP events: {class: (ms_sum, launches)}."""
+        k = len(self.KERNEL_CLASSES)
+        ms = (C.c_double * k)()
+        cnt = (C.c_int * k)()
+        self._call("decode_profile", int(first_id), int(n), ms, cnt, k)
+        return {name: (ms[i], cnt[i]) for i, name in enumerate(self.KERNEL_CLASSES)}
+
+    def decode_bytes(self, length):
+        b = C.c_double()
+        self._call("decode_bytes", int(length), C.byref(b))
+        return b.value
+
+
+class LlamaModel(DecoderModel):
+    """llama.rs:129-280.  Caches live inside the model (init_kv_caches(1) happens at construction);
+    init_kv_caches / reset_kv_caches keep the reference's call shape."""
+
+    ABI = "lumen_llama_"
+
+    def __init__(self, config, ctx=None):
+        if isinstance(config, dict):
+            config = LlamaConfig.from_dict(config)
+        self.config = config
+        self.vocab_size = config.vocab_size
+        self.ctx = ctx or default_ctx()
+        c = _lib.LlamaConfigStruct(
+            config.vocab_size, config.hidden_size, config.intermediate_size, config.num_hidden_layers,
+            config.num_attention_heads, config.num_key_value_heads, config.rms_norm_eps, config.max_seq_len,
+            config.rope_theta, config.head_dim or 0, int(config.qk_norm), int(config.tie_embeddings),
+            _lib.DTYPE_BF16 if config.weight_dtype == "bf16" else _lib.DTYPE_F32)
+        h = C.c_void_p()
+        check(lib.lumen_llama_create(self.ctx.handle, C.byref(c), C.byref(h)))
+        self.handle = h
+
+    # -- weights ------------------------------------------------------------
     def named_parameter_shapes(self):
         return synth.param_shapes(self.config.as_dict())
 
@@ -154,20 +208,15 @@ class LlamaModel:
         check(lib.lumen_llama_forward(self.handle, ids.ctypes.data, s, out.ctypes.data, int(all_rows)))
         return out
 
-    def decode_greedy(self, first_id, n, want_logits=False):
-        """The generation loop of main.rs:340-378 with greedy picks, entirely on the GPU."""
-        ids = np.empty(n, np.int32)
-        logits = np.empty((n, self.config.vocab_size), np.float32) if want_logits else None
-        check(lib.lumen_llama_decode_greedy(self.handle, int(first_id), n, ids.ctypes.data,
-                                            logits.ctypes.data if want_logits else None))
-        return (ids, logits) if want_logits else ids
-
-    DECODE_MODES = {"eager": _lib.DECODE_EAGER, "graph": _lib.DECODE_GRAPH, "persistent": _lib.DECODE_PERSISTENT}
-
-    def set_decode_mode(self, mode):
-        """'graph' (HIP graph replay per token) or 'eager' (kernel by kernel); 'persistent' is refused
-        (the library holds no such kernel)."""
-        check(lib.lumen_llama_set_decode_mode(self.handle, self.DECODE_MODES[mode]))
+    def step(self, token_ids, want):
+        ids = np.ascontiguousarray(token_ids, np.float32).reshape(-1)
+        want = np.asarray(want, np.int64)
+        if want.size == 0:
+            check(lib.lumen_llama_forward(self.handle, ids.ctypes.data, ids.size, None, 0))
+            return np.empty((0, self.vocab_size), np.float32)
+        if want.size == 1 and want[0] == ids.size - 1:
+            return self.forward(ids, all_rows=False)[None]
+        return self.forward(ids, all_rows=True)[want]
 
     def set_handover(self, enable=-1, spin_limit=-1, pre_sleep=-1, poll_delay=-1, poll_gap=-1):
         """The chained launch of short caches: 0 separate launches, 1 attention -> o_proj, 2 q|k|v -> attention ->
@@ -189,19 +238,6 @@ class LlamaModel:
         buf = C.create_string_buffer(160)
         check(lib.lumen_llama_profile_kernel_name(self.handle, self.KERNEL_CLASSES.index(kernel_class), buf, 160))
         return buf.value.decode()
-
-    def decode_profile(self, first_id, n):
-        """n greedy steps with every launch bracketed by HIP events: {class: (ms_sum, launches)}."""
-        k = len(self.KERNEL_CLASSES)
-        ms = (C.c_double * k)()
-        cnt = (C.c_int * k)()
-        check(lib.lumen_llama_decode_profile(self.handle, int(first_id), int(n), ms, cnt, k))
-        return {name: (ms[i], cnt[i]) for i, name in enumerate(self.KERNEL_CLASSES)}
-
-    def decode_bytes(self, length):
-        b = C.c_double()
-        check(lib.lumen_llama_decode_bytes(self.handle, int(length), C.byref(b)))
-        return b.value
 
 
 class LlamaMLP:

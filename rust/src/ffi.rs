@@ -57,6 +57,9 @@ pub const LUMEN_GEMV_EPI_ROPE_QKV: c_int = 4;
 pub const LUMEN_DECODE_EAGER: c_int = 0;
 pub const LUMEN_DECODE_GRAPH: c_int = 1;
 pub const LUMEN_DECODE_PERSISTENT: c_int = 2;
+pub const LUMEN_MIXER_WINDOW_ATTENTION: c_int = 0;
+pub const LUMEN_MIXER_WKV: c_int = 1;
+pub const LUMEN_MIXER_CHANNEL_DELTA: c_int = 2;
 
 extern "C" {
     pub fn lumen_last_error() -> *const c_char;
@@ -133,6 +136,29 @@ extern "C" {
     pub fn lumen_decoder_layer_create(ctx: *mut lumen_ctx, cfg: *const lumen_llama_config, out: *mut *mut lumen_decoder_layer) -> c_int;
     pub fn lumen_decoder_layer_destroy(layer: *mut lumen_decoder_layer) -> c_int;
     pub fn lumen_decoder_layer_decode_f32(layer: *mut lumen_decoder_layer, cache: *mut lumen_kv_cache, wqkv_dev: *const c_void, wo_dev: *const c_void, wgu_dev: *const c_void, wdown_dev: *const c_void, input_norm_dev: *const c_float, post_norm_dev: *const c_float, q_norm_dev: *const c_float, k_norm_dev: *const c_float, x_dev: *const c_float, y_dev: *mut c_float) -> c_int;
+    pub fn lumen_hybrid_create(ctx: *mut lumen_ctx, cfg: *const lumen_hybrid_config, layers: *const lumen_hybrid_layer, out: *mut *mut lumen_hybrid) -> c_int;
+    pub fn lumen_hybrid_destroy(model: *mut lumen_hybrid) -> c_int;
+    pub fn lumen_hybrid_num_params(model: *const lumen_hybrid, n_out: *mut c_int) -> c_int;
+    pub fn lumen_hybrid_param_info(model: *const lumen_hybrid, index: c_int, name: *mut c_char, name_len: c_int, shape_out: *mut i64, ndim_out: *mut c_int) -> c_int;
+    pub fn lumen_hybrid_set_param(model: *mut lumen_hybrid, name: *const c_char, data_host: *const c_void, dtype: c_int, shape: *const i64, ndim: c_int) -> c_int;
+    pub fn lumen_hybrid_load_safetensors(model: *mut lumen_hybrid, path: *const c_char, n_loaded_out: *mut c_int, n_missing_out: *mut c_int) -> c_int;
+    pub fn lumen_hybrid_forward(model: *mut lumen_hybrid, ids_host: *const i32, s: c_int, want_host: *const i32, n_want: c_int, logits_host: *mut c_float, residual_host: *mut c_float) -> c_int;
+    pub fn lumen_hybrid_decode_greedy(model: *mut lumen_hybrid, first_id: c_int, n: c_int, ids_out_host: *mut i32, logits_out_host: *mut c_float) -> c_int;
+    pub fn lumen_hybrid_generate_turn(model: *mut lumen_hybrid, new_tokens: *const i32, n_new: c_int, history: *const i32, n_history: c_int, sampling: *const lumen_sampling, stop_ids: *const i32, n_stop: c_int, out_ids: *mut i32, out_cap: c_int, n_out: *mut c_int) -> c_int;
+    pub fn lumen_hybrid_decode_profile(model: *mut lumen_hybrid, first_id: c_int, n: c_int, ms_sum_out: *mut f64, count_out: *mut c_int, n_classes: c_int) -> c_int;
+    pub fn lumen_hybrid_set_decode_mode(model: *mut lumen_hybrid, mode: c_int) -> c_int;
+    pub fn lumen_hybrid_reset(model: *mut lumen_hybrid) -> c_int;
+    pub fn lumen_hybrid_len(model: *const lumen_hybrid, len_out: *mut c_int) -> c_int;
+    pub fn lumen_hybrid_num_runs(model: *const lumen_hybrid, n_out: *mut c_int) -> c_int;
+    pub fn lumen_hybrid_decode_bytes(model: *const lumen_hybrid, len: c_int, bytes_out: *mut f64) -> c_int;
+    pub fn lumen_polynorm_f32(ctx: *mut lumen_ctx, z_dev: *const c_float, coef_dev: *const c_float, out_dev: *mut c_float, rows: c_int, dim: c_int, eps: c_float) -> c_int;
+    pub fn lumen_token_shift_f32(ctx: *mut lumen_ctx, h_dev: *const c_float, mu_dev: *const c_float, prev_dev: *const c_float, next_dev: *mut c_float, mixes_dev: *mut c_float, n: c_int, s: c_int, dim: c_int) -> c_int;
+    pub fn lumen_recurrence_state_rows(dim: c_int, rows_out: *mut c_int) -> c_int;
+    pub fn lumen_wkv_f32(ctx: *mut lumen_ctx, r_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, z_dev: *const c_float, bias_dev: *const c_float, u_dev: *const c_float, state_dev: *mut c_float, out_dev: *mut c_float, s: c_int, heads: c_int, dim: c_int) -> c_int;
+    pub fn lumen_channel_delta_f32(ctx: *mut lumen_ctx, q_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, z_dev: *const c_float, b_dev: *const c_float, bias_dev: *const c_float, a_log_dev: *const c_float, state_dev: *mut c_float, out_dev: *mut c_float, s: c_int, heads: c_int, kv_heads: c_int, dim: c_int, vdim: c_int) -> c_int;
+    pub fn lumen_conv_unit_f32(ctx: *mut lumen_ctx, qkv_dev: *const c_float, taps_dev: *const c_float, prev_dev: *const c_float, next_dev: *mut c_float, q_dev: *mut c_float, k_dev: *mut c_float, v_dev: *mut c_float, s: c_int, taps: c_int, heads: c_int, kv_heads: c_int, dim: c_int, vdim: c_int, unit_eps: c_float, q_scale: c_float) -> c_int;
+    pub fn lumen_head_norm_gate_f32(ctx: *mut lumen_ctx, o_dev: *mut c_float, gain_dev: *const c_float, gain_shared: c_int, gate_dev: *const c_float, gate_act: c_int, rows: c_int, heads: c_int, vdim: c_int, eps: c_float) -> c_int;
+    pub fn lumen_window_attn_f32(ctx: *mut lumen_ctx, q_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, gate_dev: *const c_float, q_norm_dev: *const c_float, k_norm_dev: *const c_float, r1_dev: *const c_float, r2_dev: *const c_float, k_ring_dev: *mut c_float, v_ring_dev: *mut c_float, cap: c_int, out_dev: *mut c_float, s: c_int, pos: c_int, heads: c_int, kv_heads: c_int, dim: c_int, vdim: c_int, window: c_int, scale: c_float, softcap: c_float, norm_eps: c_float) -> c_int;
 }
 
 /// status -> panic with the library's message: the reference's own error behaviour (Cargo.toml: panic = "abort")
