@@ -54,11 +54,17 @@ def main():
     ap.add_argument("--resident", action="store_true",
                     help="--workload gemv: every launch reads the SAME copy of W (what the caches hold counts: the "
                          "figure is no longer HBM bandwidth); default: >= 1.2 GB of copies in rotation")
-    ap.add_argument("--workload", choices=["decode", "gemv", "gemm", "prefill", "copy"], default="decode",
+    ap.add_argument("--workload", choices=["decode", "gemv", "gemm", "prefill", "copy", "hybrid"], default="decode",
                     help="decode: the headline batch-1 decode benchmark; gemv: the isolated M=1 GEMV shapes; "
                          "gemm: the prompt-pass GEMM shapes against the fp32 matrix-core peak; prefill: one long "
                          "prompt pass (3968 tokens, TinyLlama shape with a 4096-row cache); "
-                         "copy: a plain 1 GiB copy kernel (calibrates the FETCH_SIZE / WRITE_SIZE counters)")
+                         "copy: a plain 1 GiB copy kernel (calibrates the FETCH_SIZE / WRITE_SIZE counters); "
+                         "hybrid: prompt passes and decode of the layered hybrid decoder (Pinavik) beside a Llama of "
+                         "equal size (--hybrid-width, --hybrid-dtype)")
+    ap.add_argument("--hybrid-width", type=int, default=2048, help="--workload hybrid: width of both models (a multiple of 256)")
+    ap.add_argument("--hybrid-dtype", choices=["bf16", "f32"], default="bf16", help="--workload hybrid: storage of the matrices")
+    ap.add_argument("--hybrid-only", choices=["hybrid", "llama"], default=None,
+                    help="--workload hybrid: one of the two models (for a kernel trace)")
     args = ap.parse_args()
     if args.gpus != 1:
         sys.exit("bench.py: this build runs the batch-1 decode path on ONE GPU; --gpus %d is not supported "
@@ -72,6 +78,8 @@ def main():
         return gemm_microbench(args)
     if args.workload == "prefill":
         return prefill_bench(args)
+    if args.workload == "hybrid":
+        return hybrid_bench(args)
 
     import numpy as np
 
@@ -439,6 +447,94 @@ def prefill_bench(args):
                                   "random ids into an empty cache of %d rows" % (S, cfg["max_seq_len"])}}
     out.update(prefill_report(cfg, S, ms))
     out["passes_ms"] = [round(x, 3) for x in passes]
+    print(json.dumps(out))
+
+
+HYBRID_PROMPTS = (16, 128, 512, 2048)
+
+
+def hybrid_bench(args):
+    """The layered hybrid decoder beside a Llama of equal width, layer runs and feed-forward volume: prompt passes of
+    several lengths (mean of the last two of five, last-row logits), then decode after the longest prompt, random
+    weights.  Decode kernels: event-bracketed averages; products also as a share of the HBM bandwidth."""
+    import numpy as np
+
+    from lumen_amd import synth
+    from lumen_amd.hybrid import HybridModel
+    from lumen_amd.models import LlamaModel
+
+    W, dt = args.hybrid_width, args.hybrid_dtype
+    steps, warmup = args.steps, args.warmup
+    rows = {}
+    for name in ("hybrid", "llama"):
+        if args.hybrid_only not in (None, name):
+            continue
+        t0 = time.time()
+        if name == "hybrid":
+            cfg = synth.hybrid_shape(W, dt)
+            model = HybridModel(cfg)
+            shapes = model.named_parameter_shapes()
+            one = lambda n: synth.hybrid_param(n, shapes[n], 0)  # noqa: E731
+            length = lambda: model.length  # noqa: E731
+            vocab = cfg.vocab_size
+        else:
+            cfg = synth.llama_beside(W, dt)
+            model = LlamaModel(cfg)
+            shapes = model.named_parameter_shapes()
+            one = lambda n: synth.make_param(n, shapes[n], 0)  # noqa: E731
+            length = lambda: model.kv_len  # noqa: E731
+            vocab = cfg["vocab_size"]
+        from concurrent.futures import ThreadPoolExecutor
+        with ThreadPoolExecutor(8) as pool:
+            for n, a in zip(shapes, pool.map(one, shapes)):
+                model.set_param(n, a)
+        model.set_decode_mode(args.mode)
+        ctx = model.ctx
+        prompts = {}
+        for S in HYBRID_PROMPTS:
+            ids = synth.make_tokens(S, vocab, seed=0)
+            ms = []
+            for _ in range(5):
+                model.reset()
+                ctx.synchronize()
+                ctx.timer_start()
+                last = model.step(ids, [S - 1])[0]
+                ms.append(ctx.timer_stop())
+            if not np.isfinite(last).all():
+                raise SystemExit("bench: logits that are not finite")
+            prompts[str(S)] = {"ms": round(0.5 * (ms[-1] + ms[-2]), 3), "tokens_per_s": round(2e3 * S / (ms[-1] + ms[-2]), 1)}
+        tok = int(np.argmax(last))
+        if warmup:
+            tok = int(model.decode_greedy(tok, warmup)[-1])
+        ctx.synchronize()
+        len0 = length()
+        ctx.timer_start()
+        picks = model.decode_greedy(tok, steps)
+        ms = ctx.timer_stop() / steps
+        nbytes = model.decode_bytes(len0 + steps // 2)
+        prof_steps = min(steps, 32)
+        model.set_decode_mode("eager")
+        ctx.timer_start()
+        model.decode_greedy(int(picks[-1]), prof_steps)
+        eager = ctx.timer_stop()
+        prof = model.decode_profile(int(picks[-1]), prof_steps)
+        launches = sum(n for _, n in prof.values())
+        over = max(0.0, (sum(t for t, _ in prof.values()) - eager) / max(launches, 1))
+        rows[name] = {"prompt": prompts,
+                      "decode": {"ms_per_token": round(ms, 4), "tokens_per_s": round(1e3 / ms, 1), "bytes_per_token": nbytes,
+                                 "frac_of_8TBps": round(nbytes / ms / 1e6 / HBM_PEAK_GBS, 4), "kv_len": [len0, len0 + steps]},
+                      "decode_kernels": {k: {"avg_us": round(1e3 * (t / n - over), 2), "per_token": n // prof_steps}
+                                         for k, (t, n) in prof.items() if n},
+                      "setup_s": round(time.time() - t0, 1)}
+        del model
+    out = {"metric": "hybrid decoder tokens/s", "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": warmup,
+           "dtype": "%s weights, f32 activations" % dt, "data": "synthetic", "higher_is_better": True,
+           "config": {"workload": "layered hybrid decoder (attention over 1024 tokens, channel_delta, wkv, channel_delta) x 3, the "
+                                  "middle group twice = 16 layer runs, feed-forward 4 x width; Llama of 16 layers beside it; "
+                                  "width %d, vocabulary 32000, random weights" % W}}
+    out.update(rows)
+    if "hybrid" in rows:
+        out["value"] = rows["hybrid"]["decode"]["tokens_per_s"]
     print(json.dumps(out))
 
 

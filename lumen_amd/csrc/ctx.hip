@@ -81,6 +81,7 @@ extern "C" int lumen_ctx_destroy(lumen_ctx *ctx) {
     if (ctx->bounce) hipHostFree(ctx->bounce);
     if (ctx->err_host) hipHostFree(ctx->err_host);
     if (ctx->gemm_ws) hipFree(ctx->gemm_ws);
+    if (ctx->mixer_ws) hipFree(ctx->mixer_ws);
     hipEventDestroy(ctx->ev0);
     hipEventDestroy(ctx->ev1);
     hipStreamDestroy(ctx->own_stream);

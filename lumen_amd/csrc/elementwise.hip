@@ -177,9 +177,76 @@ __global__ __launch_bounds__(256) void polynorm_kernel(const float *z, const flo
     }
 }
 
+// The same for 16-byte aligned rows of up to 4096 VPT elements: read once, kept in registers between the two passes.
+template <int VPT>
+__global__ __launch_bounds__(1024) void polynorm_vec_kernel(const float *z, const float *__restrict__ coef, float *out, int dim,
+                                                            int stride, float eps) {
+    __shared__ float red[3][16];
+    const float *zr = z + (size_t)blockIdx.x * stride;
+    float *o = out + (size_t)blockIdx.x * stride;
+    const int tid = threadIdx.x, nt = blockDim.x, nw = nt >> 6;
+    v4f v[VPT];
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const int k = (tid + i * nt) * 4;
+        v[i] = v4f{0.f, 0.f, 0.f, 0.f};
+        if (k < stride) v[i] = *(const v4f *)(zr + k);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            if (k + e >= dim) v[i][e] = 0.f;
+    }
+    float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const float q = v[i][e] * v[i][e], q2 = q * q;
+            s1 += q;
+            s2 += q2;
+            s3 = fmaf(q2, q, s3);
+        }
+    s1 = wave_sum(s1);
+    s2 = wave_sum(s2);
+    s3 = wave_sum(s3);
+    if ((tid & 63) == 0) {
+        red[0][tid >> 6] = s1;
+        red[1][tid >> 6] = s2;
+        red[2][tid >> 6] = s3;
+    }
+    __syncthreads();
+    s1 = s2 = s3 = 0.f;
+    for (int w = 0; w < nw; ++w) {
+        s1 += red[0][w];
+        s2 += red[1][w];
+        s3 += red[2][w];
+    }
+    const float n = (float)dim;
+    const float a1 = coef[0] / sqrtf(s1 / n + eps), a2 = coef[1] / sqrtf(s2 / n + eps), a3 = coef[2] / sqrtf(s3 / n + eps), c3 = coef[3];
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+        const int k = (tid + i * nt) * 4;
+        if (k < stride) {
+            v4f r;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) r[e] = k + e < dim ? fmaf(fmaf(fmaf(a3, v[i][e], a2), v[i][e], a1), v[i][e], c3) : 0.f;
+            *(v4f *)(o + k) = r;
+        }
+    }
+}
+
 int launch_polynorm(lumen_ctx *ctx, const float *z, const float *coef, float *out, int rows, int dim, int stride, float eps) {
     if (rows <= 0 || dim <= 0) return LUMEN_OK;
-    hipLaunchKernelGGL(polynorm_kernel, dim3(rows), dim3(256), 0, ctx->stream, z, coef, out, dim, stride, eps);
+    if (stride % 4 == 0 && stride <= 16384 && (((uintptr_t)z | (uintptr_t)out) & 15) == 0) {
+        const int pieces = stride / 4, threads = pieces <= 256 ? 256 : pieces <= 512 ? 512 : 1024;
+        if (pieces <= threads)
+            hipLaunchKernelGGL(polynorm_vec_kernel<1>, dim3(rows), dim3(threads), 0, ctx->stream, z, coef, out, dim, stride, eps);
+        else if (pieces <= 2 * threads)
+            hipLaunchKernelGGL(polynorm_vec_kernel<2>, dim3(rows), dim3(threads), 0, ctx->stream, z, coef, out, dim, stride, eps);
+        else
+            hipLaunchKernelGGL(polynorm_vec_kernel<4>, dim3(rows), dim3(threads), 0, ctx->stream, z, coef, out, dim, stride, eps);
+    } else {
+        hipLaunchKernelGGL(polynorm_kernel, dim3(rows), dim3(256), 0, ctx->stream, z, coef, out, dim, stride, eps);
+    }
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
 }
@@ -196,10 +263,33 @@ __global__ __launch_bounds__(256) void token_shift_kernel(const float *__restric
     }
 }
 
+// 16-byte pieces: workgroup (token, block of 1024 channels), all mixes' factors requested together
+__global__ __launch_bounds__(256) void token_shift_vec_kernel(const float *__restrict__ h, const float *__restrict__ mu,
+                                                              const float *__restrict__ prev, float *__restrict__ next,
+                                                              float *__restrict__ mixes, int n, int s, int dim) {
+    const int t = blockIdx.x, i = ((int)blockIdx.y * 256 + (int)threadIdx.x) * 4;
+    if (i >= dim) return;
+    const float *cur = h + (size_t)t * dim, *bef = t ? cur - dim : prev;
+    const v4f c = *(const v4f *)(cur + i), d = *(const v4f *)(bef + i) - c;
+#pragma unroll 5
+    for (int m = 0; m < n; ++m) {
+        const v4f f = *(const v4f *)(mu + (size_t)m * dim + i);
+        v4f r;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) r[e] = fmaf(d[e], f[e], c[e]);
+        *(v4f *)(mixes + ((size_t)m * s + t) * dim + i) = r;
+    }
+    if (t == s - 1) *(v4f *)(next + i) = c;
+}
+
 int launch_token_shift(lumen_ctx *ctx, const float *h, const float *mu, const float *prev, float *next, float *mixes, int n,
                        int s, int dim) {
     if (s <= 0 || dim <= 0) return LUMEN_OK;
-    hipLaunchKernelGGL(token_shift_kernel, dim3(s), dim3(256), 0, ctx->stream, h, mu, prev, next, mixes, n, s, dim);
+    const bool vec = dim % 4 == 0 && (((uintptr_t)h | (uintptr_t)mu | (uintptr_t)prev | (uintptr_t)next | (uintptr_t)mixes) & 15) == 0;
+    if (vec)
+        hipLaunchKernelGGL(token_shift_vec_kernel, dim3(s, (dim + 1023) / 1024), dim3(256), 0, ctx->stream, h, mu, prev, next, mixes, n, s, dim);
+    else
+        hipLaunchKernelGGL(token_shift_kernel, dim3(s), dim3(256), 0, ctx->stream, h, mu, prev, next, mixes, n, s, dim);
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
 }

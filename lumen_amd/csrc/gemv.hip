@@ -13,6 +13,8 @@
 #include "wave_reduce.h"
 #include "stage_times.h"
 
+#include <algorithm>
+
 typedef float v4f __attribute__((ext_vector_type(4)));
 typedef unsigned int v4u __attribute__((ext_vector_type(4)));
 
@@ -286,7 +288,8 @@ typedef float v2f __attribute__((ext_vector_type(2)));
 __device__ __forceinline__ void stage_attn_fold(float *xs, const GemvArgs &a, int K, int kpad, int nwaves) {
     const int tid = threadIdx.x, nthreads = nwaves * 64;
     const int D = a.attn_d, S = a.attn_nslices, stride = D + 2;
-    const int rows = *a.attn_pos + 1;
+    int rows = *a.attn_pos + 1;
+    if (a.attn_window > 0) rows = min(rows, a.attn_window);
     int nact = 1;
     if (rows > a.attn_short_rows) nact = min(S, (rows + a.attn_trip - 1) / a.attn_trip);
     for (int k = tid * 4; k < kpad; k += nthreads * 4) {
@@ -320,6 +323,11 @@ __device__ __forceinline__ void stage_attn_fold(float *xs, const GemvArgs &a, in
             }
             const float inv = 1.0f / (L + 1e-9f);
             v.x *= inv; v.y *= inv; v.z *= inv; v.w *= inv;
+            if (a.attn_gate) {
+                const v4f gz = *(const v4f *)(a.attn_gate + k);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] *= 1.0f / (1.0f + expf(-gz[e]));
+            }
         }
         *(v4f *)(xs + k) = v;
     }
@@ -787,7 +795,7 @@ int launch_gemv(lumen_ctx *ctx, const GemvArgs &a) {
     }
     if (a.pro == PRO_ATTN_FOLD) {
         if (a.epi != EPI_RESIDUAL || p.R != 1 || !a.attn_part || !a.attn_pos || a.attn_d <= 0 || a.attn_d % 4 ||
-            a.K % a.attn_d || a.attn_nslices < 1 || a.attn_nslices > GEMV_FOLD_MAX_SLICES)
+            a.K % a.attn_d || ((uintptr_t)a.attn_gate & 15) || a.attn_nslices < 1 || a.attn_nslices > GEMV_FOLD_MAX_SLICES)
             LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over attention partials: one row per unit, residual epilogue, at most %d slices (got %d)",
                        GEMV_FOLD_MAX_SLICES, a.attn_nslices);
     }
@@ -807,7 +815,18 @@ int launch_gemv(lumen_ctx *ctx, const GemvArgs &a) {
             LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "arg-max epilogue: %d rows (at most %d)", a.N, (1 << 24) - 1);
         if (a.spin_limit > HANDOVER_MAX_SPINS) LUMEN_FAIL(LUMEN_ERR_INVALID, "arg-max epilogue: poll limit %u", a.spin_limit);
     }
-    const int threads = p.threads, blocks = p.blocks;
+    int blocks = p.blocks;
+    if (a.pro == PRO_SHIFT) {
+        // one round of workgroups over all the products: each stages a normalised, mixed x of its own first, so more,
+        // shorter workgroups would spend the time there
+        const int waves = p.threads / 64, nunits = (a.N + p.R - 1) / p.R;
+        const int cap = std::max(1, ctx->num_cus * std::max(1, 16 / waves) / a.shift_segs);
+        if (blocks > cap) {
+            const int per_wave = (nunits + cap * waves - 1) / (cap * waves);
+            blocks = (nunits + waves * per_wave - 1) / (waves * per_wave);
+        }
+    }
+    const int threads = p.threads;
     const size_t lds = p.lds;
     dim3 grid(blocks);
 #define LAUNCH_GEMV_K(BF, RR, KAV)                                                       \

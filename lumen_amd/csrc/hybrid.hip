@@ -47,6 +47,7 @@ struct Layer {
     float *mu = nullptr, *bias = nullptr, *u = nullptr, *a_log = nullptr, *taps = nullptr, *gain = nullptr;
     int lo_rank = 0, hi_rank = 0;        // rounded
     int window = 0, cap = 0, slices = 1;
+    bool fold = false;                   // the output projection folds the slices of a decode step
     int channels() const { return 2 * c.kv_heads * c.dim + c.heads * c.vdim; }
 };
 
@@ -160,7 +161,7 @@ static int check_layer(const lumen_hybrid_layer &c, int i) {
     }
     if (c.rank_lo > MIX_MAX_RANK || c.rank_hi > MIX_MAX_RANK)
         LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: ranks above %d", i, MIX_MAX_RANK);
-    if (c.ff > 16384 || c.heads * c.vdim > 16384)
+    if (c.ff > 16384 || c.heads * c.vdim > 16384 || c.heads * c.dim > 16384)
         LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: inner sizes above 16384 do not fit the GEMV's LDS stage", i);
     return LUMEN_OK;
 }
@@ -200,6 +201,10 @@ static int create_layer(lumen_hybrid *m, Layer &L, int i) {
         L.window = c.window > 0 ? std::min(c.window, max_seq) : max_seq;
         L.cap = std::min(max_seq, L.window - 1 + m->cfg.max_chunk);
         L.slices = window_attn_slices(L.window);
+        // (every workgroup of the output projection then reads every slice's state: it pays while that stays tens of MB)
+        const size_t fold_bytes = (size_t)gemv_grid(m->ctx, m->W, L.od, m->bf16, EPI_RESIDUAL, nullptr) * L.od * GEMV_FOLD_MAX_SLICES * sizeof(float);
+        L.fold = L.slices > 1 && L.slices <= GEMV_FOLD_MAX_SLICES && Dv % 4 == 0 && L.od == H * Dv && m->W < 8192 &&
+                 fold_bytes <= ((size_t)64 << 20);
     } else if (c.mixer == LUMEN_MIXER_WKV) {
         L.seg = pad8(H * D);
         L.seg_last = L.lo_rank;
@@ -551,7 +556,7 @@ static int enqueue_decode_step(lumen_hybrid *m, const Tap *tap = nullptr) {
         }
         if (L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION) {
             WindowAttnArgs a = attn_args(m, L, r, m->proj, L.n_proj);
-            a.out = m->mixed; a.pos_dev = m->d_pos; a.part = m->part;
+            a.out = m->mixed; a.pos_dev = m->d_pos; a.part = m->part; a.leave_slices = L.fold;
             LUMEN_TRY(timed(m, HC_ATTN, do_attn, &a));
         } else {
             const bool wkv = L.c.mixer == LUMEN_MIXER_WKV;
@@ -570,6 +575,10 @@ static int enqueue_decode_step(lumen_hybrid *m, const Tap *tap = nullptr) {
         {
             GemvArgs g = gemv_args(m, L.w_o, W, L.od, m->mixed, out());
             gemv_residual(g, cur, c.residual_mult);
+            if (L.fold) {
+                g.pro = PRO_ATTN_FOLD; g.attn_part = m->part; g.attn_pos = m->d_pos; g.attn_nslices = L.slices; g.attn_d = L.c.vdim;
+                g.attn_trip = WINDOW_SLICE_KEYS; g.attn_short_rows = 0; g.attn_window = L.window; g.attn_gate = m->proj + L.off_g;
+            }
             LUMEN_TRY(timed(m, HC_OUT, do_gemv, &g));
             cur = g.y;
         }

@@ -56,6 +56,8 @@ struct lumen_ctx {
     int *err_host = nullptr;
     float *gemm_ws = nullptr;      // split-K workspace of the prefill GEMM, grown on demand
     size_t gemm_ws_bytes = 0;
+    float *mixer_ws = nullptr;     // per-chunk operands of the recurrences, grown on demand
+    size_t mixer_ws_bytes = 0;
     // this device's address of the fixed scratch array behind lumen_attn_decode_static_f32
     unsigned char *attn_static = nullptr;
     size_t attn_static_bytes = 0;
@@ -146,6 +148,8 @@ struct GemvArgs {
     const float *attn_part;
     const int *attn_pos;
     int attn_nslices, attn_d, attn_trip, attn_short_rows;
+    int attn_window;         // > 0: at most that many rows are in use (a sliding window)
+    const float *attn_gate;  // [K] or null: x is multiplied by the sigmoid of it
 };
 #define GEMV_FOLD_MAX_SLICES 16  // PRO_ATTN_FOLD reads this many slice states per element, whatever the count in use
 int launch_gemv(lumen_ctx *ctx, const GemvArgs &a);

@@ -44,10 +44,11 @@ struct WindowAttnArgs {
     int pos;                         // prompt: position of the first of s tokens
     int s;
     float *qn;                       // prompt: normalised queries [s][heads * dim], may be q's own rows when stride fits
-    float *part;                     // decode over more than one slice: states [heads][slices][vdim + 2]
+    float *part;                     // decode over more than one slice: states [heads][slices][vdim + 2] (ctx, max in log2 units, sum)
     int slices;
+    int leave_slices;                // ... for the output projection to fold (PRO_ATTN_FOLD), gate included: out is not written
 };
-#define WINDOW_SLICE_KEYS 512
+#define WINDOW_SLICE_KEYS 256
 int window_attn_slices(int window);                       // slices of a decode step over that window
 int launch_window_attn_decode(lumen_ctx *ctx, const WindowAttnArgs &a);   // one token: norm, append, attend, gate
 int launch_window_attn_prefill(lumen_ctx *ctx, const WindowAttnArgs &a);  // s tokens; cap >= window - 1 + s

@@ -69,7 +69,7 @@ __device__ __forceinline__ float column_step(float (&S)[KR], const float (&q)[KR
     return row16_sum(o);
 }
 
-// ------------------------------------------------------------------ prompt
+// ---------------------------------------------------------- prompt, token by token
 #define REC_TOK 16  // tokens staged at a time
 #define REC_COLS 16 // columns of a workgroup: 4 wavefronts x 4 rows of lanes
 
@@ -140,10 +140,257 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceArgs a) {
     if (live) store_kr<KR>(Sg, S);
 }
 
+// ---------------------------------------------------------- prompt, 16 tokens at a time
+// Over a chunk of 16 tokens both recurrences are matrix products with the state S the chunk starts from.  With G_t the
+// product of the decays up to token t (WKV reads the state before its own token: up to t - 1), and G_t / G_s always
+// the product of the decays in between -- formed by multiplying, never by dividing, so that strong decays stay exact --
+//   delta: U = T (V - K~ S),  T = (I + diag(b) tril(A, -1))^-1 diag(b),  A_ts = sum_d k_t k_s G_t / G_s,  K~_t = G_t k_t
+//   WKV:   U = V
+//   O = Q~ S + B U,  B_ts = sum_d q_t k_s G_t / G_s  (WKV: s < t, and sum_d q u k on the diagonal),  Q~_t = G_t q_t
+//   S <- diag(G_16) S + K^^T U,  K^_s = (G_16 / G_s) k_s.
+// K~, Q~, K^, T, B and G_16 do not depend on S: recurrence_chunk_prep_kernel makes them for all chunks in parallel;
+// recurrence_chunk_kernel then walks the chunks of a head with S in the accumulators of the f32 matrix instruction.
+#define REC_CHUNK 16
+static __host__ __device__ __forceinline__ size_t rec_ws_floats(int dp) { return (size_t)49 * dp + 512; }
+struct ChunkWs {  // one chunk of one head
+    float *kt, *qt, *kh, *gc, *t, *b;  // [16][dp], [16][dp], [dp][16], [dp], [16][16], [16][16]
+    __device__ ChunkWs(float *base, int dp) : kt(base), qt(base + 16 * dp), kh(base + 32 * dp), gc(base + 48 * dp), t(base + 49 * dp), b(base + 49 * dp + 256) {}
+};
+
+template <int KIND, int KR>
+__global__ __launch_bounds__(256) void recurrence_chunk_prep_kernel(RecurrenceArgs a, float *ws_base) {
+    constexpr int DP = 16 * KR;
+    __shared__ __align__(16) float qs[REC_CHUNK][DP], ks[REC_CHUNK][DP], gs[REC_CHUNK][DP];
+    __shared__ float As[REC_CHUNK][REC_CHUNK + 1], bs[REC_CHUNK];
+    const int tid = threadIdx.x, s = tid >> 4, i16 = tid & 15;
+    const int h = blockIdx.y, hk = h / a.rep, D = a.dim, t0 = blockIdx.x * REC_CHUNK;
+    const bool live = t0 + s < a.s;
+    const float decay_a = KIND == REC_DELTA ? expf(a.a_log[h]) : 0.f;
+    float q[KR], k[KR], g[KR], uk[KR];
+#pragma unroll
+    for (int i = 0; i < KR; ++i) {
+        const int c = i16 * KR + i;
+        const bool ok = live && c < D;
+        const size_t t = (size_t)(t0 + s);
+        q[i] = ok ? a.q[t * a.q_stride + hk * D + c] : 0.f;
+        k[i] = ok ? a.k[t * a.k_stride + hk * D + c] : 0.f;
+        g[i] = ok ? decay_r<KIND>(a.z[t * a.z_stride + h * D + c], a.bias[h * D + c], decay_a) : 1.f;  // (a missing token changes nothing)
+        uk[i] = KIND == REC_WKV && ok ? a.u[h * D + c] * k[i] : 0.f;
+    }
+    store_kr<KR>(&qs[s][i16 * KR], q);
+    store_kr<KR>(&ks[s][i16 * KR], k);
+    store_kr<KR>(&gs[s][i16 * KR], g);
+    if (KIND == REC_DELTA && tid < REC_CHUNK) bs[tid] = t0 + tid < a.s ? sigmoid_r(a.b[(size_t)(t0 + tid) * a.b_stride + h]) : 0.f;
+    __syncthreads();
+    ChunkWs w(ws_base + ((size_t)h * gridDim.x + blockIdx.x) * rec_ws_floats(DP), DP);
+    // decays up to this token, and the rows that meet the chunk's first state
+    float G[KR], kr[KR];
+#pragma unroll
+    for (int i = 0; i < KR; ++i) {
+        G[i] = 1.f;
+        kr[i] = k[i];
+    }
+    for (int t = 0; t < REC_CHUNK; ++t) {
+        float gt[KR], qt[KR];
+        load_kr<KR>(gt, &gs[t][i16 * KR]);
+        load_kr<KR>(qt, &qs[t][i16 * KR]);
+        const bool before = t < s, after = t > s;
+        float da = 0.f, db = 0.f;
+#pragma unroll
+        for (int i = 0; i < KR; ++i) {
+            G[i] *= before ? gt[i] : 1.f;
+            if (KIND == REC_DELTA) kr[i] *= after ? gt[i] : 1.f;
+            db = fmaf(KIND == REC_WKV && !after ? uk[i] : kr[i], qt[i], db);
+        }
+        if (KIND == REC_DELTA) {
+            float kt[KR];
+            load_kr<KR>(kt, &ks[t][i16 * KR]);
+#pragma unroll
+            for (int i = 0; i < KR; ++i) da = fmaf(kr[i], kt[i], da);
+            da = row16_sum(da);
+        } else {
+#pragma unroll
+            for (int i = 0; i < KR; ++i) kr[i] *= after ? gt[i] : 1.f;
+        }
+        db = row16_sum(db);
+        if (i16 == 0) {
+            w.b[t * REC_CHUNK + s] = before ? 0.f : db;
+            if (KIND == REC_DELTA) As[t][s] = after ? da : 0.f;
+        }
+    }
+    float rq[KR], rk[KR];
+#pragma unroll
+    for (int i = 0; i < KR; ++i) {
+        const float inc = G[i] * g[i];
+        rq[i] = q[i] * (KIND == REC_DELTA ? inc : G[i]);
+        rk[i] = k[i] * inc;
+        G[i] = inc;
+        w.kh[(i16 * KR + i) * REC_CHUNK + s] = kr[i];
+    }
+    store_kr<KR>(w.qt + s * DP + i16 * KR, rq);
+    if (KIND == REC_DELTA) store_kr<KR>(w.kt + s * DP + i16 * KR, rk);
+    if (s == REC_CHUNK - 1) store_kr<KR>(w.gc + i16 * KR, G);
+    if (KIND == REC_DELTA) {
+        __syncthreads();
+        if (tid < REC_CHUNK) {  // column tid of T by forward substitution
+            float x[REC_CHUNK];
+#pragma unroll
+            for (int i = 0; i < REC_CHUNK; ++i) {
+                float sum = 0.f;
+#pragma unroll
+                for (int l = 0; l < i; ++l) sum = fmaf(As[i][l], x[l], sum);
+                x[i] = (i == tid ? 1.f : 0.f) - bs[i] * sum;
+                w.t[i * REC_CHUNK + tid] = x[i] * bs[tid];
+            }
+        }
+    }
+}
+
+template <int RT>
+struct ChunkFrag {
+    v4f kt[RT], qt[RT], kh[RT], gc[RT], t, b;
+    float v[4];
+};
+
+// Workgroup = 16 columns of one head; its four wavefronts hold a quarter of the key rows each (RT tiles of 16), their
+// partial products meet in LDS, everything after that is done by each wavefront for itself.  Operands: lane (c, g) gives
+// A[c][.] and B[.][c] for the four contraction indices 4 g + r of step r; accumulator r is row 4 g + r, column c -- so an
+// accumulator tile is the B operand of the next product as it stands.
+template <int KIND, int RT>
+__global__ __launch_bounds__(256) void recurrence_chunk_kernel(RecurrenceArgs a, float *ws_base, int chunks) {
+    constexpr int DP = RT * 64;
+    __shared__ float red[2][4][2][4][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int h = blockIdx.x, col = blockIdx.y * 16 + c, Dv = a.vdim;
+    const bool live = col < Dv;
+    float *Sg = a.state + ((size_t)h * Dv + (live ? col : 0)) * DP + wave * RT * 16 + g * 4;
+    v4f S[RT];
+#pragma unroll
+    for (int i = 0; i < RT; ++i) S[i] = *(const v4f *)(Sg + i * 16);
+    auto load = [&](ChunkFrag<RT> &f, int n) {
+        const ChunkWs w(ws_base + ((size_t)h * chunks + n) * rec_ws_floats(DP), DP);
+        const int d0 = wave * RT * 16;
+#pragma unroll
+        for (int i = 0; i < RT; ++i) {
+            f.qt[i] = *(const v4f *)(w.qt + c * DP + d0 + i * 16 + g * 4);
+            if (KIND == REC_DELTA) f.kt[i] = *(const v4f *)(w.kt + c * DP + d0 + i * 16 + g * 4);
+            f.kh[i] = *(const v4f *)(w.kh + (d0 + i * 16 + c) * REC_CHUNK + g * 4);
+            f.gc[i] = *(const v4f *)(w.gc + d0 + i * 16 + g * 4);
+        }
+        if (KIND == REC_DELTA) f.t = *(const v4f *)(w.t + c * REC_CHUNK + g * 4);
+        f.b = *(const v4f *)(w.b + c * REC_CHUNK + g * 4);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int t = n * REC_CHUNK + g * 4 + r;
+            f.v[r] = live && t < a.s ? a.v[(size_t)t * a.v_stride + h * Dv + col] : 0.f;
+        }
+    };
+    auto work = [&](const ChunkFrag<RT> &f, int n) {
+        v4f P = {0.f, 0.f, 0.f, 0.f}, O = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < RT; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                if (KIND == REC_DELTA) P = __builtin_amdgcn_mfma_f32_16x16x4f32(f.kt[i][r], S[i][r], P, 0, 0, 0);
+                O = __builtin_amdgcn_mfma_f32_16x16x4f32(f.qt[i][r], S[i][r], O, 0, 0, 0);
+            }
+        float (*rd)[2][4][64] = red[n & 1];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            if (KIND == REC_DELTA) rd[wave][0][r][lane] = P[r];
+            rd[wave][1][r][lane] = O[r];
+        }
+        __syncthreads();  // (one per chunk: the other half of red is written before the next one)
+        v4f U = {0.f, 0.f, 0.f, 0.f};
+        if (KIND == REC_DELTA) {
+            v4f R;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) R[r] = f.v[r] - ((rd[0][0][r][lane] + rd[1][0][r][lane]) + (rd[2][0][r][lane] + rd[3][0][r][lane]));
+#pragma unroll
+            for (int r = 0; r < 4; ++r) U = __builtin_amdgcn_mfma_f32_16x16x4f32(f.t[r], R[r], U, 0, 0, 0);
+        } else {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) U[r] = f.v[r];
+        }
+#pragma unroll
+        for (int i = 0; i < RT; ++i) {
+            S[i] *= f.gc[i];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.kh[i][r], U[r], S[i], 0, 0, 0);
+        }
+        if (wave == (n & 3)) {  // the wavefronts take turns with the output
+#pragma unroll
+            for (int r = 0; r < 4; ++r) O[r] = (rd[0][1][r][lane] + rd[1][1][r][lane]) + (rd[2][1][r][lane] + rd[3][1][r][lane]);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) O = __builtin_amdgcn_mfma_f32_16x16x4f32(f.b[r], U[r], O, 0, 0, 0);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int t = n * REC_CHUNK + g * 4 + r;
+                if (live && t < a.s) a.out[(size_t)t * a.out_stride + h * Dv + col] = O[r];
+            }
+        }
+    };
+    ChunkFrag<RT> fa, fb;  // the next chunk's operands travel while this one is worked on
+    load(fa, 0);
+    for (int n = 0; n < chunks; n += 2) {
+        if (n + 1 < chunks) load(fb, n + 1);
+        work(fa, n);
+        if (n + 1 < chunks) {
+            if (n + 2 < chunks) load(fa, n + 2);
+            work(fb, n + 1);
+        }
+    }
+    if (live)
+#pragma unroll
+        for (int i = 0; i < RT; ++i) *(v4f *)(Sg + i * 16) = S[i];
+}
+
+static int mixer_reserve_workspace(lumen_ctx *ctx, size_t bytes) {
+    if (ctx->mixer_ws_bytes >= bytes) return LUMEN_OK;
+    HIP_TRY(hipStreamSynchronize(ctx->stream));
+    if (ctx->mixer_ws) hipFree(ctx->mixer_ws);
+    ctx->mixer_ws = nullptr;
+    ctx->mixer_ws_bytes = 0;
+    HIP_TRY(hipMalloc((void **)&ctx->mixer_ws, bytes));
+    ctx->mixer_ws_bytes = bytes;
+    return LUMEN_OK;
+}
+
+size_t recurrence_workspace_bytes(int s, int heads, int dim) {
+    return (size_t)((s + REC_CHUNK - 1) / REC_CHUNK) * heads * rec_ws_floats(recurrence_rows(dim)) * sizeof(float);
+}
+
+// below this many tokens they are taken one by one
+#define REC_CHUNKED_MIN 8
+
 int launch_recurrence(lumen_ctx *ctx, const RecurrenceArgs &a) {
     if (a.s <= 0) return LUMEN_OK;
-    dim3 grid((a.vdim + REC_COLS - 1) / REC_COLS, a.heads);
     const int rows = recurrence_rows(a.dim);
+    if (a.s >= REC_CHUNKED_MIN) {
+        LUMEN_TRY(mixer_reserve_workspace(ctx, recurrence_workspace_bytes(a.s, a.heads, a.dim)));
+        const int chunks = (a.s + REC_CHUNK - 1) / REC_CHUNK;
+        // (heads along x: the column blocks of a head, which read the same operands, share an XCD's L2 when the heads
+        // are a multiple of 8)
+        const dim3 pgrid(chunks, a.heads), grid(a.heads, (a.vdim + 15) / 16);
+        float *ws = ctx->mixer_ws;
+#define REC_LAUNCH(KR)                                                                                                            \
+    do {                                                                                                                          \
+        if (a.kind == REC_WKV) {                                                                                                  \
+            hipLaunchKernelGGL((recurrence_chunk_prep_kernel<REC_WKV, KR>), pgrid, dim3(256), 0, ctx->stream, a, ws);             \
+            hipLaunchKernelGGL((recurrence_chunk_kernel<REC_WKV, KR / 4>), grid, dim3(256), 0, ctx->stream, a, ws, chunks);       \
+        } else {                                                                                                                  \
+            hipLaunchKernelGGL((recurrence_chunk_prep_kernel<REC_DELTA, KR>), pgrid, dim3(256), 0, ctx->stream, a, ws);           \
+            hipLaunchKernelGGL((recurrence_chunk_kernel<REC_DELTA, KR / 4>), grid, dim3(256), 0, ctx->stream, a, ws, chunks);     \
+        }                                                                                                                         \
+    } while (0)
+        if (rows == 64) REC_LAUNCH(4);
+        else if (rows == 128) REC_LAUNCH(8);
+        else REC_LAUNCH(16);
+#undef REC_LAUNCH
+        LUMEN_CHECK_LAUNCH();
+        return LUMEN_OK;
+    }
+    const dim3 grid((a.vdim + REC_COLS - 1) / REC_COLS, a.heads);
 #define REC_LAUNCH(KR)                                                                                            \
     do {                                                                                                          \
         if (a.kind == REC_WKV) hipLaunchKernelGGL((recurrence_kernel<REC_WKV, KR>), grid, dim3(256), 0, ctx->stream, a); \
@@ -197,82 +444,111 @@ __device__ __forceinline__ float conv_at(const float *__restrict__ in, int strid
     return acc;
 }
 
-// One workgroup per token: q and k of all kv heads go through LDS for their unit norms, v straight out.
-__global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepArgs a) {
-    LUMEN_DYNAMIC_LDS(float, qk);  // [2][kv_heads * dim]
-    const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int nq = a.kv_heads * a.dim, nv = a.heads * a.vdim, channels = 2 * nq + nv;
-    for (int c = tid; c < channels; c += 256) {
-        const int off = c < nq ? a.off_q + c : c < 2 * nq ? a.off_k + (c - nq) : a.off_v + (c - 2 * nq);
-        const float y = silu_r(conv_at(a.in + off, a.stride, a.taps_w + (size_t)c * a.taps, a.taps, t, a.conv_prev, channels, c));
-        if (c < 2 * nq) qk[c] = y;
-        else a.v[(size_t)t * nv + (c - 2 * nq)] = y;
-        if (t == a.s - 1) {  // the last taps - 1 inputs stay for the next portion
-            for (int j = 0; j < a.taps - 1; ++j) {
-                const int src = a.s - (a.taps - 1) + j;
-                a.conv_next[(size_t)j * channels + c] = src >= 0 ? a.in[(size_t)src * a.stride + off]
-                                                                 : a.conv_prev[(size_t)(a.taps - 1 + src) * channels + c];
+// One wavefront per token and head: unit u is a head of q, of k, or of v (convolution + SiLU, for q and k the unit
+// norm), or the copy of the two low-rank blocks.
+__global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepArgs a, int units) {
+    const long id = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63, t = (int)(id / units), u = (int)(id % units);
+    if (t >= a.s) return;  // (a whole wavefront)
+    const int G = a.kv_heads, nq = G * a.dim, nv = a.heads * a.vdim, channels = 2 * nq + nv;
+    if (u == units - 1) {
+        const float *row = a.in + (size_t)t * a.stride;
+        for (int i = lane; i < a.ra; i += 64) a.a1[(size_t)t * a.ra + i] = row[a.off_a1 + i];
+        for (int i = lane; i < a.rg; i += 64) a.g1[(size_t)t * a.rg + i] = row[a.off_g1 + i];
+        return;
+    }
+    const int part = u < G ? 0 : u < 2 * G ? 1 : 2, head = u - part * G, n = part == 2 ? a.vdim : a.dim;
+    const int ch0 = part * nq + head * n, off = (part == 0 ? a.off_q : part == 1 ? a.off_k : a.off_v) + head * n;
+    float y[MIX_MAX_DIM / 64], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < MIX_MAX_DIM / 64; ++i) {
+        const int c = i * 64 + lane;
+        y[i] = 0.f;
+        if (c < n) {
+            y[i] = silu_r(conv_at(a.in + off + c, a.stride, a.taps_w + (size_t)(ch0 + c) * a.taps, a.taps, t, a.conv_prev, channels, ch0 + c));
+            ss = fmaf(y[i], y[i], ss);
+            if (t == a.s - 1) {  // the last taps - 1 inputs stay for the next portion
+                for (int j = 0; j < a.taps - 1; ++j) {
+                    const int src = a.s - (a.taps - 1) + j;
+                    a.conv_next[(size_t)j * channels + ch0 + c] = src >= 0 ? a.in[(size_t)src * a.stride + off + c]
+                                                                           : a.conv_prev[(size_t)(a.taps - 1 + src) * channels + ch0 + c];
+                }
             }
         }
     }
-    const float *row = a.in + (size_t)t * a.stride;
-    for (int i = tid; i < a.ra; i += 256) a.a1[(size_t)t * a.ra + i] = row[a.off_a1 + i];
-    for (int i = tid; i < a.rg; i += 256) a.g1[(size_t)t * a.rg + i] = row[a.off_g1 + i];
-    __syncthreads();
-    for (int u = wave; u < 2 * a.kv_heads; u += 4) {  // head u of q (u < kv_heads) or of k
-        const float *p = qk + (size_t)u * a.dim;
-        float ss = 0.f;
-        for (int c = lane; c < a.dim; c += 64) ss = fmaf(p[c], p[c], ss);
-        ss = wave_sum(ss);
-        const bool is_q = u < a.kv_heads;
-        const float inv = (is_q ? a.q_scale : 1.0f) / sqrtf(ss + a.unit_eps);
-        float *dst = is_q ? a.q + (size_t)t * nq + (size_t)u * a.dim : a.k + (size_t)t * nq + (size_t)(u - a.kv_heads) * a.dim;
-        for (int c = lane; c < a.dim; c += 64) dst[c] = p[c] * inv;
-    }
+    ss = wave_sum(ss);
+    const float f = part == 2 ? 1.0f : (part == 0 ? a.q_scale : 1.0f) / sqrtf(ss + a.unit_eps);
+    float *dst = (part == 0 ? a.q + (size_t)t * nq : part == 1 ? a.k + (size_t)t * nq : a.v + (size_t)t * nv) + (size_t)head * n;
+#pragma unroll
+    for (int i = 0; i < MIX_MAX_DIM / 64; ++i)
+        if (i * 64 + lane < n) dst[i * 64 + lane] = y[i] * f;
 }
 
 int launch_delta_prep(lumen_ctx *ctx, const DeltaPrepArgs &a) {
     if (a.s <= 0) return LUMEN_OK;
-    const size_t lds = (size_t)2 * a.kv_heads * a.dim * sizeof(float);
-    if (lds > 64 * 1024)
-        HIP_TRY(hipFuncSetAttribute((const void *)delta_prep_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-    hipLaunchKernelGGL(delta_prep_kernel, dim3(a.s), dim3(256), lds, ctx->stream, a);
+    const int units = 2 * a.kv_heads + a.heads + 1;
+    hipLaunchKernelGGL(delta_prep_kernel, dim3((unsigned)(((long)a.s * units + 3) / 4)), dim3(256), 0, ctx->stream, a, units);
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
 }
 
 // ------------------------------------------------------------------ decode
-#define RD_THREADS 512
+#define RD_THREADS 1024
 #define RD_WAVES (RD_THREADS / 64)
+#define RD_COLS (RD_WAVES * 4)  // state columns per trip
 
-// dot product of a weight row of n (a multiple of 8) values with a vector in LDS
+// A quarter of the dot product of a weight row of n (a multiple of 8) values with a vector in LDS: lane p of four takes
+// every fourth 8-value piece; pieces are requested RD_AHEAD at a time.
+#define RD_AHEAD 4
 template <bool BF16>
-__device__ __forceinline__ float row_dot(const void *w, size_t row, const float *xs, int n) {
-    float s = 0.f;
-    if (BF16) {
-        const uint16_t *p = (const uint16_t *)w + row * n;
-        for (int k = 0; k < n; k += 8) {
-            const v4u r = *(const v4u *)(p + k);
+struct RowPart {
+    v4u w[RD_AHEAD][BF16 ? 1 : 2];
+    const char *row;
+    int n, p;
+    __device__ void fetch(int k0) {
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                s = fmaf(__uint_as_float(r[e] << 16), xs[k + 2 * e], s);
-                s = fmaf(__uint_as_float(r[e] & 0xffff0000u), xs[k + 2 * e + 1], s);
-            }
-        }
-    } else {
-        const float *p = (const float *)w + row * n;
-        for (int k = 0; k < n; k += 4) {
-            const v4f r = *(const v4f *)(p + k);
+        for (int i = 0; i < RD_AHEAD; ++i) {
+            const int k = min(k0 + i * 32 + p * 8, n - 8);
 #pragma unroll
-            for (int e = 0; e < 4; ++e) s = fmaf(r[e], xs[k + e], s);
+            for (int e = 0; e < (BF16 ? 1 : 2); ++e) w[i][e] = *(const v4u *)(row + (size_t)k * (BF16 ? 2 : 4) + 16 * e);
         }
     }
-    return s;
-}
+    __device__ void start(const void *base, size_t r, int n_, int p_) {
+        row = (const char *)base + r * n_ * (BF16 ? 2 : 4);
+        n = n_;
+        p = p_;
+        fetch(0);
+    }
+    __device__ float dot(const float *xs) {
+        float s = 0.f;
+        for (int k0 = 0; k0 < n; k0 += RD_AHEAD * 32) {
+            if (k0) fetch(k0);
+#pragma unroll
+            for (int i = 0; i < RD_AHEAD; ++i) {
+                const int k = k0 + i * 32 + p * 8;
+                if (k < n) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        if (BF16) {
+                            s = fmaf(__uint_as_float(w[i][0][e] << 16), xs[k + 2 * e], s);
+                            s = fmaf(__uint_as_float(w[i][0][e] & 0xffff0000u), xs[k + 2 * e + 1], s);
+                        } else {
+                            s = fmaf(__uint_as_float(w[i][0][e]), xs[k + e], s);
+                            s = fmaf(__uint_as_float(w[i][BF16 ? 0 : 1][e]), xs[k + 4 + e], s);
+                        }
+                    }
+                }
+            }
+        }
+        s += __shfl_xor(s, 1, 64);
+        s += __shfl_xor(s, 2, 64);
+        return s;
+    }
+};
 
-// One workgroup per head, 32 state columns per trip.  The state is requested first (it depends on nothing), then the
-// head's inputs are made: convolution and unit norms (delta), decay and gate rows of the low-rank products.
-template <int KIND, int KR, bool BF16>
+// One workgroup per head, 64 state columns per trip, NT trips.  The state and the low-rank rows are requested first
+// (they depend on nothing), then the head's inputs are made: convolution and unit norms (delta), decay and gate rows.
+template <int KIND, int KR, int NT, bool BF16>
 __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(RecurrenceDecodeArgs a) {
     constexpr int DP = 16 * KR;
     __shared__ __align__(16) float qs[DP], ks[DP], ws[DP];
@@ -281,10 +557,19 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
     __shared__ float red[2], red_o[RD_WAVES];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, i16 = lane & 15;
     const int h = blockIdx.x, rep = a.heads / a.kv_heads, hk = h / rep, D = a.dim, Dv = a.vdim;
+    // low-rank rows: four lanes per row, decay rows first
+    const int lr_rows = D + (KIND == REC_DELTA ? Dv : 0), lr_part = tid & 3;
+    RowPart<BF16> lr;
+    auto lr_start = [&](int r) {
+        if (r < D) lr.start(a.w_lo, (size_t)h * D + r, a.r_lo, lr_part);
+        else lr.start(a.w_hi, (size_t)h * Dv + (r - D), a.r_hi, lr_part);
+    };
+    lr_start(min(tid >> 2, lr_rows - 1));
     float *Sh = a.state + (size_t)h * Dv * DP + i16 * KR;
     const int c0 = wave * 4 + (lane >> 4);
-    float S[KR];
-    load_kr<KR>(S, Sh + (size_t)min(c0, Dv - 1) * DP);
+    float S[NT][KR];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) load_kr<KR>(S[n], Sh + (size_t)min(n * RD_COLS + c0, Dv - 1) * DP);
 
     for (int i = tid; i < a.r_lo; i += RD_THREADS) {
         const float x = a.proj[a.off_lo + i];
@@ -296,6 +581,7 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
         for (int i = tid; i < DP; i += RD_THREADS) {
             qs[i] = i < D ? a.proj[a.off_q + h * D + i] : 0.f;
             ks[i] = i < D ? a.proj[a.off_k + h * D + i] : 0.f;
+            ws[i] = 0.f;
         }
         for (int i = tid; i < Dv; i += RD_THREADS) {
             vs[i] = a.proj[a.off_v + h * Dv + i];
@@ -311,6 +597,7 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
             const int c = i - part * DP;
             if (part < 2 && c >= D) {
                 (part ? ks : qs)[c] = 0.f;
+                ws[c] = 0.f;
                 continue;
             }
             const int ch = part == 2 ? 2 * nq + h * Dv + c : part * nq + hk * D + c;
@@ -329,19 +616,22 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
         }
     }
     __syncthreads();
-    // decay and gate rows; the sums of squares of q and k meanwhile sit with the first two wavefronts
     const float decay_a = KIND == REC_DELTA ? expf(a.a_log[h]) : 0.f;
-    if (KIND == REC_DELTA && wave < 2) {
+    if (KIND == REC_DELTA && wave < 2) {  // the sums of squares of q and of k
         const float *p = wave ? ks : qs;
         float ss = 0.f;
         for (int c = lane; c < D; c += 64) ss = fmaf(p[c], p[c], ss);
         ss = wave_sum(ss);
         if (lane == 0) red[wave] = (wave ? 1.0f : a.q_scale) / sqrtf(ss + a.unit_eps);
     }
-    for (int i = tid; i < DP + (KIND == REC_DELTA ? Dv : 0); i += RD_THREADS) {
-        if (i < D) ws[i] = decay_r<KIND>(row_dot<BF16>(a.w_lo, (size_t)h * D + i, lo, a.r_lo), a.bias[h * D + i], decay_a);
-        else if (i < DP) ws[i] = 0.f;
-        else gs[i - DP] = sigmoid_r(row_dot<BF16>(a.w_hi, (size_t)h * Dv + (i - DP), hi, a.r_hi));
+    for (int r0 = 0; r0 < lr_rows; r0 += RD_THREADS / 4) {  // (uniform trips, rows clamped: the lanes exchange parts)
+        const int r = r0 + (tid >> 2), rc = min(r, lr_rows - 1);
+        if (r0) lr_start(rc);
+        const float z = lr.dot(rc < D ? lo : hi);
+        if (lr_part == 0 && r < lr_rows) {
+            if (r < D) ws[r] = decay_r<KIND>(z, a.bias[h * D + r], decay_a);
+            else gs[r - D] = sigmoid_r(z);
+        }
     }
     __syncthreads();
     float q[KR], k[KR], w[KR], u[KR];
@@ -364,12 +654,12 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
         u[i] = KIND == REC_WKV && kc < D ? a.u[h * D + kc] : 0.f;
     }
     float ss = 0.f;
-    for (int cb = 0; cb < Dv; cb += RD_WAVES * 4) {  // (uniform trips: the lane exchanges need whole wavefronts)
-        const int c = cb + c0;
-        if (cb) load_kr<KR>(S, Sh + (size_t)min(c, Dv - 1) * DP);
-        const float o = column_step<KIND, KR>(S, q, k, w, u, vs[min(c, Dv - 1)], beta);
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+        const int c = n * RD_COLS + c0;
+        const float o = column_step<KIND, KR>(S[n], q, k, w, u, vs[min(c, Dv - 1)], beta);
         if (c < Dv) {
-            store_kr<KR>(Sh + (size_t)c * DP, S);
+            store_kr<KR>(Sh + (size_t)c * DP, S[n]);
             if (i16 == 0) {
                 os[c] = o;
                 ss = fmaf(o, o, ss);
@@ -388,22 +678,29 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
 }
 
 int launch_recurrence_decode(lumen_ctx *ctx, const RecurrenceDecodeArgs &a) {
-    const int rows = recurrence_rows(a.dim);
-    note_kernel(ctx, "recurrence_decode_kernel<%d, %d, %s>", a.kind, rows / 16, a.w_bf16 ? "true" : "false");
-#define RD_LAUNCH(KIND, KR)                                                                                               \
+    const int rows = recurrence_rows(a.dim), trips = (a.vdim + RD_COLS - 1) / RD_COLS, nt = trips <= 1 ? 1 : trips <= 2 ? 2 : 4;
+    note_kernel(ctx, "recurrence_decode_kernel<%d, %d, %d, %s>", a.kind, rows / 16, nt, a.w_bf16 ? "true" : "false");
+#define RD_LAUNCH(KIND, KR, NT)                                                                                           \
     do {                                                                                                                  \
-        if (a.w_bf16) hipLaunchKernelGGL((recurrence_decode_kernel<KIND, KR, true>), dim3(a.heads), dim3(RD_THREADS), 0, ctx->stream, a); \
-        else hipLaunchKernelGGL((recurrence_decode_kernel<KIND, KR, false>), dim3(a.heads), dim3(RD_THREADS), 0, ctx->stream, a);         \
+        if (a.w_bf16) hipLaunchKernelGGL((recurrence_decode_kernel<KIND, KR, NT, true>), dim3(a.heads), dim3(RD_THREADS), 0, ctx->stream, a); \
+        else hipLaunchKernelGGL((recurrence_decode_kernel<KIND, KR, NT, false>), dim3(a.heads), dim3(RD_THREADS), 0, ctx->stream, a);         \
+    } while (0)
+#define RD_TRIPS(KIND, KR)                     \
+    do {                                       \
+        if (nt == 1) RD_LAUNCH(KIND, KR, 1);   \
+        else if (nt == 2) RD_LAUNCH(KIND, KR, 2); \
+        else RD_LAUNCH(KIND, KR, 4);           \
     } while (0)
 #define RD_KIND(KIND)                   \
     do {                                \
-        if (rows == 64) RD_LAUNCH(KIND, 4);  \
-        else if (rows == 128) RD_LAUNCH(KIND, 8); \
-        else RD_LAUNCH(KIND, 16);       \
+        if (rows == 64) RD_TRIPS(KIND, 4);  \
+        else if (rows == 128) RD_TRIPS(KIND, 8); \
+        else RD_TRIPS(KIND, 16);        \
     } while (0)
     if (a.kind == REC_WKV) RD_KIND(REC_WKV);
     else RD_KIND(REC_DELTA);
 #undef RD_KIND
+#undef RD_TRIPS
 #undef RD_LAUNCH
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;

@@ -7,11 +7,30 @@
 
 typedef float v4f __attribute__((ext_vector_type(4)));
 
-__device__ __forceinline__ float shaped_score(float dot, float scale, float softcap, float r1, float r2, int dist) {
-    float s = dot * scale;
-    if (softcap > 0.f) s = softcap * tanhf(s / softcap);
-    return s - r1 * logf(1.0f + r2 * (float)dist);
+// tanh by the continued fraction x / (1 + x^2 / (3 + x^2 / (5 + x^2 / (7 + x^2 / 9)))) up to 0.9 (truncation below
+// 2.4e-8 there), by 1 - 2 / (e^{2 |x|} + 1) beyond: the absolute error stays small against x, which a soft cap multiplies.
+__device__ __forceinline__ float tanh_w(float x) {
+    const float y = x * x;
+    const float near = x * fmaf(y, y + 105.0f, 945.0f) * __builtin_amdgcn_rcpf(fmaf(y, fmaf(y, 15.0f, 420.0f), 945.0f));
+    const float far = 1.0f - 2.0f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(2.88539008177792681f * fabsf(x)) + 1.0f);
+    return y <= 0.81f ? near : copysignf(far, x);
 }
+
+// Scores are kept in log2 units (times log2 e), so that a weight is one base-2 exponential and the distance bias
+// r1 ln(1 + r2 d) is r1 log2(1 + r2 d).
+struct ScoreShape {
+    float in, out, r1, r2;  // score = out tanh(in dot), or in dot when out is 0
+    __device__ ScoreShape(float scale, float softcap, float r1_, float r2_) : r1(r1_), r2(r2_) {
+        const float log2e = 1.44269504088896341f;
+        in = softcap > 0.f ? scale / softcap : scale * log2e;
+        out = softcap > 0.f ? softcap * log2e : 0.f;
+    }
+    __device__ float operator()(float dot, int dist) const {
+        float s = in * dot;
+        if (out > 0.f) s = out * tanh_w(s);
+        return fmaf(-r1, __builtin_amdgcn_logf(fmaf(r2, (float)dist, 1.0f)), s);
+    }
+};
 
 __device__ __forceinline__ float gate_w(float z, int act) {
     const float sig = 1.0f / (1.0f + expf(-z));
@@ -32,6 +51,7 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
     constexpr int GROUPS = WD_THREADS / LV;
     constexpr int KEYS = WINDOW_SLICE_KEYS / (WD_WAVES * 4);  // keys of a row of 16 lanes
     constexpr int U = DB == 1 ? 8 : DB == 2 ? 4 : 2;          // key rows in flight
+    constexpr int VA = WINDOW_SLICE_KEYS / GROUPS < 8 ? WINDOW_SLICE_KEYS / GROUPS : 8;  // value rows requested ahead
     __shared__ __align__(16) float qs[DB * 64], kn[DB * 64], vn[LV * 4];
     __shared__ float sc[WINDOW_SLICE_KEYS];
     __shared__ __align__(16) float ctx[GROUPS][LV * 4];
@@ -61,6 +81,15 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
         }
     };
     fetch(0);
+    const int grp = tid / LV, d4 = (tid % LV) * 4;
+    auto value_row = [&](int key) {
+        v4f v = {0.f, 0.f, 0.f, 0.f};
+        if (key < n && d4 < a.vpad) v = *(const v4f *)(vr + (size_t)((lo + key) % a.cap) * a.vpad + d4);
+        return v;
+    };
+    v4f vb[VA];
+#pragma unroll
+    for (int i = 0; i < VA; ++i) vb[i] = value_row(grp + i * GROUPS);
 
     // queries and the new key, normalised over all heads together
     float sq = 0.f, sk = 0.f;
@@ -131,17 +160,17 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
         }
     }
     __syncthreads();
-    const float r1 = a.r1 ? a.r1[h] : 0.f, r2 = a.r1 ? a.r2[h] : 0.f;
+    const ScoreShape shape(a.scale, a.softcap, a.r1 ? a.r1[h] : 0.f, a.r1 ? a.r2[h] : 0.f);
     float s = -INFINITY;
-    if (tid < n) s = shaped_score(sc[tid], a.scale, a.softcap, r1, r2, pos - lo - tid);
+    if (tid < n) s = shape(sc[tid], pos - lo - tid);
     float m = wave_max(s);
     if (lane == 0) red_m[wave] = m;
     __syncthreads();
     m = red_m[0];
 #pragma unroll
     for (int w = 1; w < WD_WAVES; ++w) m = fmaxf(m, red_m[w]);
-    const float p = tid < n ? expf(s - m) : 0.f;
-    sc[tid] = p;
+    const float p = tid < n ? __builtin_amdgcn_exp2f(s - m) : 0.f;
+    if (tid < WINDOW_SLICE_KEYS) sc[tid] = p;
     float l = wave_sum(p);
     if (lane == 0) red_l[wave] = l;
     __syncthreads();
@@ -149,18 +178,17 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
 #pragma unroll
     for (int w = 0; w < WD_WAVES; ++w) l += red_l[w];
 
-    const int grp = tid / LV, d4 = (tid % LV) * 4;
     v4f acc = {0.f, 0.f, 0.f, 0.f};
-    const bool col_ok = d4 < a.vpad;
-#pragma unroll 8
-    for (int key = grp; key < n; key += GROUPS) {
-        v4f v4 = {0.f, 0.f, 0.f, 0.f};
+    auto add = [&](int key, v4f v4) {
         if (lo + key == pos) v4 = *(const v4f *)(vn + d4);
-        else if (col_ok) v4 = *(const v4f *)(vr + (size_t)((lo + key) % a.cap) * a.vpad + d4);
-        const float w = sc[key];
+        const float w = key < n ? sc[key] : 0.f;
 #pragma unroll
         for (int e = 0; e < 4; ++e) acc[e] = fmaf(w, v4[e], acc[e]);
-    }
+    };
+#pragma unroll
+    for (int i = 0; i < VA; ++i) add(grp + i * GROUPS, vb[i]);
+#pragma unroll 4
+    for (int key = grp + VA * GROUPS; key < n; key += GROUPS) add(key, value_row(key));
     *(v4f *)(&ctx[grp][d4]) = acc;
     __syncthreads();
     for (int d = tid; d < Dv; d += WD_THREADS) {
@@ -185,10 +213,10 @@ __global__ __launch_bounds__(256) void window_merge_kernel(WindowAttnArgs a) {
     float m = -INFINITY;
     for (int s = 0; s < used; ++s) m = fmaxf(m, part[(size_t)s * (Dv + 2) + Dv]);
     float l = 0.f;
-    for (int s = 0; s < used; ++s) l = fmaf(part[(size_t)s * (Dv + 2) + Dv + 1], expf(part[(size_t)s * (Dv + 2) + Dv] - m), l);
+    for (int s = 0; s < used; ++s) l = fmaf(part[(size_t)s * (Dv + 2) + Dv + 1], __builtin_amdgcn_exp2f(part[(size_t)s * (Dv + 2) + Dv] - m), l);
     for (int d = threadIdx.x; d < Dv; d += 256) {
         float o = 0.f;
-        for (int s = 0; s < used; ++s) o = fmaf(part[(size_t)s * (Dv + 2) + d], expf(part[(size_t)s * (Dv + 2) + Dv] - m), o);
+        for (int s = 0; s < used; ++s) o = fmaf(part[(size_t)s * (Dv + 2) + d], __builtin_amdgcn_exp2f(part[(size_t)s * (Dv + 2) + Dv] - m), o);
         a.out[h * Dv + d] = o / l * (a.gate ? gate_w(a.gate[h * Dv + d], a.gate_act) : 1.0f);
     }
 }
@@ -207,7 +235,7 @@ int launch_window_attn_decode(lumen_ctx *ctx, const WindowAttnArgs &a) {
     else if (db == 2) WD_LAUNCH(2);
     else WD_LAUNCH(4);
 #undef WD_LAUNCH
-    if (a.slices > 1) hipLaunchKernelGGL(window_merge_kernel, dim3(a.heads), dim3(256), 0, ctx->stream, a);
+    if (a.slices > 1 && !a.leave_slices) hipLaunchKernelGGL(window_merge_kernel, dim3(a.heads), dim3(256), 0, ctx->stream, a);
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
 }
@@ -266,7 +294,7 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
     const int t0 = blockIdx.x * WP_Q, tw = t0 + wave * 16, t = tw + c;  // first token of the workgroup / wavefront, own token
     const int last = min(t0 + WP_Q, a.s) - 1;
     const int i = a.pos + t;  // own position
-    const float r1 = a.r1 ? a.r1[h] : 0.f, r2 = a.r1 ? a.r2[h] : 0.f;
+    const ScoreShape shape(a.scale, a.softcap, a.r1 ? a.r1[h] : 0.f, a.r1 ? a.r2[h] : 0.f);
     const float *kr = a.k_ring + (size_t)hk * a.cap * a.dpad, *vr = a.v_ring + (size_t)hk * a.cap * a.vpad;
 
     v4f qf[NB], acc[NB];
@@ -322,20 +350,20 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int dist = i - (j0 + u * 16 + g * 4 + r);
-                sc[u][r] = dist >= 0 && dist < a.window ? shaped_score(sc[u][r], a.scale, a.softcap, r1, r2, dist) : -INFINITY;
+                sc[u][r] = dist >= 0 && dist < a.window ? shape(sc[u][r], dist) : -INFINITY;
                 mx = fmaxf(mx, sc[u][r]);
             }
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
         mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
         const float base = mx > -INFINITY ? mx : 0.f;  // (a query that has seen nothing yet keeps zero weights)
-        const float f = expf(m - base);
+        const float f = __builtin_amdgcn_exp2f(m - base);
         m = mx;
         l *= f;
 #pragma unroll
         for (int u = 0; u < 2; ++u)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                sc[u][r] = expf(sc[u][r] - base);
+                sc[u][r] = __builtin_amdgcn_exp2f(sc[u][r] - base);
                 l += sc[u][r];
             }
 #pragma unroll

@@ -5,6 +5,7 @@ HybridConfig holds a model of that family whatever its origin; pinavik_config re
 model into one.
 """
 import ctypes as C
+import warnings
 from dataclasses import dataclass, field
 from typing import List
 
@@ -111,7 +112,7 @@ class HybridModel(DecoderModel):
 def _known(d, keys, where):
     extra = sorted(set(d) - set(keys))
     if extra:
-        raise LumenError(ERR_INVALID, "config.json: %s: unknown %s" % (where, ", ".join(extra)))
+        warnings.warn("config.json: %s: ignoring unknown %s" % (where, ", ".join(extra)))
 
 
 def pinavik_config(cfg, shape_of, max_seq_len, weight_dtype):
@@ -129,7 +130,7 @@ def pinavik_config(cfg, shape_of, max_seq_len, weight_dtype):
         pre = "l%d.mix." % i
         if kind == "attention":
             _known(m, ("heads", "kv_heads", "dim", "vdim", "mask", "scale", "softcap"), "attention of layer %d" % i)
-            y.window, y.scale, y.softcap = m["mask"]["size"], m["scale"], m["softcap"]
+            y.window, y.scale, y.softcap = m["mask"]["size"], m["scale"], m.get("softcap") or 0.0
         elif kind == "wkv":
             _known(m, ("heads", "dim"), "wkv of layer %d" % i)
             y.rank_lo = shape_of(pre + "w1")[0]

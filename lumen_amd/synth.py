@@ -118,3 +118,52 @@ def bf16_round(x):
 def bf16_widen(bits):
     """bf16 bits -> f32, exact (the reference's load-time upcast, src/loader.rs:58)."""
     return (np.ascontiguousarray(bits, np.uint16).astype(np.uint32) << 16).view(np.float32)
+
+
+# --- layered hybrid decoder (lumen_amd/hybrid.py) beside a Llama of the same size ----------------------
+def hybrid_shape(width, weight_dtype="bf16", groups=3, max_seq_len=8192):
+    """A HybridConfig whose layers resemble a real model's: groups of attention (window 1024), channel_delta, wkv,
+    channel_delta, the middle group run twice; heads of 64 (attention, wkv) and 128 (delta), feed-forward 4 x width
+    (two matrices of it hold what three of 8/3 x width do in a SwiGLU layer)."""
+    from .hybrid import HybridConfig, HybridLayer
+    ff = 4 * width
+    delta = dict(heads=width // 128, kv_heads=width // 128, dim=128, vdim=128, conv=4, rank_lo=128, rank_hi=128, ff=ff)
+    group = [HybridLayer("attention", heads=width // 64, kv_heads=max(width // 256, 1), dim=64, vdim=64, window=1024,
+                         scale=0.125, softcap=30.0, ff=ff),
+             HybridLayer("channel_delta", **delta),
+             HybridLayer("wkv", heads=width // 64, kv_heads=width // 64, dim=64, vdim=64, rank_lo=64, ff=ff),
+             HybridLayer("channel_delta", **delta)]
+    mid = groups // 2 * 4
+    return HybridConfig(32000, width, group * groups, mid, mid + 4, 2, embed_scale=width ** 0.5, norm_offset=1.0,
+                        residual_mult=0.6, max_seq_len=max_seq_len, weight_dtype=weight_dtype)
+
+
+def llama_beside(width, weight_dtype="bf16", layers=16, max_seq_len=8192):
+    """The Llama shape of equal width, layer runs and feed-forward volume."""
+    return dict(vocab_size=32000, hidden_size=width, intermediate_size=(8 * width // 3 + 127) // 128 * 128,
+                num_hidden_layers=layers, num_attention_heads=width // 64, num_key_value_heads=max(width // 256, 1),
+                rms_norm_eps=1e-6, max_seq_len=max_seq_len, rope_theta=10000.0, weight_dtype=weight_dtype)
+
+
+def hybrid_param(name, shape, seed):
+    """A tensor of a hybrid model: N(0, fan_in^-1/2) matrices, decays that let the state live for tens of tokens."""
+    rng = _rng(seed, name)
+    leaf = name.split(".")[-1]
+    a = rng.standard_normal(shape, dtype=np.float32)
+    if name.endswith("conv"):
+        return a * np.float32(shape[-1] ** -0.5)
+    if leaf in ("norm1", "norm2") or name == "final.norm":
+        return a * np.float32(0.1)
+    if leaf == "norm":
+        return 1 + a * np.float32(0.1)
+    if name.startswith("loop.step"):
+        return a * np.float32(0.1)
+    if len(shape) == 2 and leaf not in ("u",):
+        return a * np.float32(shape[-1] ** -0.5)
+    if leaf == "act":
+        return np.array([0.5, 0.3, 0.2, 0.05], np.float32) + a * np.float32(0.02)
+    if leaf in ("r1", "r2") or ".mu." in name:
+        return np.abs(a) * np.float32(0.3)
+    if leaf in ("w0", "dt_bias"):
+        return a * np.float32(0.5) - np.float32(2.5)
+    return a * np.float32(0.3)

@@ -7,7 +7,7 @@
 //
 // Wavefront-wide operations (DPP rotations, lane reads, shuffles) exchange values through a slot array of the
 // wavefront once every live lane has arrived: every lane must reach the call, as on the GPU.
-// The matrix-core instructions are not emulated: a kernel that issues one stops the program.
+// The matrix-core instructions the library issues are emulated lane by lane (slowly).
 #pragma once
 #define LUMEN_CPU_EMU 1
 #include <stdint.h>
@@ -86,6 +86,8 @@ static inline unsigned __float_as_uint(float f) { return emu_bits_of(f); }
 static inline int __float_as_int(float f) { return (int)emu_bits_of(f); }
 static inline float __int_as_float(int i) { return emu_bits_to<float>((uint32_t)i); }
 #define __builtin_amdgcn_exp2f(x) exp2f(x)
+#define __builtin_amdgcn_logf(x) log2f(x)  // (v_log_f32 is the base-2 logarithm)
+#define __builtin_amdgcn_rcpf(x) (1.0f / (x))
 #define __builtin_amdgcn_s_waitcnt(x) ((void)0)
 #define __builtin_amdgcn_sched_group_barrier(a, b, c) ((void)0)
 void emu_sleep();
@@ -105,7 +107,32 @@ static inline unsigned emu_perm(unsigned hi, unsigned lo, unsigned sel) {  // v_
     return out;
 }
 #define __builtin_amdgcn_perm(hi, lo, sel) emu_perm((hi), (lo), (sel))
-#define __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, x, y, z) (emu::not_emulated("v_mfma_f32_32x32x16_bf16"), (c))
+// v_mfma_f32_32x32x16_bf16: D[i][j] = C[i][j] + sum over k < 16 of A[i][k] B[k][j]; lane l gives the eight bf16
+// A[l % 32][8 (l / 32) + e] and B[8 (l / 32) + e][l % 32] and holds D[8 (r / 4) + 4 (l / 32) + r % 4][l % 32] in element r.
+template <typename A, typename V>
+static inline V emu_mfma_32x32x16bf16(A a, A b, V c) {
+    static_assert(sizeof(A) == 16, "eight bf16 values");
+    const int lane = (int)(threadIdx.x & 63), j = lane & 31, g = lane >> 5;
+    uint32_t aw[4], bw[4];
+    memcpy(aw, &a, 16);
+    memcpy(bw, &b, 16);
+    float bk[16];
+    for (int h = 0; h < 2; ++h)
+        for (int w = 0; w < 4; ++w) {
+            const uint32_t u = emu::wave_exchange(bw[w], h * 32 + j);
+            bk[h * 8 + 2 * w] = emu_bits_to<float>(u << 16);
+            bk[h * 8 + 2 * w + 1] = emu_bits_to<float>(u & 0xffff0000u);
+        }
+    for (int r = 0; r < 16; ++r)
+        for (int h = 0; h < 2; ++h)
+            for (int w = 0; w < 4; ++w) {
+                const uint32_t u = emu::wave_exchange(aw[w], h * 32 + 8 * (r / 4) + 4 * g + r % 4);
+                c[r] = fmaf(emu_bits_to<float>(u << 16), bk[h * 8 + 2 * w], c[r]);
+                c[r] = fmaf(emu_bits_to<float>(u & 0xffff0000u), bk[h * 8 + 2 * w + 1], c[r]);
+            }
+    return c;
+}
+#define __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, x, y, z) emu_mfma_32x32x16bf16((a), (b), (c))
 // v_mfma_f32_16x16x4_f32: D[i][j] = C[i][j] + sum over k < 4 of A[i][k] B[k][j]; lane l gives A[l % 16][l / 16] and
 // B[l / 16][l % 16] and holds D[4 (l / 16) + r][l % 16] in element r.  (The order of the four products inside the
 // instruction is the hardware's; results are compared to a tolerance.)
