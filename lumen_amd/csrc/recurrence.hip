@@ -167,15 +167,26 @@ __global__ __launch_bounds__(256) void recurrence_chunk_prep_kernel(RecurrenceAr
     const bool live = t0 + s < a.s;
     const float decay_a = KIND == REC_DELTA ? expf(a.a_log[h]) : 0.f;
     float q[KR], k[KR], g[KR], uk[KR];
+    {   // (positions beyond the head or the sequence are clamped, so that all requests go out together)
+        const size_t t = (size_t)min(t0 + s, a.s - 1);
+        float z[KR], bias[KR], u[KR];
 #pragma unroll
-    for (int i = 0; i < KR; ++i) {
-        const int c = i16 * KR + i;
-        const bool ok = live && c < D;
-        const size_t t = (size_t)(t0 + s);
-        q[i] = ok ? a.q[t * a.q_stride + hk * D + c] : 0.f;
-        k[i] = ok ? a.k[t * a.k_stride + hk * D + c] : 0.f;
-        g[i] = ok ? decay_r<KIND>(a.z[t * a.z_stride + h * D + c], a.bias[h * D + c], decay_a) : 1.f;  // (a missing token changes nothing)
-        uk[i] = KIND == REC_WKV && ok ? a.u[h * D + c] * k[i] : 0.f;
+        for (int i = 0; i < KR; ++i) {
+            const int c = min(i16 * KR + i, D - 1);
+            q[i] = a.q[t * a.q_stride + hk * D + c];
+            k[i] = a.k[t * a.k_stride + hk * D + c];
+            z[i] = a.z[t * a.z_stride + h * D + c];
+            bias[i] = a.bias[h * D + c];
+            u[i] = KIND == REC_WKV ? a.u[h * D + c] : 0.f;
+        }
+#pragma unroll
+        for (int i = 0; i < KR; ++i) {
+            const bool ok = live && i16 * KR + i < D;
+            q[i] = ok ? q[i] : 0.f;
+            k[i] = ok ? k[i] : 0.f;
+            g[i] = ok ? decay_r<KIND>(z[i], bias[i], decay_a) : 1.f;  // (a missing token changes nothing)
+            uk[i] = u[i] * k[i];
+        }
     }
     store_kr<KR>(&qs[s][i16 * KR], q);
     store_kr<KR>(&ks[s][i16 * KR], k);
@@ -281,8 +292,9 @@ __global__ __launch_bounds__(256) void recurrence_chunk_kernel(RecurrenceArgs a,
         f.b = *(const v4f *)(w.b + c * REC_CHUNK + g * 4);
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const int t = n * REC_CHUNK + g * 4 + r;
-            f.v[r] = live && t < a.s ? a.v[(size_t)t * a.v_stride + h * Dv + col] : 0.f;
+            // (clamped, not skipped: a load behind a branch would make the wavefront wait for all that are in flight)
+            const int t = min(n * REC_CHUNK + g * 4 + r, a.s - 1);
+            f.v[r] = a.v[(size_t)t * a.v_stride + h * Dv + min(col, Dv - 1)];
         }
     };
     auto work = [&](const ChunkFrag<RT> &f, int n) {
@@ -305,12 +317,12 @@ __global__ __launch_bounds__(256) void recurrence_chunk_kernel(RecurrenceArgs a,
         if (KIND == REC_DELTA) {
             v4f R;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) R[r] = f.v[r] - ((rd[0][0][r][lane] + rd[1][0][r][lane]) + (rd[2][0][r][lane] + rd[3][0][r][lane]));
+            for (int r = 0; r < 4; ++r) R[r] = (n * REC_CHUNK + g * 4 + r < a.s ? f.v[r] : 0.f) - ((rd[0][0][r][lane] + rd[1][0][r][lane]) + (rd[2][0][r][lane] + rd[3][0][r][lane]));
 #pragma unroll
             for (int r = 0; r < 4; ++r) U = __builtin_amdgcn_mfma_f32_16x16x4f32(f.t[r], R[r], U, 0, 0, 0);
         } else {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) U[r] = f.v[r];
+            for (int r = 0; r < 4; ++r) U[r] = n * REC_CHUNK + g * 4 + r < a.s ? f.v[r] : 0.f;
         }
 #pragma unroll
         for (int i = 0; i < RT; ++i) {
@@ -432,62 +444,91 @@ int launch_head_norm_gate(lumen_ctx *ctx, float *o, int stride, const float *gai
     return LUMEN_OK;
 }
 
-// Causal convolution of one channel at token t of this portion: taps_w[taps - 1] is the current token's.
-__device__ __forceinline__ float conv_at(const float *__restrict__ in, int stride, const float *__restrict__ w, int taps, int t,
-                                         const float *__restrict__ prev, int channels, int ch) {
-    float acc = 0.f;
-    for (int j = 0; j < taps; ++j) {
-        const int src = t - (taps - 1) + j;
-        const float x = src >= 0 ? in[(size_t)src * stride] : prev[(size_t)(taps - 1 + src) * channels + ch];
-        acc = fmaf(w[j], x, acc);
-    }
-    return acc;
-}
-
-// One wavefront per token and head: unit u is a head of q, of k, or of v (convolution + SiLU, for q and k the unit
-// norm), or the copy of the two low-rank blocks.
+// Causal convolution + SiLU of a head of q, of k or of v, the unit norm of the first two: one wavefront per head (unit) and
+// 8 tokens, weights and the inputs' sliding window in registers.  TAPS: taps the registers are laid out for (missing
+// ones have weight zero); CH: 64-channel blocks of a head.  The last unit copies the two low-rank blocks.
+#define PREP_TOK 8
+template <int TAPS, int CH>
 __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepArgs a, int units) {
     const long id = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-    const int lane = threadIdx.x & 63, t = (int)(id / units), u = (int)(id % units);
-    if (t >= a.s) return;  // (a whole wavefront)
-    const int G = a.kv_heads, nq = G * a.dim, nv = a.heads * a.vdim, channels = 2 * nq + nv;
+    const int lane = threadIdx.x & 63, t0 = (int)(id / units) * PREP_TOK, u = (int)(id % units);
+    if (t0 >= a.s) return;  // (a whole wavefront)
+    const int G = a.kv_heads, nq = G * a.dim, nv = a.heads * a.vdim, channels = 2 * nq + nv, keep = a.taps - 1;
+    const int nt = min(PREP_TOK, a.s - t0);
     if (u == units - 1) {
-        const float *row = a.in + (size_t)t * a.stride;
-        for (int i = lane; i < a.ra; i += 64) a.a1[(size_t)t * a.ra + i] = row[a.off_a1 + i];
-        for (int i = lane; i < a.rg; i += 64) a.g1[(size_t)t * a.rg + i] = row[a.off_g1 + i];
+        for (int t = t0; t < t0 + nt; ++t) {
+            const float *row = a.in + (size_t)t * a.stride;
+            for (int i = lane; i < a.ra; i += 64) a.a1[(size_t)t * a.ra + i] = row[a.off_a1 + i];
+            for (int i = lane; i < a.rg; i += 64) a.g1[(size_t)t * a.rg + i] = row[a.off_g1 + i];
+        }
         return;
     }
     const int part = u < G ? 0 : u < 2 * G ? 1 : 2, head = u - part * G, n = part == 2 ? a.vdim : a.dim;
     const int ch0 = part * nq + head * n, off = (part == 0 ? a.off_q : part == 1 ? a.off_k : a.off_v) + head * n;
-    float y[MIX_MAX_DIM / 64], ss = 0.f;
+    float y[CH][PREP_TOK], ss[PREP_TOK];
 #pragma unroll
-    for (int i = 0; i < MIX_MAX_DIM / 64; ++i) {
-        const int c = i * 64 + lane;
-        y[i] = 0.f;
-        if (c < n) {
-            y[i] = silu_r(conv_at(a.in + off + c, a.stride, a.taps_w + (size_t)(ch0 + c) * a.taps, a.taps, t, a.conv_prev, channels, ch0 + c));
-            ss = fmaf(y[i], y[i], ss);
-            if (t == a.s - 1) {  // the last taps - 1 inputs stay for the next portion
-                for (int j = 0; j < a.taps - 1; ++j) {
-                    const int src = a.s - (a.taps - 1) + j;
-                    a.conv_next[(size_t)j * channels + ch0 + c] = src >= 0 ? a.in[(size_t)src * a.stride + off + c]
-                                                                           : a.conv_prev[(size_t)(a.taps - 1 + src) * channels + ch0 + c];
-                }
+    for (int t = 0; t < PREP_TOK; ++t) ss[t] = 0.f;
+#pragma unroll
+    for (int b = 0; b < CH; ++b) {
+        const bool ok = b * 64 + lane < n;
+        const int c = min(b * 64 + lane, n - 1);
+        float w[TAPS], x[TAPS - 1 + PREP_TOK];
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) {
+            const int jj = j - (TAPS - a.taps);
+            w[j] = a.taps_w[(size_t)(ch0 + c) * a.taps + max(jj, 0)];
+            w[j] = jj >= 0 ? w[j] : 0.f;
+        }
+#pragma unroll
+        for (int i = 0; i < TAPS - 1 + PREP_TOK; ++i) {  // input of token t0 - (TAPS - 1) + i, or the state's
+            const int src = min(t0 - (TAPS - 1) + i, a.s - 1);
+            const float *p = src >= 0 || src < -keep ? a.in + (size_t)max(src, 0) * a.stride + off + c
+                                                     : a.conv_prev + (size_t)(keep + src) * channels + ch0 + c;
+            x[i] = *p;
+        }
+#pragma unroll
+        for (int t = 0; t < PREP_TOK; ++t) {
+            float acc = 0.f;
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) acc = fmaf(w[j], x[t + j], acc);
+            y[b][t] = ok ? silu_r(acc) : 0.f;
+            ss[t] = fmaf(y[b][t], y[b][t], ss[t]);
+        }
+        if (ok && t0 + nt == a.s) {  // the last taps - 1 inputs stay for the next portion
+            for (int j = 0; j < keep; ++j) {
+                const int src = a.s - keep + j;
+                a.conv_next[(size_t)j * channels + ch0 + c] = src >= 0 ? a.in[(size_t)src * a.stride + off + c]
+                                                                       : a.conv_prev[(size_t)(keep + src) * channels + ch0 + c];
             }
         }
     }
-    ss = wave_sum(ss);
-    const float f = part == 2 ? 1.0f : (part == 0 ? a.q_scale : 1.0f) / sqrtf(ss + a.unit_eps);
-    float *dst = (part == 0 ? a.q + (size_t)t * nq : part == 1 ? a.k + (size_t)t * nq : a.v + (size_t)t * nv) + (size_t)head * n;
+    float *dst = part == 0 ? a.q : part == 1 ? a.k : a.v;
+    const int row = part == 2 ? nv : nq;
 #pragma unroll
-    for (int i = 0; i < MIX_MAX_DIM / 64; ++i)
-        if (i * 64 + lane < n) dst[i * 64 + lane] = y[i] * f;
+    for (int t = 0; t < PREP_TOK; ++t) {
+        const float f = part == 2 ? 1.0f : (part == 0 ? a.q_scale : 1.0f) / sqrtf(wave_sum(ss[t]) + a.unit_eps);
+        if (t < nt) {
+#pragma unroll
+            for (int b = 0; b < CH; ++b)
+                if (b * 64 + lane < n) dst[(size_t)(t0 + t) * row + (size_t)head * n + b * 64 + lane] = y[b][t] * f;
+        }
+    }
 }
 
 int launch_delta_prep(lumen_ctx *ctx, const DeltaPrepArgs &a) {
     if (a.s <= 0) return LUMEN_OK;
-    const int units = 2 * a.kv_heads + a.heads + 1;
-    hipLaunchKernelGGL(delta_prep_kernel, dim3((unsigned)(((long)a.s * units + 3) / 4)), dim3(256), 0, ctx->stream, a, units);
+    const int units = 2 * a.kv_heads + a.heads + 1, widest = a.dim > a.vdim ? a.dim : a.vdim;
+    const long waves = (long)((a.s + PREP_TOK - 1) / PREP_TOK) * units;
+    const dim3 grid((unsigned)((waves + 3) / 4));
+#define PREP_LAUNCH(CH)                                                                                              \
+    do {                                                                                                             \
+        if (a.taps <= 4) hipLaunchKernelGGL((delta_prep_kernel<4, CH>), grid, dim3(256), 0, ctx->stream, a, units);  \
+        else hipLaunchKernelGGL((delta_prep_kernel<MIX_MAX_TAPS, CH>), grid, dim3(256), 0, ctx->stream, a, units);   \
+    } while (0)
+    if (widest <= 64) PREP_LAUNCH(1);
+    else if (widest <= 128) PREP_LAUNCH(2);
+    else PREP_LAUNCH(4);
+#undef PREP_LAUNCH
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
 }

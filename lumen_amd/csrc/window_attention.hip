@@ -64,6 +64,11 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
     if (n <= 0) return;
     const bool has_new = lo + n - 1 == pos;
     const float *kr = a.k_ring + (size_t)hk * a.cap * a.dpad, *vr = a.v_ring + (size_t)hk * a.cap * a.vpad;
+    const int slot_lo = lo % a.cap;
+    auto slot_of = [&](int key) {  // (a slice never wraps twice: it is no longer than the ring)
+        const int x = slot_lo + key;
+        return (size_t)(x >= a.cap ? x - a.cap : x);
+    };
 
     const int row0 = wave * 4 + (lane >> 4);  // this row's keys: row0, row0 + 32, ...
     v4f kb[U][DB];
@@ -71,7 +76,7 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
 #pragma unroll
         for (int i = 0; i < U; ++i) {
             const int key = min(row0 + (i0 + i) * (WD_WAVES * 4), n - 1);
-            const float *p = kr + (size_t)((lo + key) % a.cap) * a.dpad;
+            const float *p = kr + slot_of(key) * a.dpad;
 #pragma unroll
             for (int b = 0; b < DB; ++b) {
                 const int d = b * 64 + i16 * 4;
@@ -84,7 +89,7 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
     const int grp = tid / LV, d4 = (tid % LV) * 4;
     auto value_row = [&](int key) {
         v4f v = {0.f, 0.f, 0.f, 0.f};
-        if (key < n && d4 < a.vpad) v = *(const v4f *)(vr + (size_t)((lo + key) % a.cap) * a.vpad + d4);
+        if (key < n && d4 < a.vpad) v = *(const v4f *)(vr + slot_of(key) * a.vpad + d4);
         return v;
     };
     v4f vb[VA];
@@ -314,21 +319,37 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
     float m = -INFINITY, l = 0.f;
     const int j_first = max(0, a.pos + t0 - a.window + 1), j_last = a.pos + last;
     const int w_first = max(0, a.pos + tw - a.window + 1), w_last = a.pos + min(tw + 15, a.s - 1);  // of this wavefront
+    // The tile in front travels in registers while this one is worked on.  Positions past the last key and channels past
+    // the rows are clamped: the former get no weight, the latter meet zero queries or no output.
+    constexpr int PER = (WP_K * NB * 4 + 255) / 256;  // 16-byte pieces of K and of V per thread
+    v4f tk[PER], tv[PER];
+    auto fetch = [&](int j0, int slot0) {
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const int e = tid + i * 256;
+            int row = e / (nd * 4), x = slot0 + min(min(row, WP_K - 1), j_last - j0);
+            x = x >= a.cap ? x - a.cap : x;
+            tk[i] = *(const v4f *)(kr + (size_t)x * a.dpad + min((e % (nd * 4)) * 4, a.dpad - 4));
+            row = e / (nv * 4);
+            x = slot0 + min(min(row, WP_K - 1), j_last - j0);
+            x = x >= a.cap ? x - a.cap : x;
+            tv[i] = *(const v4f *)(vr + (size_t)x * a.vpad + min((e % (nv * 4)) * 4, a.vpad - 4));
+        }
+    };
+    int slot = j_first % a.cap;
+    fetch(j_first, slot);
     for (int j0 = j_first; j0 <= j_last; j0 += WP_K) {
         __syncthreads();
-        for (int e = tid; e < WP_K * nd * 4; e += 256) {
-            const int row = e / (nd * 4), d = (e % (nd * 4)) * 4;
-            v4f v = {0.f, 0.f, 0.f, 0.f};
-            if (j0 + row <= j_last && d < a.dpad) v = *(const v4f *)(kr + (size_t)((j0 + row) % a.cap) * a.dpad + d);
-            *(v4f *)(ks + row * kld + d) = v;
-        }
-        for (int e = tid; e < WP_K * nv * 4; e += 256) {
-            const int row = e / (nv * 4), d = (e % (nv * 4)) * 4;
-            v4f v = {0.f, 0.f, 0.f, 0.f};
-            if (j0 + row <= j_last && d < a.vpad) v = *(const v4f *)(vr + (size_t)((j0 + row) % a.cap) * a.vpad + d);
-            *(v4f *)(vs + row * vld + d) = v;
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const int e = tid + i * 256;
+            if (e < WP_K * nd * 4) *(v4f *)(ks + e / (nd * 4) * kld + e % (nd * 4) * 4) = tk[i];
+            if (e < WP_K * nv * 4) *(v4f *)(vs + e / (nv * 4) * vld + e % (nv * 4) * 4) = tv[i];
         }
         __syncthreads();
+        slot += WP_K;
+        while (slot >= a.cap) slot -= a.cap;
+        if (j0 + WP_K <= j_last) fetch(j0 + WP_K, slot);
         if (tw >= a.s || j0 > w_last || j0 + WP_K - 1 < w_first) continue;  // (uniform in the wavefront)
         v4f sc[2];
 #pragma unroll

@@ -15,8 +15,8 @@ OUT = os.path.join(HERE, "src", "ffi.rs")
 
 SCALARS = {"int": "c_int", "float": "c_float", "double": "f64", "size_t": "usize", "int32_t": "i32", "uint16_t": "u16",
            "int64_t": "i64", "uint64_t": "u64", "char": "c_char", "void": "c_void"}
-OPAQUE = ["lumen_ctx", "lumen_rope", "lumen_kv_cache", "lumen_llama"]
-STRUCTS = {"lumen_llama_config", "lumen_sampling"}
+OPAQUE = ["lumen_ctx", "lumen_rope", "lumen_kv_cache", "lumen_llama", "lumen_decoder_layer", "lumen_hybrid"]
+STRUCTS = {"lumen_llama_config", "lumen_sampling", "lumen_hybrid_config", "lumen_hybrid_layer"}
 
 
 def rust_type(ctype):

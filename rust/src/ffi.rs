@@ -7,6 +7,44 @@ use std::os::raw::{c_char, c_float, c_int, c_void};
 #[repr(C)] pub struct lumen_rope { _private: [u8; 0] }
 #[repr(C)] pub struct lumen_kv_cache { _private: [u8; 0] }
 #[repr(C)] pub struct lumen_llama { _private: [u8; 0] }
+#[repr(C)] pub struct lumen_decoder_layer { _private: [u8; 0] }
+#[repr(C)] pub struct lumen_hybrid { _private: [u8; 0] }
+
+#[repr(C)]
+#[derive(Clone, Copy, Debug)]
+pub struct lumen_hybrid_config {
+    pub vocab_size: c_int,
+    pub width: c_int,
+    pub num_layers: c_int,
+    pub loop_start: c_int,
+    pub loop_stop: c_int,
+    pub loop_times: c_int,
+    pub embed_scale: c_float,
+    pub norm_eps: c_float,
+    pub norm_offset: c_float,
+    pub residual_mult: c_float,
+    pub unit_eps: c_float,
+    pub max_seq_len: c_int,
+    pub max_chunk: c_int,
+    pub weight_dtype: c_int,
+}
+
+#[repr(C)]
+#[derive(Clone, Copy, Debug)]
+pub struct lumen_hybrid_layer {
+    pub mixer: c_int,
+    pub heads: c_int,
+    pub kv_heads: c_int,
+    pub dim: c_int,
+    pub vdim: c_int,
+    pub window: c_int,
+    pub scale: c_float,
+    pub softcap: c_float,
+    pub conv: c_int,
+    pub rank_lo: c_int,
+    pub rank_hi: c_int,
+    pub ff: c_int,
+}
 
 #[repr(C)]
 #[derive(Clone, Copy, Debug)]
