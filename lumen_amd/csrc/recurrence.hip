@@ -342,15 +342,20 @@ __global__ __launch_bounds__(256) void recurrence_chunk_kernel(RecurrenceArgs a,
             }
         }
     };
-    ChunkFrag<RT> fa, fb;  // the next chunk's operands travel while this one is worked on
-    load(fa, 0);
-    for (int n = 0; n < chunks; n += 2) {
-        if (n + 1 < chunks) load(fb, n + 1);
-        work(fa, n);
-        if (n + 1 < chunks) {
-            if (n + 2 < chunks) load(fa, n + 2);
-            work(fb, n + 1);
-        }
+    // the operands of the next two chunks travel while one is worked on (they come from beyond L2: one chunk's work is
+    // shorter than that trip); requests past the end repeat the last chunk
+    ChunkFrag<RT> f0, f1, f2;
+    load(f0, 0);
+    load(f1, min(1, chunks - 1));
+    for (int n = 0; n < chunks; n += 3) {
+        load(f2, min(n + 2, chunks - 1));
+        work(f0, n);
+        if (n + 1 >= chunks) break;
+        load(f0, min(n + 3, chunks - 1));
+        work(f1, n + 1);
+        if (n + 2 >= chunks) break;
+        load(f1, min(n + 4, chunks - 1));
+        work(f2, n + 2);
     }
     if (live)
 #pragma unroll

@@ -9,9 +9,12 @@ typedef float v4f __attribute__((ext_vector_type(4)));
 
 // tanh by the continued fraction x / (1 + x^2 / (3 + x^2 / (5 + x^2 / (7 + x^2 / 9)))) up to 0.9 (truncation below
 // 2.4e-8 there), by 1 - 2 / (e^{2 |x|} + 1) beyond: the absolute error stays small against x, which a soft cap multiplies.
-__device__ __forceinline__ float tanh_w(float x) {
+__device__ __forceinline__ float tanh_near(float x) {
     const float y = x * x;
-    const float near = x * fmaf(y, y + 105.0f, 945.0f) * __builtin_amdgcn_rcpf(fmaf(y, fmaf(y, 15.0f, 420.0f), 945.0f));
+    return x * fmaf(y, y + 105.0f, 945.0f) * __builtin_amdgcn_rcpf(fmaf(y, fmaf(y, 15.0f, 420.0f), 945.0f));
+}
+__device__ __forceinline__ float tanh_w(float x) {
+    const float y = x * x, near = tanh_near(x);
     const float far = 1.0f - 2.0f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(2.88539008177792681f * fabsf(x)) + 1.0f);
     return y <= 0.81f ? near : copysignf(far, x);
 }
@@ -28,8 +31,11 @@ struct ScoreShape {
     __device__ float operator()(float dot, int dist) const {
         float s = in * dot;
         if (out > 0.f) s = out * tanh_w(s);
-        return fmaf(-r1, __builtin_amdgcn_logf(fmaf(r2, (float)dist, 1.0f)), s);
+        return less_bias(s, dist);
     }
+    // the same in steps, for a wavefront that looks at its scores together
+    __device__ float capped_near(float x) const { return out * tanh_near(x); }
+    __device__ float less_bias(float s, int dist) const { return fmaf(-r1, __builtin_amdgcn_logf(fmaf(r2, (float)dist, 1.0f)), s); }
 };
 
 __device__ __forceinline__ float gate_w(float z, int act) {
@@ -289,8 +295,9 @@ __global__ __launch_bounds__(256) void window_append_kernel(WindowAttnArgs a) {
 // are laid out for.
 #define WP_Q 64
 #define WP_K 32
-template <int NB>
-__global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, int nd, int nv) {
+template <int NB, bool FULL>
+__global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, int nd_, int nv_) {
+    const int nd = FULL ? NB : nd_, nv = FULL ? NB : nv_;
     LUMEN_DYNAMIC_LDS(float, lds);
     const int kld = nd * 16 + 4, vld = nv * 16 + 4;
     float *ks = lds, *vs = lds + WP_K * kld;
@@ -366,14 +373,49 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
                     for (int u = 0; u < 2; ++u) sc[u] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[u][e], qf[b][e], sc[u], 0, 0, 0);
             }
         float mx = m;
+        const int dist0 = i - j0 - g * 4;
+        if (shape.out > 0.f) {
+            // (most scores stay well below the cap: the far form of tanh is left out where the whole wavefront does)
+            bool far = false;
+#pragma unroll
+            for (int u = 0; u < 2; ++u)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    sc[u][r] *= shape.in;
+                    far |= fabsf(sc[u][r]) > 0.9f;
+                }
+            if (__any(far)) {
+#pragma unroll
+                for (int u = 0; u < 2; ++u)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) sc[u][r] = shape.out * tanh_w(sc[u][r]);
+            } else {
+#pragma unroll
+                for (int u = 0; u < 2; ++u)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) sc[u][r] = shape.capped_near(sc[u][r]);
+            }
+        } else {
+            sc[0] *= shape.in;
+            sc[1] *= shape.in;
+        }
 #pragma unroll
         for (int u = 0; u < 2; ++u)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int dist = i - (j0 + u * 16 + g * 4 + r);
-                sc[u][r] = dist >= 0 && dist < a.window ? shape(sc[u][r], dist) : -INFINITY;
-                mx = fmaxf(mx, sc[u][r]);
-            }
+            for (int r = 0; r < 4; ++r) sc[u][r] = shape.less_bias(sc[u][r], dist0 - (u * 16 + r));
+        if (j0 + WP_K - 1 > a.pos + tw || j0 <= w_last - a.window) {  // (a tile every query of the wavefront sees whole needs no mask)
+#pragma unroll
+            for (int u = 0; u < 2; ++u)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int dist = dist0 - (u * 16 + r);
+                    sc[u][r] = dist >= 0 && dist < a.window ? sc[u][r] : -INFINITY;
+                }
+        }
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) mx = fmaxf(mx, sc[u][r]);
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
         mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
         const float base = mx > -INFINITY ? mx : 0.f;  // (a query that has seen nothing yet keeps zero weights)
@@ -388,15 +430,15 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
                 l += sc[u][r];
             }
 #pragma unroll
-        for (int b = 0; b < NB; ++b)
-            if (b < nv) {
-                acc[b] *= f;
+        for (int b = 0; b < NB; ++b) acc[b] *= f;
 #pragma unroll
-                for (int u = 0; u < 2; ++u)
+        for (int u = 0; u < 2; ++u)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r)
+            for (int r = 0; r < 4; ++r)
+#pragma unroll
+                for (int b = 0; b < NB; ++b)  // (accumulators take turns: none waits for its own last product)
+                    if (b < nv)
                         acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(vs[(u * 16 + g * 4 + r) * vld + b * 16 + c], sc[u][r], acc[b], 0, 0, 0);
-            }
     }
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
@@ -423,16 +465,22 @@ int launch_window_attn_prefill(lumen_ctx *ctx, const WindowAttnArgs &a) {
     const size_t lds = (size_t)WP_K * ((nd + nv) * 16 + 8) * sizeof(float);
     const dim3 grid((a.s + WP_Q - 1) / WP_Q, a.heads);
     const int nb = nd > nv ? nd : nv;
-#define WP_LAUNCH(NB)                                                                                                         \
-    do {                                                                                                                      \
-        if (lds > 64 * 1024)                                                                                                  \
-            HIP_TRY(hipFuncSetAttribute((const void *)window_prefill_kernel<NB>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); \
-        hipLaunchKernelGGL(window_prefill_kernel<NB>, grid, dim3(256), lds, ctx->stream, a, nd, nv);                          \
+#define WP_LAUNCH_F(NB, FULL)                                                                                                       \
+    do {                                                                                                                            \
+        if (lds > 64 * 1024)                                                                                                        \
+            HIP_TRY(hipFuncSetAttribute((const void *)window_prefill_kernel<NB, FULL>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); \
+        hipLaunchKernelGGL((window_prefill_kernel<NB, FULL>), grid, dim3(256), lds, ctx->stream, a, nd, nv);                        \
+    } while (0)
+#define WP_LAUNCH(NB)                                    \
+    do {                                                 \
+        if (nd == NB && nv == NB) WP_LAUNCH_F(NB, true); \
+        else WP_LAUNCH_F(NB, false);                     \
     } while (0)
     if (nb <= 4) WP_LAUNCH(4);
     else if (nb <= 8) WP_LAUNCH(8);
     else WP_LAUNCH(16);
 #undef WP_LAUNCH
+#undef WP_LAUNCH_F
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
 }

@@ -81,6 +81,12 @@ static inline int emu_update_dpp(int src, int ctrl) {
 static inline int emu_readlane(int v, int lane) { return (int)emu::wave_exchange((uint32_t)v, lane); }
 #define __builtin_amdgcn_readlane(v, lane) emu_readlane((v), (lane))
 
+static inline int __any(int pred) {
+    int any = 0;
+    for (int l = 0; l < 64; ++l) any |= (int)emu::wave_exchange((uint32_t)(pred != 0), l);
+    return any;
+}
+
 static inline float __uint_as_float(unsigned u) { return emu_bits_to<float>(u); }
 static inline unsigned __float_as_uint(float f) { return emu_bits_of(f); }
 static inline int __float_as_int(float f) { return (int)emu_bits_of(f); }
