@@ -263,84 +263,97 @@ struct ChunkFrag {
     float v[4];
 };
 
-// Workgroup = 16 columns of one head; its four wavefronts hold a quarter of the key rows each (RT tiles of 16), their
-// partial products meet in LDS, everything after that is done by each wavefront for itself.  Operands: lane (c, g) gives
-// A[c][.] and B[.][c] for the four contraction indices 4 g + r of step r; accumulator r is row 4 g + r, column c -- so an
-// accumulator tile is the B operand of the next product as it stands.
+// Workgroup = 16 columns of one head; its four wavefronts hold a quarter of the key rows each (RT tiles of 16).  Operands:
+// lane (c, g) gives A[c][.] and B[.][c] for the four contraction indices 4 g + r of step r; accumulator r is row 4 g + r,
+// column c -- so an accumulator tile is the B operand of the next product as it stands.  The wavefronts' partial K~ S meet
+// in LDS once per chunk; their partial outputs (a quarter of Q~ S and of B U each) ride along with the NEXT chunk's
+// meeting, and each wavefront then writes a quarter of the finished rows.
 template <int KIND, int RT>
 __global__ __launch_bounds__(256) void recurrence_chunk_kernel(RecurrenceArgs a, float *ws_base, int chunks) {
     constexpr int DP = RT * 64;
-    __shared__ float red[2][4][2][4][64];
+    __shared__ float red[2][2][4][4][64];  // [parity][K~ S, output][wavefront][r][lane]
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
-    const int h = blockIdx.x, col = blockIdx.y * 16 + c, Dv = a.vdim;
+    const int h = blockIdx.x, col = blockIdx.y * 16 + c, Dv = a.vdim, T = a.s;
     const bool live = col < Dv;
     float *Sg = a.state + ((size_t)h * Dv + (live ? col : 0)) * DP + wave * RT * 16 + g * 4;
     v4f S[RT];
 #pragma unroll
     for (int i = 0; i < RT; ++i) S[i] = *(const v4f *)(Sg + i * 16);
+    // lane offsets from a chunk's (uniform) base pointers
+    const unsigned d0 = wave * RT * 16, off_q = c * DP + d0 + g * 4, off_kh = (d0 + c) * REC_CHUNK + g * 4, off_gc = d0 + g * 4, off_t = c * REC_CHUNK + g * 4;
+    const unsigned colc = h * Dv + min(col, Dv - 1), vs = a.v_stride;
+    unsigned off_v[4], off_v_last[4];  // ... of the last chunk, whose tokens may end early: clamped, not skipped (a load behind a
+                             // branch would make the wavefront wait for all that are in flight)
+    const int t_last = (chunks - 1) * REC_CHUNK;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        off_v[r] = (unsigned)(g * 4 + r) * vs + colc;
+        off_v_last[r] = (unsigned)(min(t_last + g * 4 + r, T - 1) - t_last) * vs + colc;
+    }
+    const float *wsh = ws_base + (size_t)h * chunks * rec_ws_floats(DP);
     auto load = [&](ChunkFrag<RT> &f, int n) {
-        const ChunkWs w(ws_base + ((size_t)h * chunks + n) * rec_ws_floats(DP), DP);
-        const int d0 = wave * RT * 16;
+        const ChunkWs w(const_cast<float *>(wsh) + (size_t)n * rec_ws_floats(DP), DP);
 #pragma unroll
         for (int i = 0; i < RT; ++i) {
-            f.qt[i] = *(const v4f *)(w.qt + c * DP + d0 + i * 16 + g * 4);
-            if (KIND == REC_DELTA) f.kt[i] = *(const v4f *)(w.kt + c * DP + d0 + i * 16 + g * 4);
-            f.kh[i] = *(const v4f *)(w.kh + (d0 + i * 16 + c) * REC_CHUNK + g * 4);
-            f.gc[i] = *(const v4f *)(w.gc + d0 + i * 16 + g * 4);
+            f.qt[i] = *(const v4f *)(w.qt + (off_q + i * 16));
+            if (KIND == REC_DELTA) f.kt[i] = *(const v4f *)(w.kt + (off_q + i * 16));
+            f.kh[i] = *(const v4f *)(w.kh + (off_kh + i * 16 * REC_CHUNK));
+            f.gc[i] = *(const v4f *)(w.gc + (off_gc + i * 16));
         }
-        if (KIND == REC_DELTA) f.t = *(const v4f *)(w.t + c * REC_CHUNK + g * 4);
-        f.b = *(const v4f *)(w.b + c * REC_CHUNK + g * 4);
+        if (KIND == REC_DELTA) f.t = *(const v4f *)(w.t + off_t);
+        f.b = *(const v4f *)(w.b + off_t);
+        const bool last = n == chunks - 1;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            // (clamped, not skipped: a load behind a branch would make the wavefront wait for all that are in flight)
-            const int t = min(n * REC_CHUNK + g * 4 + r, a.s - 1);
-            f.v[r] = a.v[(size_t)t * a.v_stride + h * Dv + min(col, Dv - 1)];
-        }
+        for (int r = 0; r < 4; ++r) f.v[r] = *(a.v + (size_t)n * REC_CHUNK * vs + (last ? off_v_last[r] : off_v[r]));
+    };
+    v4f O = {0.f, 0.f, 0.f, 0.f};  // this wavefront's part of the chunk before
+    auto put = [&](int what, int n, const v4f x) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) red[n & 1][what][wave][r][lane] = x[r];
+    };
+    auto sum = [&](int what, int n, int r) {
+        return (red[n & 1][what][0][r][lane] + red[n & 1][what][1][r][lane]) + (red[n & 1][what][2][r][lane] + red[n & 1][what][3][r][lane]);
+    };
+    auto write_out = [&](int n, float o) {  // row `wave` of each group of four tokens of chunk n
+        const int t = n * REC_CHUNK + g * 4 + wave;
+        if (live && t < T) a.out[(size_t)t * a.out_stride + h * Dv + col] = o;
     };
     auto work = [&](const ChunkFrag<RT> &f, int n) {
-        v4f P = {0.f, 0.f, 0.f, 0.f}, O = {0.f, 0.f, 0.f, 0.f};
+        v4f P = {0.f, 0.f, 0.f, 0.f}, Q = {0.f, 0.f, 0.f, 0.f};
+        put(1, n, O);
 #pragma unroll
         for (int i = 0; i < RT; ++i)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 if (KIND == REC_DELTA) P = __builtin_amdgcn_mfma_f32_16x16x4f32(f.kt[i][r], S[i][r], P, 0, 0, 0);
-                O = __builtin_amdgcn_mfma_f32_16x16x4f32(f.qt[i][r], S[i][r], O, 0, 0, 0);
+                Q = __builtin_amdgcn_mfma_f32_16x16x4f32(f.qt[i][r], S[i][r], Q, 0, 0, 0);
             }
-        float (*rd)[2][4][64] = red[n & 1];
+        if (KIND == REC_DELTA) put(0, n, P);
+        __syncthreads();  // (one per chunk: the other half of red is written before the next one)
+        v4f U = {0.f, 0.f, 0.f, 0.f}, R;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            if (KIND == REC_DELTA) rd[wave][0][r][lane] = P[r];
-            rd[wave][1][r][lane] = O[r];
+            R[r] = n * REC_CHUNK + g * 4 + r < T ? f.v[r] : 0.f;
+            if (KIND == REC_DELTA) R[r] -= sum(0, n, r);
         }
-        __syncthreads();  // (one per chunk: the other half of red is written before the next one)
-        v4f U = {0.f, 0.f, 0.f, 0.f};
         if (KIND == REC_DELTA) {
-            v4f R;
-#pragma unroll
-            for (int r = 0; r < 4; ++r) R[r] = (n * REC_CHUNK + g * 4 + r < a.s ? f.v[r] : 0.f) - ((rd[0][0][r][lane] + rd[1][0][r][lane]) + (rd[2][0][r][lane] + rd[3][0][r][lane]));
 #pragma unroll
             for (int r = 0; r < 4; ++r) U = __builtin_amdgcn_mfma_f32_16x16x4f32(f.t[r], R[r], U, 0, 0, 0);
         } else {
-#pragma unroll
-            for (int r = 0; r < 4; ++r) U[r] = n * REC_CHUNK + g * 4 + r < a.s ? f.v[r] : 0.f;
+            U = R;
         }
+        const float o_before = sum(1, n, wave);
 #pragma unroll
-        for (int i = 0; i < RT; ++i) {
-            S[i] *= f.gc[i];
+        for (int i = 0; i < RT; ++i) S[i] *= f.gc[i];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.kh[i][r], U[r], S[i], 0, 0, 0);
-        }
-        if (wave == (n & 3)) {  // the wavefronts take turns with the output
+        for (int r = 0; r < 4; ++r)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) O[r] = (rd[0][1][r][lane] + rd[1][1][r][lane]) + (rd[2][1][r][lane] + rd[3][1][r][lane]);
-#pragma unroll
-            for (int r = 0; r < 4; ++r) O = __builtin_amdgcn_mfma_f32_16x16x4f32(f.b[r], U[r], O, 0, 0, 0);
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = n * REC_CHUNK + g * 4 + r;
-                if (live && t < a.s) a.out[(size_t)t * a.out_stride + h * Dv + col] = O[r];
-            }
-        }
+            for (int i = 0; i < RT; ++i) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.kh[i][r], U[r], S[i], 0, 0, 0);
+        // (the quarter of B U that this wavefront adds: contraction step `wave`)
+        const float bw = wave == 0 ? f.b[0] : wave == 1 ? f.b[1] : wave == 2 ? f.b[2] : f.b[3];
+        const float uw = wave == 0 ? U[0] : wave == 1 ? U[1] : wave == 2 ? U[2] : U[3];
+        O = __builtin_amdgcn_mfma_f32_16x16x4f32(bw, uw, Q, 0, 0, 0);
+        if (n > 0) write_out(n - 1, o_before);
     };
     // the operands of the next two chunks travel while one is worked on (they come from beyond L2: one chunk's work is
     // shorter than that trip); requests past the end repeat the last chunk
@@ -357,6 +370,9 @@ __global__ __launch_bounds__(256) void recurrence_chunk_kernel(RecurrenceArgs a,
         load(f1, min(n + 4, chunks - 1));
         work(f2, n + 2);
     }
+    put(1, chunks, O);
+    __syncthreads();
+    write_out(chunks - 1, sum(1, chunks, wave));
     if (live)
 #pragma unroll
         for (int i = 0; i < RT; ++i) *(v4f *)(Sg + i * 16) = S[i];
