@@ -158,7 +158,7 @@ struct ChunkWs {  // one chunk of one head
 };
 
 template <int KIND, int KR>
-__global__ __launch_bounds__(256) void recurrence_chunk_prep_kernel(RecurrenceArgs a, float *ws_base) {
+__global__ __launch_bounds__(256) void recurrence_chunk_prep_kernel(RecurrenceArgs a, float *ws_base, int vec) {
     constexpr int DP = 16 * KR;
     __shared__ __align__(16) float qs[REC_CHUNK][DP], ks[REC_CHUNK][DP], gs[REC_CHUNK][DP];
     __shared__ float As[REC_CHUNK][REC_CHUNK + 1], bs[REC_CHUNK];
@@ -169,15 +169,34 @@ __global__ __launch_bounds__(256) void recurrence_chunk_prep_kernel(RecurrenceAr
     float q[KR], k[KR], g[KR], uk[KR];
     {   // (positions beyond the head or the sequence are clamped, so that all requests go out together)
         const size_t t = (size_t)min(t0 + s, a.s - 1);
+        const float *pq = a.q + t * a.q_stride + hk * D, *pk = a.k + t * a.k_stride + hk * D, *pz = a.z + t * a.z_stride + h * D;
+        const float *pb = a.bias + h * D, *pu = KIND == REC_WKV ? a.u + h * D : pb;
         float z[KR], bias[KR], u[KR];
+        if (vec) {  // rows of whole 16-byte pieces
 #pragma unroll
-        for (int i = 0; i < KR; ++i) {
-            const int c = min(i16 * KR + i, D - 1);
-            q[i] = a.q[t * a.q_stride + hk * D + c];
-            k[i] = a.k[t * a.k_stride + hk * D + c];
-            z[i] = a.z[t * a.z_stride + h * D + c];
-            bias[i] = a.bias[h * D + c];
-            u[i] = KIND == REC_WKV ? a.u[h * D + c] : 0.f;
+            for (int i = 0; i < KR; i += 4) {
+                const int c = min(i16 * KR + i, D - 4);
+                const v4f vq = *(const v4f *)(pq + c), vk = *(const v4f *)(pk + c), vz = *(const v4f *)(pz + c), vb = *(const v4f *)(pb + c),
+                          vu = *(const v4f *)(pu + c);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    q[i + e] = vq[e];
+                    k[i + e] = vk[e];
+                    z[i + e] = vz[e];
+                    bias[i + e] = vb[e];
+                    u[i + e] = vu[e];
+                }
+            }
+        } else {
+#pragma unroll
+            for (int i = 0; i < KR; ++i) {
+                const int c = min(i16 * KR + i, D - 1);
+                q[i] = pq[c];
+                k[i] = pk[c];
+                z[i] = pz[c];
+                bias[i] = pb[c];
+                u[i] = pu[c];
+            }
         }
 #pragma unroll
         for (int i = 0; i < KR; ++i) {
@@ -236,13 +255,18 @@ __global__ __launch_bounds__(256) void recurrence_chunk_prep_kernel(RecurrenceAr
         rq[i] = q[i] * (KIND == REC_DELTA ? inc : G[i]);
         rk[i] = k[i] * inc;
         G[i] = inc;
-        w.kh[(i16 * KR + i) * REC_CHUNK + s] = kr[i];
     }
     store_kr<KR>(w.qt + s * DP + i16 * KR, rq);
     if (KIND == REC_DELTA) store_kr<KR>(w.kt + s * DP + i16 * KR, rk);
     if (s == REC_CHUNK - 1) store_kr<KR>(w.gc + i16 * KR, G);
+    __syncthreads();  // (everyone is done with qs; As is complete)
+    store_kr<KR>(&qs[s][i16 * KR], kr);
+    __syncthreads();
+    for (int e = tid; e < DP * 4; e += 256) {  // K^ goes out transposed
+        const int d = e >> 2, s4 = (e & 3) * 4;
+        *(v4f *)(w.kh + d * REC_CHUNK + s4) = v4f{qs[s4][d], qs[s4 + 1][d], qs[s4 + 2][d], qs[s4 + 3][d]};
+    }
     if (KIND == REC_DELTA) {
-        __syncthreads();
         if (tid < REC_CHUNK) {  // column tid of T by forward substitution
             float x[REC_CHUNK];
 #pragma unroll
@@ -406,13 +430,15 @@ int launch_recurrence(lumen_ctx *ctx, const RecurrenceArgs &a) {
         // are a multiple of 8)
         const dim3 pgrid(chunks, a.heads), grid(a.heads, (a.vdim + 15) / 16);
         float *ws = ctx->mixer_ws;
+        const int vec = a.dim % 4 == 0 && a.q_stride % 4 == 0 && a.k_stride % 4 == 0 && a.z_stride % 4 == 0 &&
+                        (((uintptr_t)a.q | (uintptr_t)a.k | (uintptr_t)a.z | (uintptr_t)a.bias | (uintptr_t)a.u) & 15) == 0;
 #define REC_LAUNCH(KR)                                                                                                            \
     do {                                                                                                                          \
         if (a.kind == REC_WKV) {                                                                                                  \
-            hipLaunchKernelGGL((recurrence_chunk_prep_kernel<REC_WKV, KR>), pgrid, dim3(256), 0, ctx->stream, a, ws);             \
+            hipLaunchKernelGGL((recurrence_chunk_prep_kernel<REC_WKV, KR>), pgrid, dim3(256), 0, ctx->stream, a, ws, vec);        \
             hipLaunchKernelGGL((recurrence_chunk_kernel<REC_WKV, KR / 4>), grid, dim3(256), 0, ctx->stream, a, ws, chunks);       \
         } else {                                                                                                                  \
-            hipLaunchKernelGGL((recurrence_chunk_prep_kernel<REC_DELTA, KR>), pgrid, dim3(256), 0, ctx->stream, a, ws);           \
+            hipLaunchKernelGGL((recurrence_chunk_prep_kernel<REC_DELTA, KR>), pgrid, dim3(256), 0, ctx->stream, a, ws, vec);      \
             hipLaunchKernelGGL((recurrence_chunk_kernel<REC_DELTA, KR / 4>), grid, dim3(256), 0, ctx->stream, a, ws, chunks);     \
         }                                                                                                                         \
     } while (0)
