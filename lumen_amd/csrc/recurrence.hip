@@ -658,6 +658,20 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
     float S[NT][KR];
 #pragma unroll
     for (int n = 0; n < NT; ++n) load_kr<KR>(S[n], Sh + (size_t)min(n * RD_COLS + c0, Dv - 1) * DP);
+    // small things that are needed late, requested now (clamped where a thread has no use for them)
+    const int own_row = min(tid >> 2, D - 1), own_col = min(tid, Dv - 1);
+    const float bias0 = a.bias[h * D + own_row], gain0 = a.gain[(a.gain_shared ? 0 : (size_t)h * Dv) + own_col];
+    const float a_log = KIND == REC_DELTA ? a.a_log[h] : 0.f, b_raw = KIND == REC_DELTA ? a.proj[a.off_b + h] : 0.f;
+    float u[KR];
+#pragma unroll
+    for (int i = 0; i < KR; ++i) {
+        const int kc = i16 * KR + i;
+        u[i] = 0.f;
+        if (KIND == REC_WKV) {
+            u[i] = a.u[h * D + min(kc, D - 1)];
+            u[i] = kc < D ? u[i] : 0.f;
+        }
+    }
 
     for (int i = tid; i < a.r_lo; i += RD_THREADS) {
         const float x = a.proj[a.off_lo + i];
@@ -693,10 +707,21 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
             const float *w = a.taps_w + (size_t)ch * a.taps;
             const bool keeper = part == 2 || h % rep == 0;  // one workgroup leaves a shared channel's inputs
             float acc = 0.f;
-            for (int j = 0; j < keep; ++j) {
-                const float p = prev[(size_t)j * channels + ch];
-                acc = fmaf(w[j], p, acc);
-                if (keeper && j > 0) next[(size_t)(j - 1) * channels + ch] = p;
+            for (int j0 = 0; j0 < keep; j0 += 3) {  // (three earlier inputs and their weights per trip to memory)
+                float p[3], wj[3];
+#pragma unroll
+                for (int j = 0; j < 3; ++j) {
+                    const int jc = min(j0 + j, keep - 1);
+                    p[j] = prev[(size_t)jc * channels + ch];
+                    wj[j] = w[jc];
+                }
+#pragma unroll
+                for (int j = 0; j < 3; ++j) {
+                    if (j0 + j < keep) {
+                        acc = fmaf(wj[j], p[j], acc);
+                        if (keeper && j0 + j > 0) next[(size_t)(j0 + j - 1) * channels + ch] = p[j];
+                    }
+                }
             }
             if (keeper && keep > 0) next[(size_t)(keep - 1) * channels + ch] = x;
             acc = silu_r(fmaf(w[keep], x, acc));
@@ -704,7 +729,7 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
         }
     }
     __syncthreads();
-    const float decay_a = KIND == REC_DELTA ? expf(a.a_log[h]) : 0.f;
+    const float decay_a = KIND == REC_DELTA ? expf(a_log) : 0.f;
     if (KIND == REC_DELTA && wave < 2) {  // the sums of squares of q and of k
         const float *p = wave ? ks : qs;
         float ss = 0.f;
@@ -717,12 +742,12 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
         if (r0) lr_start(rc);
         const float z = lr.dot(rc < D ? lo : hi);
         if (lr_part == 0 && r < lr_rows) {
-            if (r < D) ws[r] = decay_r<KIND>(z, a.bias[h * D + r], decay_a);
+            if (r < D) ws[r] = decay_r<KIND>(z, r0 ? a.bias[h * D + r] : bias0, decay_a);
             else gs[r - D] = sigmoid_r(z);
         }
     }
     __syncthreads();
-    float q[KR], k[KR], w[KR], u[KR];
+    float q[KR], k[KR], w[KR];
     load_kr<KR>(q, qs + i16 * KR);
     load_kr<KR>(k, ks + i16 * KR);
     load_kr<KR>(w, ws + i16 * KR);
@@ -734,12 +759,7 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
             q[i] *= iq;
             k[i] *= ik;
         }
-        beta = sigmoid_r(a.proj[a.off_b + h]);
-    }
-#pragma unroll
-    for (int i = 0; i < KR; ++i) {
-        const int kc = i16 * KR + i;
-        u[i] = KIND == REC_WKV && kc < D ? a.u[h * D + kc] : 0.f;
+        beta = sigmoid_r(b_raw);
     }
     float ss = 0.f;
 #pragma unroll
@@ -761,8 +781,7 @@ __global__ __launch_bounds__(RD_THREADS) void recurrence_decode_kernel(Recurrenc
 #pragma unroll
     for (int i = 0; i < RD_WAVES; ++i) tot += red_o[i];
     const float inv = 1.0f / sqrtf(tot / (float)Dv + a.norm_eps);
-    const float *gain = a.gain + (a.gain_shared ? 0 : (size_t)h * Dv);
-    for (int c = tid; c < Dv; c += RD_THREADS) a.out[(size_t)h * Dv + c] = os[c] * inv * gain[c] * gs[c];
+    if (tid < Dv) a.out[(size_t)h * Dv + tid] = os[tid] * inv * gain0 * gs[tid];
 }
 
 int launch_recurrence_decode(lumen_ctx *ctx, const RecurrenceDecodeArgs &a) {

@@ -76,6 +76,8 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
         return (size_t)(x >= a.cap ? x - a.cap : x);
     };
 
+    // Every load is issued unconditionally, positions clamped: keys past the slice get no weight, channels past a row meet
+    // zero queries or no output.  (A load behind a condition would be waited for before the next one goes out.)
     const int row0 = wave * 4 + (lane >> 4);  // this row's keys: row0, row0 + 32, ...
     v4f kb[U][DB];
     auto fetch = [&](int i0) {
@@ -84,30 +86,34 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
             const int key = min(row0 + (i0 + i) * (WD_WAVES * 4), n - 1);
             const float *p = kr + slot_of(key) * a.dpad;
 #pragma unroll
-            for (int b = 0; b < DB; ++b) {
-                const int d = b * 64 + i16 * 4;
-                kb[i][b] = v4f{0.f, 0.f, 0.f, 0.f};
-                if (d < a.dpad) kb[i][b] = *(const v4f *)(p + d);
-            }
+            for (int b = 0; b < DB; ++b) kb[i][b] = *(const v4f *)(p + min(b * 64 + i16 * 4, a.dpad - 4));
         }
     };
     fetch(0);
     const int grp = tid / LV, d4 = (tid % LV) * 4;
-    auto value_row = [&](int key) {
-        v4f v = {0.f, 0.f, 0.f, 0.f};
-        if (key < n && d4 < a.vpad) v = *(const v4f *)(vr + slot_of(key) * a.vpad + d4);
-        return v;
-    };
+    auto value_row = [&](int key) { return *(const v4f *)(vr + slot_of(min(key, n - 1)) * a.vpad + min(d4, a.vpad - 4)); };
     v4f vb[VA];
 #pragma unroll
     for (int i = 0; i < VA; ++i) vb[i] = value_row(grp + i * GROUPS);
 
-    // queries and the new key, normalised over all heads together
+    // queries and the new key, normalised over all heads together; what each thread turns into the head's q, k and v is
+    // requested along with the values the sums are taken over
+    const int dq = min(tid, D - 1), dv = min(tid, Dv - 1);
+    const float own_q = a.q[h * D + dq], own_k = a.k[hk * D + dq], own_v = a.v[hk * Dv + dv];
+    const float gain_q = a.q_norm_w ? a.q_norm_w[h * D + dq] : 1.f, gain_k = a.k_norm_w ? a.k_norm_w[hk * D + dq] : 1.f;
+    const float gate = a.gate && a.slices == 1 ? a.gate[h * Dv + dv] : 0.f;
+    const float r1 = a.r1 ? a.r1[h] : 0.f, r2 = a.r1 ? a.r2[h] : 0.f;
     float sq = 0.f, sk = 0.f;
-    if (a.q_norm_w)
-        for (int i = tid; i < a.heads * D; i += WD_THREADS) sq = fmaf(a.q[i], a.q[i], sq);
-    if (a.k_norm_w && has_new)
-        for (int i = tid; i < a.kv_heads * D; i += WD_THREADS) sk = fmaf(a.k[i], a.k[i], sk);
+    if (a.q_norm_w) {
+        const int nq = a.heads * D;
+#pragma unroll 4
+        for (int i = tid; i < nq; i += WD_THREADS) sq = fmaf(a.q[i], a.q[i], sq);
+    }
+    if (a.k_norm_w && has_new) {
+        const int nk = a.kv_heads * D;
+#pragma unroll 4
+        for (int i = tid; i < nk; i += WD_THREADS) sk = fmaf(a.k[i], a.k[i], sk);
+    }
     sq = wave_sum(sq);
     sk = wave_sum(sk);
     if (lane == 0) {
@@ -121,28 +127,21 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
         sq += red[0][w];
         sk += red[1][w];
     }
-    const float iq = 1.0f / sqrtf(sq / (float)(a.heads * D) + a.norm_eps);
-    const float ik = 1.0f / sqrtf(sk / (float)(a.kv_heads * D) + a.norm_eps);
+    const float iq = a.q_norm_w ? 1.0f / sqrtf(sq / (float)(a.heads * D) + a.norm_eps) : 1.f;
+    const float ik = a.k_norm_w ? 1.0f / sqrtf(sk / (float)(a.kv_heads * D) + a.norm_eps) : 1.f;
     const bool writer = has_new && h % rep == 0;
     const size_t slot = (size_t)(pos % a.cap);
-    for (int d = tid; d < DB * 64; d += WD_THREADS) {
-        float q = 0.f, k = 0.f;
-        if (d < D) {
-            q = a.q[h * D + d];
-            if (a.q_norm_w) q = q * iq * a.q_norm_w[h * D + d];
-            if (has_new) {
-                k = a.k[hk * D + d];
-                if (a.k_norm_w) k = k * ik * a.k_norm_w[hk * D + d];
-            }
-        }
-        qs[d] = q;
-        kn[d] = k;
-        if (writer && d < a.dpad) a.k_ring[((size_t)hk * a.cap + slot) * a.dpad + d] = k;
+    static_assert(DB * 64 <= WD_THREADS && LV * 4 <= WD_THREADS, "one thread per channel");
+    if (tid < DB * 64) {
+        const float k = has_new && tid < D ? own_k * ik * gain_k : 0.f;
+        qs[tid] = tid < D ? own_q * iq * gain_q : 0.f;
+        kn[tid] = k;
+        if (writer && tid < a.dpad) a.k_ring[((size_t)hk * a.cap + slot) * a.dpad + tid] = k;
     }
-    for (int d = tid; d < LV * 4; d += WD_THREADS) {
-        const float v = has_new && d < Dv ? a.v[hk * Dv + d] : 0.f;
-        vn[d] = v;
-        if (writer && d < a.vpad) a.v_ring[((size_t)hk * a.cap + slot) * a.vpad + d] = v;
+    if (tid < LV * 4) {
+        const float v = has_new && tid < Dv ? own_v : 0.f;
+        vn[tid] = v;
+        if (writer && tid < a.vpad) a.v_ring[((size_t)hk * a.cap + slot) * a.vpad + tid] = v;
     }
     __syncthreads();
 
@@ -171,7 +170,7 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
         }
     }
     __syncthreads();
-    const ScoreShape shape(a.scale, a.softcap, a.r1 ? a.r1[h] : 0.f, a.r1 ? a.r2[h] : 0.f);
+    const ScoreShape shape(a.scale, a.softcap, r1, r2);
     float s = -INFINITY;
     if (tid < n) s = shape(sc[tid], pos - lo - tid);
     float m = wave_max(s);
@@ -202,12 +201,12 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
     for (int key = grp + VA * GROUPS; key < n; key += GROUPS) add(key, value_row(key));
     *(v4f *)(&ctx[grp][d4]) = acc;
     __syncthreads();
-    for (int d = tid; d < Dv; d += WD_THREADS) {
+    if (tid < Dv) {
         float o = 0.f;
 #pragma unroll 8
-        for (int g = 0; g < GROUPS; ++g) o += ctx[g][d];
-        if (a.slices > 1) a.part[((size_t)h * a.slices + slice) * (Dv + 2) + d] = o;
-        else a.out[h * Dv + d] = o / l * (a.gate ? gate_w(a.gate[h * Dv + d], a.gate_act) : 1.0f);
+        for (int g = 0; g < GROUPS; ++g) o += ctx[g][tid];
+        if (a.slices > 1) a.part[((size_t)h * a.slices + slice) * (Dv + 2) + tid] = o;
+        else a.out[h * Dv + tid] = o / l * (a.gate ? gate_w(gate, a.gate_act) : 1.0f);
     }
     if (a.slices > 1 && tid == 0) {
         float *pp = a.part + ((size_t)h * a.slices + slice) * (Dv + 2) + Dv;
