@@ -140,6 +140,6 @@ def pinavik_config(cfg, shape_of, max_seq_len, weight_dtype):
         layers.append(y)
     loop = cfg.get("loop") or {"start": 0, "stop": 0, "times": 0}
     return HybridConfig(cfg["vocab"], cfg["width"], layers, loop["start"], loop["stop"], loop["times"],
-                        embed_scale=cfg["embedding"]["scale"], norm_eps=cfg["norm"]["eps"], norm_offset=1.0,
-                        residual_mult=cfg["residual_mult"], unit_eps=1e-6, max_seq_len=max_seq_len,
+                        embed_scale=cfg.get("embedding", {}).get("scale", 1.0), norm_eps=cfg["norm"]["eps"], norm_offset=1.0,
+                        residual_mult=cfg.get("residual_mult", 1.0), unit_eps=1e-6, max_seq_len=max_seq_len,
                         weight_dtype=weight_dtype)
