@@ -391,11 +391,13 @@ int lumen_decoder_layer_decode_f32(lumen_decoder_layer *layer, lumen_kv_cache *c
 
 /* ------------------------------------------------- layered hybrid decoder
  * A decoder-only model whose layers differ in their sequence mixer (no counterpart in the reference; beside
- * lumen_llama_*, with the same loader, sampler, turn loop, decode graph and products).  x = embed[token] * embed_scale;
- * a layer is x += residual_mult * mixer(norm1(x)), then x += residual_mult * ff(norm2(x)); norms are RMS norms whose
- * stored weight has norm_offset added (1: weights stored around zero); logits = head final_norm(x).
+ * lumen_llama_*, with the same loader, sampler, turn loop, decode graph and products).  x = embed[token] * embed_scale,
+ * plus pos[position] with max_positions > 0; a layer is x += residual_mult * mixer(norm1(x)), then x += residual_mult *
+ * ff(norm2(x)), or, with residual_gate, x += sigmoid(rg1 norm1(x) + rg1.b) * mixer(norm1(x)) and likewise rg2; norms are RMS norms
+ * whose stored weight has norm_offset added (1: weights stored around zero), or Dynamic Tanh, tanh(alpha x) w + b; logits = head
+ * final_norm(x), squashed by logit_softcap tanh(. / logit_softcap) where that is set.
  * With loop_times > 0 layers [loop_start, loop_stop) run loop_times times in a row on the same weights, each pass with
- * its own state; before pass t, x = W_in [x; x0] + step[t], x0 being the embedding output.
+ * its own state; before pass t, x = W_in [x; x0] + step[t], x0 being the embedding output, or (LUMEN_LOOP_ADD) x += step[t].
  * Mixers (h: the mixer's input; tensors "l<i>.mix.<name>"):
  *   WINDOW_ATTENTION  q, k, v, g projections; RMSNorm of the whole q and of the whole k (q.norm, k.norm); score =
  *                     softcap tanh(q.k scale / softcap) (softcap 0: plain) - r1 ln(1 + r2 distance); softmax over the
@@ -405,23 +407,51 @@ int lumen_decoder_layer_decode_f32(lumen_decoder_layer *layer, lumen_kv_cache *c
  *   CHANNEL_DELTA     causal convolution (conv taps) + SiLU on q, k, v; unit q, k per head (unit_eps under the root, q also
  *                     times dim^-1/2); decay exp(-exp(A_log) softplus(a2 a1 h + dt_bias)) per key channel; S <- g S;
  *                     S <- S + k (sigmoid(b) (v - S^T k))^T; o = S^T q; RMSNorm per head, times norm, times sigmoid(g2 g1 h); o
- * ff > 0: feed-forward mlp.down(PolyNorm(mlp.up(.))) with mlp.act = {a, b, c, e}: a N(z) + b N(z^2) + c N(z^3) + e.
+ *   GENERAL_DELTA     r, k, v projections; decay w = exp(-e^{-1/2} sigmoid(w2 tanh(w1 h) + w0)) and removal rate a = sigmoid(a h + a.b) per
+ *                     key channel; unit key u (unit_eps under the root); S <- diag(w) S - (a u) (u^T S) + k v^T, both terms reading the
+ *                     old S; o = S^T r; RMSNorm per head, times norm, times sigmoid(g h); o
+ *   PARALLEL          half the sum of two mixers of the same h, each RMS-normed over the width with its weight "left.out" / "right.out":
+ *                     left.*: attention over all positions, score = (q.k) scale temp[head] + rel[bucket(distance)][head] (the lower half of
+ *                     the bias_rows rows one per distance, the upper half a logarithmic scale up to bias_max), exp(sink[head]) in
+ *                     the softmax's denominator, head outputs times sigmoid(g h) (one per head), o
+ *                     right.*: matrix memory of mem_heads heads: log gates i = cap tanh((i h + i.b) / cap), f = log sigmoid(cap tanh((f h + f.b) /
+ *                     cap)); m' = max(f + m, i) from m = 0; S <- e^{f + m - m'} S + e^{i - m'} k v^T, n likewise with k alone; q times
+ *                     mem_dim^-1/2; S^T q / (max(|n.q|, e^{-m'}) + 1e-6); RMSNorm per head, times norm, times sigmoid(g h), o
+ * ff > 0: a feed-forward.  POLYNORM: mlp.down(PolyNorm(mlp.up(.))) with mlp.act = {a, b, c, e}: a N(z) + b N(z^2) + c N(z^3) + e.  GELU:
+ * mlp.down(z Phi(z)).  EXPERTS: scores sigmoid(mlp.router h); of the `keep` best of `groups` groups (a group's score: its two best)
+ * the `top` best experts, weights s / sum s * router_scale; expert e: down (min(g, limit) sigmoid(1.702 min(g, limit))
+ * (clamp(u, +-limit) + 1)) of g = mlp.e<e>.gate h, u = mlp.e<e>.up h.
  * The state between steps -- rolling key / value stores of window - 1 + max_chunk positions, recurrent matrices in f32,
  * convolution and token-shift inputs -- belongs to the model's one live sequence; lumen_hybrid_reset gives it back.
  * Heads up to 256 wide, inner sizes up to 16384, up to 16 taps; sizes need not be multiples of anything. */
 #define LUMEN_MIXER_WINDOW_ATTENTION 0
 #define LUMEN_MIXER_WKV 1
 #define LUMEN_MIXER_CHANNEL_DELTA 2
+#define LUMEN_MIXER_GENERAL_DELTA 3
+#define LUMEN_MIXER_PARALLEL 4
+#define LUMEN_FF_POLYNORM 0
+#define LUMEN_FF_GELU 1
+#define LUMEN_FF_EXPERTS 2
+#define LUMEN_NORM_RMS 0
+#define LUMEN_NORM_DYT 1
+#define LUMEN_LOOP_MIX 0
+#define LUMEN_LOOP_ADD 1
 typedef struct lumen_hybrid lumen_hybrid;
 typedef struct {
     int mixer;                       /* LUMEN_MIXER_* */
-    int heads, kv_heads, dim, vdim;  /* WKV: kv_heads = heads, vdim = dim */
+    int heads, kv_heads, dim, vdim;  /* WKV, GENERAL_DELTA: kv_heads = heads, vdim = dim; PARALLEL: the attention's */
     int window;                      /* attention: positions a query sees, itself included; 0: all */
     float scale, softcap;            /* attention */
     int conv;                        /* CHANNEL_DELTA: taps of the causal convolution */
-    int rank_lo;                     /* inner size of the decay's low-rank product (WKV w1 / w2, CHANNEL_DELTA a1 / a2) */
+    int rank_lo;                     /* inner size of the decay's low-rank product (WKV, GENERAL_DELTA w1 / w2, CHANNEL_DELTA a1 / a2) */
     int rank_hi;                     /* CHANNEL_DELTA: inner size of the gate's (g1 / g2) */
-    int ff;                          /* feed-forward width, 0: none */
+    int ff;                          /* feed-forward width (of an expert), 0: none */
+    int ff_kind;                     /* LUMEN_FF_* */
+    int bias_rows, bias_max;         /* PARALLEL: rows of the distance bias, distance its last row is reached at */
+    int mem_heads, mem_dim, mem_vdim;  /* PARALLEL: the matrix memory's heads */
+    float gate_cap;
+    int experts, top, groups, keep;  /* EXPERTS */
+    float router_scale, limit;
 } lumen_hybrid_layer;
 typedef struct {
     int vocab_size, width, num_layers;
@@ -430,6 +460,9 @@ typedef struct {
     int max_seq_len;                 /* tokens a sequence may hold */
     int max_chunk;                   /* longest piece a prompt is run in (0: 2048) */
     int weight_dtype;                /* LUMEN_DTYPE_F32 or _BF16: storage of the matrices; arithmetic is f32 either way */
+    int norm_kind, loop_kind;        /* LUMEN_NORM_*, LUMEN_LOOP_* */
+    int residual_gate, max_positions;
+    float logit_softcap;             /* 0: none */
 } lumen_hybrid_config;
 int lumen_hybrid_create(lumen_ctx *ctx, const lumen_hybrid_config *cfg, const lumen_hybrid_layer *layers, lumen_hybrid **out);
 int lumen_hybrid_destroy(lumen_hybrid *model);
@@ -447,7 +480,8 @@ int lumen_hybrid_decode_greedy(lumen_hybrid *model, int first_id, int n, int32_t
 int lumen_hybrid_generate_turn(lumen_hybrid *model, const int32_t *new_tokens, int n_new, const int32_t *history, int n_history,
                                const lumen_sampling *sampling, const int32_t *stop_ids, int n_stop, int32_t *out_ids, int out_cap, int *n_out);
 /* n greedy steps with every product and mixer launch between two HIP events.  Classes: 0 embedding, 1 loop input, 2 / 3
- * attention projections / mixer, 4 / 5 WKV, 6 / 7 CHANNEL_DELTA, 8 output projection, 9 up, 10 down, 11 head. */
+ * attention projections / mixer, 4 / 5 WKV, 6 / 7 CHANNEL_DELTA, 8 output projection, 9 up, 10 down, 11 head, 12 / 13
+ * GENERAL_DELTA, 14 PARALLEL projections, 15 matrix memory, 16 gated sum of a pair, 17 / 18 experts' gate|up / down. */
 int lumen_hybrid_decode_profile(lumen_hybrid *model, int first_id, int n, double *ms_sum_out, int *count_out, int n_classes);
 int lumen_hybrid_set_decode_mode(lumen_hybrid *model, int mode);
 int lumen_hybrid_reset(lumen_hybrid *model);

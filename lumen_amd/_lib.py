@@ -44,14 +44,18 @@ class LlamaConfigStruct(C.Structure):
 class HybridLayerStruct(C.Structure):  # lumen_hybrid_layer
     _fields_ = [("mixer", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int),
                 ("window", C.c_int), ("scale", C.c_float), ("softcap", C.c_float), ("conv", C.c_int),
-                ("rank_lo", C.c_int), ("rank_hi", C.c_int), ("ff", C.c_int)]
+                ("rank_lo", C.c_int), ("rank_hi", C.c_int), ("ff", C.c_int), ("ff_kind", C.c_int), ("bias_rows", C.c_int),
+                ("bias_max", C.c_int), ("mem_heads", C.c_int), ("mem_dim", C.c_int), ("mem_vdim", C.c_int), ("gate_cap", C.c_float),
+                ("experts", C.c_int), ("top", C.c_int), ("groups", C.c_int), ("keep", C.c_int), ("router_scale", C.c_float),
+                ("limit", C.c_float)]
 
 
 class HybridConfigStruct(C.Structure):  # lumen_hybrid_config
     _fields_ = [("vocab_size", C.c_int), ("width", C.c_int), ("num_layers", C.c_int), ("loop_start", C.c_int),
                 ("loop_stop", C.c_int), ("loop_times", C.c_int), ("embed_scale", C.c_float), ("norm_eps", C.c_float),
                 ("norm_offset", C.c_float), ("residual_mult", C.c_float), ("unit_eps", C.c_float),
-                ("max_seq_len", C.c_int), ("max_chunk", C.c_int), ("weight_dtype", C.c_int)]
+                ("max_seq_len", C.c_int), ("max_chunk", C.c_int), ("weight_dtype", C.c_int), ("norm_kind", C.c_int),
+                ("loop_kind", C.c_int), ("residual_gate", C.c_int), ("max_positions", C.c_int), ("logit_softcap", C.c_float)]
 
 
 _vp, _f, _i = C.c_void_p, C.c_float, C.c_int

@@ -53,6 +53,7 @@ extern "C" int lumen_ctx_create(int device, lumen_ctx **out) {
     lumen_warm_mlp_chain(c->stream);
     lumen_warm_prefill_attention(c->stream);
     lumen_warm_recurrence(c->stream);
+    lumen_warm_experts(c->stream);
     lumen_warm_window_attention(c->stream);
     HIP_TRY(hipStreamSynchronize(c->stream));
     {   // the runtime sets up its device-to-host copy path over the first few copies of a process: have them here

@@ -95,7 +95,7 @@ int launch_rmsnorm(lumen_ctx *ctx, const float *x, const float *w, float *out, i
 }
 
 // -------------------------------------------------------------- elementwise
-enum { OP_SILU, OP_ADD, OP_MUL, OP_SWIGLU, OP_COPY, OP_TANH };
+enum { OP_SILU, OP_ADD, OP_MUL, OP_SWIGLU, OP_COPY, OP_TANH, OP_GELU };
 
 template <int OP>
 __global__ __launch_bounds__(256) void ew_kernel(const float *__restrict__ a, const float *__restrict__ b,
@@ -111,6 +111,8 @@ __global__ __launch_bounds__(256) void ew_kernel(const float *__restrict__ a, co
             r = x;
         } else if (OP == OP_TANH) {
             r = tanhf(x);
+        } else if (OP == OP_GELU) {
+            r = 0.5f * x * (1.0f + erff(x * 0.70710678118654752f));
         } else if (OP == OP_ADD) {
             r = x + b[i];
         } else if (OP == OP_MUL) {
@@ -141,6 +143,126 @@ int launch_swiglu(lumen_ctx *ctx, const float *g, const float *u, float *out, si
 static int launch_copy(lumen_ctx *ctx, const float *x, float *out, size_t n) { return launch_ew<OP_COPY>(ctx, x, x, out, n); }
 
 int launch_tanh(lumen_ctx *ctx, const float *x, float *out, size_t n) { return launch_ew<OP_TANH>(ctx, x, x, out, n); }
+
+int launch_gelu(lumen_ctx *ctx, const float *x, float *out, size_t n) { return launch_ew<OP_GELU>(ctx, x, x, out, n); }
+
+__global__ __launch_bounds__(256) void softcap_kernel(float *x, float cap, size_t n) {
+    const size_t stride = (size_t)gridDim.x * blockDim.x;
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += stride) x[i] = cap * tanhf(x[i] / cap);
+}
+int launch_softcap(lumen_ctx *ctx, float *x, float cap, size_t n) {
+    if (n == 0) return LUMEN_OK;
+    const size_t blocks = (n + 255) / 256, most = (size_t)ctx->num_cus * 16;
+    hipLaunchKernelGGL(softcap_kernel, dim3((unsigned)(blocks < most ? blocks : most)), dim3(256), 0, ctx->stream, x, cap, n);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+// ----------------------------------------------------- Dynamic Tanh, gated residual
+__device__ __forceinline__ v4f dyt_row4(const v4f x, float alpha, const v4f g, const v4f b) {
+    return v4f{fmaf(tanhf(alpha * x.x), g.x, b.x), fmaf(tanhf(alpha * x.y), g.y, b.y), fmaf(tanhf(alpha * x.z), g.z, b.z),
+               fmaf(tanhf(alpha * x.w), g.w, b.w)};
+}
+__device__ __forceinline__ float sigmoid_e(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+__global__ __launch_bounds__(256) void dyt_kernel(const float *__restrict__ x, const float *__restrict__ alpha, const float *__restrict__ w,
+                                                  const float *__restrict__ b, float *__restrict__ out, int dim) {
+    const float al = *alpha;
+    const size_t base = (size_t)blockIdx.x * dim;
+    if (dim % 4 == 0) {
+        for (int i = threadIdx.x * 4; i < dim; i += 1024)
+            *(v4f *)(out + base + i) = dyt_row4(*(const v4f *)(x + base + i), al, *(const v4f *)(w + i), *(const v4f *)(b + i));
+    } else {
+        for (int i = threadIdx.x; i < dim; i += 256) out[base + i] = fmaf(tanhf(al * x[base + i]), w[i], b[i]);
+    }
+}
+int launch_dyt(lumen_ctx *ctx, const float *x, const float *alpha, const float *w, const float *b, float *out, int rows, int dim) {
+    if (rows <= 0) return LUMEN_OK;
+    hipLaunchKernelGGL(dyt_kernel, dim3(rows), dim3(256), 0, ctx->stream, x, alpha, w, b, out, dim);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+// One workgroup per row of up to 4 * blockDim * GR_VPT elements: everything a thread needs is requested at once and stays
+// in registers between the sums of squares and the result.
+#define GR_VPT 4
+__global__ __launch_bounds__(1024) void gated_residual_kernel(GatedResidualArgs a) {
+    __shared__ float red[2][16];
+    const int row = blockIdx.x, tid = threadIdx.x, nt = blockDim.x, waves = nt >> 6, W = a.dim;
+    const size_t base = (size_t)row * W;
+    v4f y[GR_VPT], y2[GR_VPT];
+    float s1 = 0.f, s2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < GR_VPT; ++i) {
+        const int k = (tid + i * nt) * 4;
+        y[i] = y2[i] = v4f{0.f, 0.f, 0.f, 0.f};
+        if (k < W) {
+            if (a.top > 0) {
+                const size_t first = (size_t)row * a.top;
+                for (int j = 0; j < a.top; ++j) {
+                    const float f = a.sel_w[first + j];
+                    const v4f v = *(const v4f *)(a.y + (first + j) * W + k);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) y[i][e] = fmaf(f, v[e], y[i][e]);
+                }
+            } else {
+                y[i] = *(const v4f *)(a.y + base + k);
+            }
+            if (a.y2) {
+                y2[i] = *(const v4f *)(a.y2 + base + k);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    s1 = fmaf(y[i][e], y[i][e], s1);
+                    s2 = fmaf(y2[i][e], y2[i][e], s2);
+                }
+            }
+        }
+    }
+    float i1 = 0.f, i2 = 0.f;
+    if (a.y2) {
+        s1 = wave_sum(s1);
+        s2 = wave_sum(s2);
+        if ((tid & 63) == 0) {
+            red[0][tid >> 6] = s1;
+            red[1][tid >> 6] = s2;
+        }
+        __syncthreads();
+        s1 = s2 = 0.f;
+        for (int w = 0; w < waves; ++w) {
+            s1 += red[0][w];
+            s2 += red[1][w];
+        }
+        i1 = a.pair_scale / sqrtf(s1 / (float)a.width + a.eps);
+        i2 = a.pair_scale / sqrtf(s2 / (float)a.width + a.eps);
+    }
+    const float alpha = a.norm_out ? *a.norm_alpha : 0.f;
+#pragma unroll
+    for (int i = 0; i < GR_VPT; ++i) {
+        const int k = (tid + i * nt) * 4;
+        if (k >= W) continue;
+        v4f v = y[i];
+        if (a.y2) {
+            const v4f w1 = *(const v4f *)(a.w1 + k), w2 = *(const v4f *)(a.w2 + k);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = fmaf(y2[i][e] * i2, w2[e], v[e] * i1 * w1[e]);
+        }
+        v4f x = *(const v4f *)(a.x + base + k);
+        const v4f gz = *(const v4f *)(a.gate + (size_t)row * a.gate_stride + k), gb = *(const v4f *)(a.gate_b + k);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x[e] = fmaf(sigmoid_e(gz[e] + gb[e]), v[e], x[e]);
+        if (a.out) *(v4f *)(a.out + base + k) = x;
+        if (a.norm_out) *(v4f *)(a.norm_out + base + k) = dyt_row4(x, alpha, *(const v4f *)(a.norm_w + k), *(const v4f *)(a.norm_b + k));
+    }
+}
+int launch_gated_residual(lumen_ctx *ctx, const GatedResidualArgs &a) {
+    if (a.rows <= 0) return LUMEN_OK;
+    int threads = 256;
+    while (threads < 1024 && (threads * 4 * GR_VPT < a.dim || (a.rows < 16 && threads * 4 < a.dim))) threads *= 2;
+    if (threads * 4 * GR_VPT < a.dim) LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "gated residual: rows of %d", a.dim);
+    hipLaunchKernelGGL(gated_residual_kernel, dim3(a.rows), dim3(threads), 0, ctx->stream, a);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
 
 // ----------------------------------------------------- PolyNorm, token shift, row helpers
 // One workgroup per row; the row is read once for the three sums and once more (from cache) for the values.
@@ -318,6 +440,37 @@ __global__ __launch_bounds__(256) void gather_rows_kernel(const float *__restric
 int launch_gather_rows(lumen_ctx *ctx, const float *x, const int *idx, float *out, int n, int dim) {
     if (n <= 0) return LUMEN_OK;
     hipLaunchKernelGGL(gather_rows_kernel, dim3(n), dim3(256), 0, ctx->stream, x, idx, out, dim);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+// out [rows][n] = tanh of columns [0, n) of rows with the given stride
+__global__ __launch_bounds__(256) void tanh_rows_kernel(const float *__restrict__ x, int stride, float *__restrict__ out, int rows, int n) {
+    const size_t total = (size_t)rows * n;
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (size_t)gridDim.x * 256) out[i] = tanhf(x[i / n * stride + i % n]);
+}
+int launch_tanh_rows(lumen_ctx *ctx, const float *x, int stride, float *out, int rows, int n) {
+    if (rows <= 0 || n <= 0) return LUMEN_OK;
+    const size_t blocks = ((size_t)rows * n + 255) / 256, most = (size_t)ctx->num_cus * 8;
+    hipLaunchKernelGGL(tanh_rows_kernel, dim3((unsigned)(blocks < most ? blocks : most)), dim3(256), 0, ctx->stream, x, stride, out, rows, n);
+    LUMEN_CHECK_LAUNCH();
+    return LUMEN_OK;
+}
+
+// Token vectors plus position vectors: row t is W[ids[t]] + P[pos0 + t] (pos0 from device memory where pos_dev is given);
+// both indexes are clamped to their tables.
+__global__ __launch_bounds__(256) void embedding_pos_kernel(const float *__restrict__ W, const int *__restrict__ ids, const float *__restrict__ P,
+                                                            const int *__restrict__ pos_dev, int pos0, int dim, int vocab, int positions,
+                                                            float *__restrict__ out) {
+    const int id = min(max(ids[blockIdx.x], 0), vocab - 1);
+    const int pos = min((pos_dev ? *pos_dev : pos0) + (int)blockIdx.x, positions - 1);
+    const float *src = W + (size_t)id * dim, *add = P + (size_t)pos * dim;
+    for (int i = threadIdx.x; i < dim; i += 256) out[(size_t)blockIdx.x * dim + i] = src[i] + add[i];
+}
+int launch_embedding_pos(lumen_ctx *ctx, const float *W, const int *ids_dev, const float *P, const int *pos_dev, int pos0, int n, int dim, int vocab,
+                         int positions, float *out) {
+    if (n <= 0) return LUMEN_OK;
+    hipLaunchKernelGGL(embedding_pos_kernel, dim3(n), dim3(256), 0, ctx->stream, W, ids_dev, P, pos_dev, pos0, dim, vocab, positions, out);
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
 }

@@ -44,7 +44,7 @@ __device__ __forceinline__ float silu_g(float g) {
 
 // The 2x2 accumulator tiles of one wavefront to memory.  Accumulator register r of lane l holds
 // C[row = 8*(r/4) + 4*(l/32) + r%4][col = l%32] of its 32x32 tile.
-template <int EPI, bool PARTIAL>
+template <int EPI, bool PARTIAL, bool GROUPED>
 __device__ __forceinline__ void store_tile(const GemmArgs &a, const v16f (&acc)[2][2], int bm, int bn, int wm, int wn,
                                            int lane) {
     const int M = a.M, N = a.N;
@@ -64,8 +64,11 @@ __device__ __forceinline__ void store_tile(const GemmArgs &a, const v16f (&acc)[
                     // columns (2c, 2c+1) = (gate_c, up_c): silu(gate) * up, src/models/llama.rs:60-63
                     const float up = __shfl_xor(v, 1, 64);
                     if (!(col & 1) && row < M && col < N) a.C[(size_t)row * (N >> 1) + (col >> 1)] = silu_g(v) * up;
+                } else if (EPI == EPI_EXPERT_ACT) {
+                    const float up = __shfl_xor(v, 1, 64);
+                    if (!(col & 1) && row < M && col < N) a.C[(size_t)row * (N >> 1) + (col >> 1)] = expert_act(v, up, a.limit);
                 } else if (row < M && col < N) {
-                    const size_t o = (size_t)row * N + col;
+                    const size_t o = (GROUPED && a.c_rows ? (size_t)a.c_rows[row] : (size_t)row) * N + col;
                     a.C[o] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, v, a.residual[o]) : v;
                 }
             }
@@ -104,15 +107,23 @@ __device__ __forceinline__ void split3(const v4f x, v2u (&plane)[3]) {
 // slice are in flight from memory during the matrix instructions of the current one, then split
 // into their bf16 parts on the way into LDS ([part][row][k], k contiguous: an operand is one
 // 16-byte LDS read).  Two workgroups share a compute unit, one computing while the other stages.
-template <bool WBF16, int EPI, bool PARTIAL>
+template <bool WBF16, int EPI, bool PARTIAL, bool GROUPED = false>
 __global__ __launch_bounds__(256) void gemm_bf16x3_kernel(GemmArgs a) {
+    int bm = blockIdx.y * BM;
+    if (GROUPED) {  // (uniform)
+        const int *tile = a.tiles + 3 * blockIdx.y;
+        if (tile[2] <= 0) return;
+        bm = tile[1];
+        a.M = tile[1] + tile[2];
+        a.W = (const char *)a.W + (size_t)tile[0] * a.N * a.K * (WBF16 ? 2 : 4);
+    }
     constexpr int PW = WBF16 ? 1 : 3;       // bf16 parts of a weight
     constexpr int WST = WBF16 ? 2 : STAGE;  // 16-byte pieces of W per thread per slice
     __shared__ __align__(16) uint16_t As[3][BM][XROW];
     __shared__ __align__(16) uint16_t Ws[PW][BN][XROW];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int wm = wave >> 1, wn = wave & 1;
-    const int bm = blockIdx.y * BM, bn = blockIdx.x * BN;
+    const int bn = blockIdx.x * BN;
     const int M = a.M, N = a.N, K = a.K;
     const float *A = a.A;
     const int slices = (K + BK - 1) / BK;
@@ -130,6 +141,12 @@ __global__ __launch_bounds__(256) void gemm_bf16x3_kernel(GemmArgs a) {
 
     v4f va[STAGE];
     v4u vw[WST];  // f32 weights: 4 floats; bf16 weights: 8 values
+    size_t arow[STAGE];
+#pragma unroll
+    for (int i = 0; i < STAGE; ++i) {
+        const int r = bm + ((tid + i * 256) >> 3);
+        arow[i] = GROUPED && a.a_rows ? (size_t)a.a_rows[min(r, M - 1)] : (size_t)r;
+    }
     // A and f32 W: piece i of this thread is row (tid + 256 i) / 8, k offset 4 * ((tid + 256 i) % 8);
     // bf16 W: row (tid + 256 i) / 4, k offset 8 * ((tid + 256 i) % 4)
     auto fetch = [&](int k0) {
@@ -138,7 +155,7 @@ __global__ __launch_bounds__(256) void gemm_bf16x3_kernel(GemmArgs a) {
             const int idx = tid + i * 256;
             const int row = idx >> 3, k4 = (idx & 7) * 4;
             va[i] = (v4f){0.f, 0.f, 0.f, 0.f};
-            if (k0 + k4 < ke && bm + row < M) va[i] = *(const v4f *)(A + (size_t)(bm + row) * K + k0 + k4);
+            if (k0 + k4 < ke && bm + row < M) va[i] = *(const v4f *)(A + arow[i] * K + k0 + k4);
         }
 #pragma unroll
         for (int i = 0; i < WST; ++i) {
@@ -207,7 +224,7 @@ __global__ __launch_bounds__(256) void gemm_bf16x3_kernel(GemmArgs a) {
         }
         __syncthreads();
     }
-    store_tile<EPI, PARTIAL>(a, acc, bm, bn, wm, wn, lane);
+    store_tile<EPI, PARTIAL, GROUPED>(a, acc, bm, bn, wm, wn, lane);
 }
 
 // The pipelined kernel: F x F tiles of 32x32 per wavefront, 2 x 2 wavefronts, 16-deep slices, LDS
@@ -1145,6 +1162,24 @@ int launch_gemm(lumen_ctx *ctx, const GemmArgs &a) {
         LUMEN_CHECK_LAUNCH();
     }
     if (want_norm && !norm_done) LUMEN_TRY(launch_rmsnorm(ctx, a.C, a.norm_w, a.norm_out, a.M, a.N, a.norm_eps));
+    return LUMEN_OK;
+}
+
+int launch_gemm_grouped(lumen_ctx *ctx, const GemmArgs &a, int max_tiles) {
+    static_assert(GEMM_GROUP_ROWS == BM, "tiles of the plain kernel");
+    if (a.M <= 0 || a.N <= 0 || max_tiles <= 0) return LUMEN_OK;
+    if ((((uintptr_t)a.A | (uintptr_t)a.W) & 15) || a.K % (a.w_bf16 ? 8 : 4) || !a.tiles || (a.epi != EPI_STORE && a.epi != EPI_EXPERT_ACT) ||
+        (a.epi == EPI_EXPERT_ACT && (a.N & 1)))
+        LUMEN_FAIL(LUMEN_ERR_INVALID, "grouped GEMM: K=%d N=%d epilogue %d", a.K, a.N, a.epi);
+    const dim3 grid((a.N + BN - 1) / BN, max_tiles);
+    if (a.w_bf16) {
+        if (a.epi == EPI_STORE) hipLaunchKernelGGL((gemm_bf16x3_kernel<true, EPI_STORE, false, true>), grid, dim3(256), 0, ctx->stream, a);
+        else hipLaunchKernelGGL((gemm_bf16x3_kernel<true, EPI_EXPERT_ACT, false, true>), grid, dim3(256), 0, ctx->stream, a);
+    } else {
+        if (a.epi == EPI_STORE) hipLaunchKernelGGL((gemm_bf16x3_kernel<false, EPI_STORE, false, true>), grid, dim3(256), 0, ctx->stream, a);
+        else hipLaunchKernelGGL((gemm_bf16x3_kernel<false, EPI_EXPERT_ACT, false, true>), grid, dim3(256), 0, ctx->stream, a);
+    }
+    LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
 }
 

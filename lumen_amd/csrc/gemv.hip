@@ -207,16 +207,18 @@ __device__ __forceinline__ void stage_shift(float *xs, const float *__restrict__
 // weights are still on their way.
 #define GEMV_EARLY 2
 template <int PRO>
-__device__ __forceinline__ void request_early(v4f (&xe)[GEMV_EARLY], v4f (&ge)[GEMV_EARLY], const float *__restrict__ x,
-                                              const float *__restrict__ g, int K, int nthreads) {
+__device__ __forceinline__ void request_early(v4f (&xe)[GEMV_EARLY], v4f (&ge)[GEMV_EARLY], v4f (&be)[GEMV_EARLY], const float *__restrict__ x,
+                                              const float *__restrict__ g, const float *__restrict__ b, int K, int nthreads) {
 #pragma unroll
     for (int i = 0; i < GEMV_EARLY; ++i) {
         const int k = ((int)threadIdx.x + i * nthreads) * 4;
         xe[i] = v4f{0.f, 0.f, 0.f, 0.f};
         ge[i] = v4f{0.f, 0.f, 0.f, 0.f};
+        be[i] = v4f{0.f, 0.f, 0.f, 0.f};
         if (k < K) {
             xe[i] = *(const v4f *)(x + k);
-            if (PRO == PRO_RMSNORM) ge[i] = *(const v4f *)(g + k);
+            if (PRO == PRO_RMSNORM || PRO == PRO_DYT) ge[i] = *(const v4f *)(g + k);
+            if (PRO == PRO_DYT) be[i] = *(const v4f *)(b + k);
         }
     }
 }
@@ -278,6 +280,46 @@ __device__ __forceinline__ void stage_x_early(float *xs, const float *__restrict
     __syncthreads();
 }
 
+__device__ __forceinline__ v4f dyt4(const v4f x, float alpha, const v4f g, const v4f b) {
+    return v4f{fmaf(tanhf(alpha * x.x), g.x, b.x), fmaf(tanhf(alpha * x.y), g.y, b.y), fmaf(tanhf(alpha * x.z), g.z, b.z),
+               fmaf(tanhf(alpha * x.w), g.w, b.w)};
+}
+
+// Dynamic Tanh of x into LDS: element by element, no sum to wait for.  EARLY: the first pieces were requested ahead.
+template <bool EARLY, int XB>
+__device__ __forceinline__ void stage_dyt(float *xs, const float *__restrict__ x, const float *__restrict__ g, const float *__restrict__ b,
+                                          float alpha, int K, int kpad, int nwaves, const v4f (&xe)[GEMV_EARLY],
+                                          const v4f (&ge)[GEMV_EARLY], const v4f (&be)[GEMV_EARLY]) {
+    const int nthreads = nwaves * 64;
+    int k0 = (int)threadIdx.x * 4;
+    if (EARLY) {
+#pragma unroll
+        for (int i = 0; i < GEMV_EARLY; ++i) {
+            const int k = k0 + i * nthreads * 4;
+            if (k < kpad) *(v4f *)(xs + k) = dyt4(xe[i], alpha, ge[i], be[i]);  // (zero gain and shift beyond K)
+        }
+        k0 += GEMV_EARLY * nthreads * 4;
+    }
+    for (; k0 < kpad; k0 += nthreads * 4 * XB) {
+        v4f v[XB], gg[XB], bb[XB];
+#pragma unroll
+        for (int i = 0; i < XB; ++i) {
+            const int k = min(k0 + i * nthreads * 4, K - 4);
+            v[i] = *(const v4f *)(x + k);
+            gg[i] = *(const v4f *)(g + k);
+            bb[i] = *(const v4f *)(b + k);
+        }
+#pragma unroll
+        for (int i = 0; i < XB; ++i) {
+            const int k = k0 + i * nthreads * 4;
+            if (k < kpad) *(v4f *)(xs + k) = k < K ? dyt4(v[i], alpha, gg[i], bb[i]) : v4f{0.f, 0.f, 0.f, 0.f};
+        }
+    }
+    __syncthreads();
+}
+
+__device__ __forceinline__ float gelu_f(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+
 // Stages the decode attention output from the attention kernel's partial states: head h, element d is
 // sum_s w_s ctx_s[d] / (sum_s w_s l_s + 1e-9) with w_s = exp2(m_s - max m) over the slices in use
 // (self_attention.rs:287-290 after the merge of the slices' online-softmax states).  A thread's loads
@@ -324,7 +366,9 @@ __device__ __forceinline__ void stage_attn_fold(float *xs, const GemvArgs &a, in
             const float inv = 1.0f / (L + 1e-9f);
             v.x *= inv; v.y *= inv; v.z *= inv; v.w *= inv;
             if (a.attn_gate) {
-                const v4f gz = *(const v4f *)(a.attn_gate + k);
+                v4f gz;
+                if (a.attn_gate_heads) gz = v4f{1.f, 1.f, 1.f, 1.f} * a.attn_gate[k / D];  // (D is a multiple of 4: one head)
+                else gz = *(const v4f *)(a.attn_gate + k);
 #pragma unroll
                 for (int e = 0; e < 4; ++e) v[e] *= 1.0f / (1.0f + expf(-gz[e]));
             }
@@ -404,11 +448,12 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
         }
     };
 
-    constexpr bool EARLY = XB == 0 && (PRO == PRO_NONE || PRO == PRO_RMSNORM);
-    v4f xe[GEMV_EARLY], ge[GEMV_EARLY];
+    constexpr bool EARLY = XB == 0 && (PRO == PRO_NONE || PRO == PRO_RMSNORM || PRO == PRO_DYT);
+    v4f xe[GEMV_EARLY], ge[GEMV_EARLY], be[GEMV_EARLY];
+    const float dyt_alpha = PRO == PRO_DYT ? *a.norm_alpha : 0.f;
     // (with a row selector -- the first layer's gather -- the address of x needs a trip to memory itself:
     // then the weights go first)
-    if (EARLY && !row_sel_hot) request_early<PRO>(xe, ge, x_hot, norm_w_hot, K, nwaves * 64);
+    if (EARLY && !row_sel_hot) request_early<PRO>(xe, ge, be, x_hot, norm_w_hot, a.norm_b, K, nwaves * 64);
 
     // the first weights of this wavefront start streaming before x is staged: they do not depend on it
     v4u rawA[R][U], rawB[R][U];
@@ -428,14 +473,14 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
     if (row_sel_hot) {
         sel_off = (long)(*row_sel_hot) * a.row_stride;
         if (a.x_sel) xin += sel_off;
-        if (EARLY) request_early<PRO>(xe, ge, xin, norm_w_hot, K, nwaves * 64);
+        if (EARLY) request_early<PRO>(xe, ge, be, xin, norm_w_hot, a.norm_b, K, nwaves * 64);
     }
     const float *residual = a.residual + (a.residual_sel ? sel_off : 0);
     // What a unit's epilogue needs from memory is requested a unit ahead -- the first one here,
     // before x is staged -- so that no load sits between the last multiply and the store:
     // cos / sin of the unit's RoPE pair, or the residual of its rows.
     const int pos = (EPI == EPI_ROPE_QKV) ? *a.pos : 0;
-    float pre0 = 0.f, pre1 = 0.f;
+    float pre0 = 0.f, pre1 = 0.f, gate0 = 0.f, gate1 = 0.f, gate_b0 = 0.f, gate_b1 = 0.f;
     auto preload = [&](int un) {
         if (EPI == EPI_ROPE_QKV && un < nunits) {
             const int j = un % half_d;
@@ -445,6 +490,15 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
         if (EPI == EPI_RESIDUAL) {
             if (un * R < N) pre0 = residual[un * R];
             if (R == 2 && un * R + 1 < N) pre1 = residual[un * R + 1];
+            if (a.res_gate) {
+                const int r0 = min(un * R, N - 1), r1 = min(un * R + R - 1, N - 1);
+                gate0 = a.res_gate[r0];
+                gate_b0 = a.res_gate_b[r0];
+                if (R == 2) {
+                    gate1 = a.res_gate[r1];
+                    gate_b1 = a.res_gate_b[r1];
+                }
+            }
         }
     };
     preload(gw);
@@ -456,6 +510,7 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
         stage_shift<(XB > 0 ? XB : 1)>(xs, xin, norm_w_hot, a.eps, a.shift_mu + (size_t)seg * K, a.shift_state + (size_t)slot * K,
                                        a.shift_state + (size_t)(slot ^ 1u) * K, seg == 0 && blockIdx.x == 0, K, kpad, nwaves);
     }
+    else if (PRO == PRO_DYT) stage_dyt<EARLY, (XB > 0 ? XB : 1)>(xs, xin, norm_w_hot, a.norm_b, dyt_alpha, K, kpad, nwaves, xe, ge, be);
     else if (EARLY) stage_x_early<PRO>(xs, xin, norm_w_hot, a.eps, K, kpad, nwaves, xe, ge);
     else stage_x<PRO, (XB > 0 ? XB : 1)>(xs, xin, norm_w_hot, a.eps, K, kpad, nwaves);
     STAGE_T(2);
@@ -521,7 +576,15 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
                         const int row = u * R + r;
                         if (row < N) {
                             // residual: x + y, src/ops/arithmetic.rs:48-51 via src/models/llama.rs:110,115
-                            y_out[row] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, acc[r], r == 0 ? pre0 : pre1) : acc[r];
+                            float v = acc[r];
+                            if (EPI == EPI_RESIDUAL) {
+                                const float f = a.res_gate ? 1.0f / (1.0f + expf(-(r == 0 ? gate0 + gate_b0 : gate1 + gate_b1))) : a.alpha;
+                                v = fmaf(f, v, r == 0 ? pre0 : pre1);
+                            } else if (EPI == EPI_STORE || EPI == EPI_ARGMAX) {
+                                if (a.softcap > 0.f) v = a.softcap * tanhf(v / a.softcap);
+                                if (EPI == EPI_STORE && a.gelu_from > 0 && row >= a.gelu_from) v = gelu_f(v);
+                            }
+                            y_out[row] = v;
                         }
                     }
                 }
@@ -690,7 +753,12 @@ static void launch_pro(const GemvArgs &a, dim3 grid, int threads, size_t lds, hi
         hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_POLYNORM, EPI_RESIDUAL, (XB == 0 ? 1 : XB), KA>), grid, dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
     else if (a.pro == PRO_SHIFT)  // token-shift products (launch_gemv checks): plain store
         hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_SHIFT, EPI_STORE, (XB == 0 ? 1 : XB), KA>), dim3(grid.x, a.shift_segs), dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
-    else if (a.pro == PRO_RMSNORM)
+    else if (a.pro == PRO_DYT) {  // projections and the head (launch_gemv checks)
+        if (a.epi == EPI_ARGMAX)
+            hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_DYT, EPI_ARGMAX, XB, KA>), grid, dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
+        else
+            hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_DYT, EPI_STORE, XB, KA>), grid, dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
+    } else if (a.pro == PRO_RMSNORM)
         launch_epi<BF16, R, PRO_RMSNORM, XB, KA>(a, grid, threads, lds, s);
     else
         launch_epi<BF16, R, PRO_NONE, XB, KA>(a, grid, threads, lds, s);
@@ -760,7 +828,7 @@ GemvPick gemv_pick(int num_cus, int N, int K, int w_bf16, int pro, int epi, bool
     // at a time from three pieces per thread on.
     const int x_pieces = (kpad + p.threads * 4 - 1) / (p.threads * 4);
     const int nunits = (N + p.R - 1) / p.R;
-    const bool early_x = (pro == PRO_NONE || pro == PRO_RMSNORM) && x_pieces <= GEMV_EARLY && kpad / piece <= 2 &&
+    const bool early_x = (pro == PRO_NONE || pro == PRO_RMSNORM || pro == PRO_DYT) && x_pieces <= GEMV_EARLY && kpad / piece <= 2 &&
                          nunits <= p.blocks * (p.threads / 64);
     p.xb = early_x ? 0 : x_pieces > 2 ? 4 : 1;
     p.ka = K % piece == 0;  // whole pieces: no clamped load positions
@@ -779,11 +847,11 @@ int launch_gemv(lumen_ctx *ctx, const GemvArgs &a) {
     if (a.N <= 0 || a.K <= 0) return LUMEN_OK;
     const int vec = a.w_bf16 ? 8 : 4;
     const bool aligned = (((uintptr_t)a.W | (uintptr_t)a.x) & 15) == 0 && (((uintptr_t)a.attn_part) & 7) == 0 &&
-                         (a.pro != PRO_RMSNORM || ((uintptr_t)a.norm_w & 15) == 0);
+                         ((a.pro != PRO_RMSNORM && a.pro != PRO_DYT) || (((uintptr_t)a.norm_w | (uintptr_t)a.norm_b) & 15) == 0);
     const GemvPick p = gemv_pick(ctx->num_cus, a.N, a.K, a.w_bf16, a.pro, a.epi, aligned);
     if (ctx->note_kernels) gemv_kernel_name(p, a.w_bf16, ctx->last_kernel, sizeof ctx->last_kernel);
     if (!p.fast) {
-        if (a.pro != PRO_NONE || a.epi != EPI_STORE || a.row_sel)
+        if (a.pro != PRO_NONE || a.epi != EPI_STORE || a.row_sel || a.softcap > 0.f || a.gelu_from > 0)
             LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "fused GEMV needs K %% %d == 0, 16-byte alignment and K <= %d (K=%d)", vec,
                        16384, a.K);
         if (a.w_bf16)
@@ -795,10 +863,13 @@ int launch_gemv(lumen_ctx *ctx, const GemvArgs &a) {
     }
     if (a.pro == PRO_ATTN_FOLD) {
         if (a.epi != EPI_RESIDUAL || p.R != 1 || !a.attn_part || !a.attn_pos || a.attn_d <= 0 || a.attn_d % 4 ||
-            a.K % a.attn_d || ((uintptr_t)a.attn_gate & 15) || a.attn_nslices < 1 || a.attn_nslices > GEMV_FOLD_MAX_SLICES)
+            a.K % a.attn_d || (!a.attn_gate_heads && ((uintptr_t)a.attn_gate & 15)) || a.attn_nslices < 1 || a.attn_nslices > GEMV_FOLD_MAX_SLICES)
             LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over attention partials: one row per unit, residual epilogue, at most %d slices (got %d)",
                        GEMV_FOLD_MAX_SLICES, a.attn_nslices);
     }
+    if (a.pro == PRO_DYT && (!a.norm_w || !a.norm_b || !a.norm_alpha || (a.epi != EPI_STORE && a.epi != EPI_ARGMAX)))
+        LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over a Dynamic Tanh input: gain, shift and alpha, store or arg-max epilogue");
+    if (a.epi == EPI_RESIDUAL && a.res_gate && !a.res_gate_b) LUMEN_FAIL(LUMEN_ERR_INVALID, "gated residual: no gate bias");
     if (a.pro == PRO_POLYNORM && (a.epi != EPI_RESIDUAL || !a.norm_w || a.norm_dim <= 0))
         LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over a PolyNorm input: residual epilogue, four coefficients and the element count");
     if (a.pro == PRO_SHIFT &&

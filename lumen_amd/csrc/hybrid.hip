@@ -1,11 +1,14 @@
 // The layered hybrid decoder: a stack of layers whose sequence mixers differ (sliding-window attention, WKV time
-// mixing, channel-wise gated delta rule), each with an optional PolyNorm feed-forward; a range of layers may run
-// several times over, every pass with a state of its own.
+// mixing, channel-wise gated delta rule, generalised delta rule, attention and a matrix memory side by side), each with an
+// optional feed-forward (PolyNorm, GELU or a mixture of experts); a range of layers may run several times over, every pass
+// with a state of its own.
 //
 // Like the Llama model, everything a step touches is allocated once, a decode step is a fixed sequence of launches
 // that reads the token and the position from device memory and is replayed as one HIP graph, and prompts run on the
 // GEMMs.  Decode, launches per layer: input norm + projections (one product; for WKV the five token-shift products
-// side by side), the mixer, output projection + residual, norm + up, PolyNorm + down + residual.
+// side by side), the mixer, output projection + residual, norm + up, PolyNorm + down + residual.  The gates of a gated
+// residual are further rows of the products that read the same normalised vector: the mixer's of the input projections,
+// the feed-forward's (and a router's) of the up product.
 //
 // Layouts: weights [out, in] with both sizes rounded up to a multiple of 8 (zeros), the input projections of a mixer
 // one after the other in one matrix; activations f32, rows of the rounded size.  A norm of the rounded row is taken
@@ -17,6 +20,7 @@
 #include <algorithm>
 #include <cmath>
 #include <cstring>
+#include <functional>
 #include <memory>
 #include <string>
 
@@ -31,6 +35,7 @@ struct Param {  // where a named tensor goes
     bool f32 = false;      // f32 on the device whatever the weight dtype
     size_t rows = 0, cols = 0, ld = 0;
     float add = 0.f, mul = 1.f;  // stored value = (v + add) * mul
+    std::function<std::vector<float>(const std::vector<float> &)> expand;  // ... or what this makes of the whole tensor, [n] f32
     void *dst2 = nullptr;  // columns from col_split on go to a second matrix
     size_t col_split = 0;
 };
@@ -39,10 +44,19 @@ struct Layer {
     lumen_hybrid_layer c = {};
     // rows of the projection matrix and where its blocks start
     int n_proj = 0, off_q = 0, off_k = 0, off_v = 0, off_g = 0, off_b = 0, off_lo = 0, off_hi = 0;
+    int off_a = 0, off_rg = 0;           // general delta: removal rates; gated residual: gate of the mixer
+    int off_mq = 0, off_mk = 0, off_mv = 0, off_mg = 0, off_mi = 0, off_mf = 0;  // parallel: the matrix memory's
+    int od2 = 0;                         // parallel: channels of the matrix memory's output (rounded)
+    int n_up = 0, up_at = 0;             // rows of the up product; where the feed-forward's (the router's) start
+    int bias_n = 0;                      // distances of the attention's bias table
     int seg = 0, seg_last = 0;           // WKV: rows of a token-shift product
     int od = 0;                          // channels of the mixer's output (rounded)
     void *w_proj = nullptr, *w_o = nullptr, *w_lo = nullptr, *w_hi = nullptr, *w_up = nullptr, *w_down = nullptr;
     float *norm1 = nullptr, *norm2 = nullptr, *act = nullptr;
+    float *norm1_b = nullptr, *norm1_a = nullptr, *norm2_b = nullptr, *norm2_a = nullptr;  // Dynamic Tanh: shift, alpha
+    float *rg1_b = nullptr, *rg2_b = nullptr, *a_bias = nullptr;
+    void *w_o2 = nullptr, *w_eup = nullptr, *w_edown = nullptr;
+    float *temp = nullptr, *bias_tab = nullptr, *sink = nullptr, *i_bias = nullptr, *f_bias = nullptr, *out1 = nullptr, *out2 = nullptr;
     float *q_norm = nullptr, *k_norm = nullptr, *r1 = nullptr, *r2 = nullptr;            // attention
     float *mu = nullptr, *bias = nullptr, *u = nullptr, *a_log = nullptr, *taps = nullptr, *gain = nullptr;
     int lo_rank = 0, hi_rank = 0;        // rounded
@@ -53,7 +67,7 @@ struct Layer {
 
 struct Run {  // one pass through one layer
     int layer = 0, pass = -1;  // pass >= 0: the loop's input step comes first
-    int st_matrix = -1, st_aux = -1, st_k = -1, st_v = -1;
+    int st_matrix = -1, st_aux = -1, st_k = -1, st_v = -1;  // (parallel: st_aux is the matrix memory's running maximum)
 };
 
 }  // namespace
@@ -68,15 +82,17 @@ struct lumen_hybrid {
     std::vector<Layer> layers;
     std::vector<Run> runs;
     std::vector<Param> params;
-    float *embed = nullptr, *final_norm = nullptr, *loop_step = nullptr;
+    float *embed = nullptr, *final_norm = nullptr, *final_b = nullptr, *final_a = nullptr, *loop_step = nullptr, *positions = nullptr;
     void *head = nullptr, *loop_x = nullptr, *loop_x0 = nullptr;
     std::unique_ptr<SeqState> state;
     int len = 0;
     unsigned step = 0;  // forward passes since the reset: which slot of a two-slot state block is current (mirror of *d_step)
-    int max_proj = 0, max_od = 0, max_ff = 0, max_lo = 0, max_hi = 0, max_heads = 0;
+    int max_proj = 0, max_od = 0, max_ff = 0, max_lo = 0, max_hi = 0, max_heads = 0, max_od2 = 0, max_top = 0, max_act = 0, max_experts = 0;
+    size_t max_raw = 0;  // floats per token of the matrix memory's raw output
     // decode
     float *x0 = nullptr, *xa = nullptr, *xb = nullptr, *proj = nullptr, *mixed = nullptr, *ff = nullptr, *logits = nullptr,
-          *steps = nullptr, *c0 = nullptr, *part = nullptr;
+          *steps = nullptr, *c0 = nullptr, *part = nullptr, *mixed2 = nullptr, *pair = nullptr, *act = nullptr;
+    int *d_sel = nullptr;
     int *d_tok = nullptr, *d_pos = nullptr, *tok_hist = nullptr, *d_err = nullptr;
     unsigned *d_step = nullptr, *amax_epoch = nullptr;
     unsigned long long *amax_word = nullptr;
@@ -88,8 +104,9 @@ struct lumen_hybrid {
     std::vector<void *> pf_allocs;
     float *p_x0 = nullptr, *p_xa = nullptr, *p_xb = nullptr, *p_n = nullptr, *p_proj = nullptr, *p_mixes = nullptr, *p_mixed = nullptr,
           *p_ff = nullptr, *p_steps = nullptr, *p_q = nullptr, *p_k = nullptr, *p_v = nullptr, *p_lo = nullptr, *p_hi = nullptr,
-          *p_z = nullptr, *p_gate = nullptr, *p_logits = nullptr, *p_rows = nullptr;
-    int *p_ids = nullptr, *p_idx = nullptr;
+          *p_z = nullptr, *p_gate = nullptr, *p_logits = nullptr, *p_rows = nullptr, *p_raw = nullptr, *p_scan = nullptr, *p_mixed2 = nullptr,
+          *p_y = nullptr, *p_y2 = nullptr, *p_rg = nullptr, *p_route = nullptr, *p_selw = nullptr, *p_act = nullptr, *p_eout = nullptr;
+    int *p_ids = nullptr, *p_idx = nullptr, *p_plan = nullptr;
     std::vector<void *> allocs;
     // per-class event times of a profiled step
     struct Probe *probe = nullptr;
@@ -134,9 +151,30 @@ static void add_matrix(lumen_hybrid *m, const std::string &name, void *base, int
 static void add_vector(lumen_hybrid *m, const std::string &name, float *dst, int n) {
     add_param(m, name, {n}, dst, true, 1, n, n);
 }
-static void add_norm(lumen_hybrid *m, const std::string &name, float *dst) {
+// A norm of the residual stream: gains, and for Dynamic Tanh the shift and alpha stored beside them.
+static int create_norm(lumen_hybrid *m, const std::string &name, float **w, float **b, float **alpha) {
     const int n = m->cfg.width;
-    add_param(m, name, {n}, dst, true, 1, n, n, m->cfg.norm_offset, sqrtf((float)n / (float)m->W));
+    LUMEN_TRY(alloc_t(m, w, m->W));
+    if (m->cfg.norm_kind == LUMEN_NORM_RMS) {
+        add_param(m, name, {n}, *w, true, 1, n, n, m->cfg.norm_offset, sqrtf((float)n / (float)m->W));
+        return LUMEN_OK;
+    }
+    LUMEN_TRY(alloc_t(m, b, m->W));
+    LUMEN_TRY(alloc_t(m, alpha, 4));
+    add_vector(m, name, *w, n);
+    add_vector(m, name + ".b", *b, n);
+    add_param(m, name + ".alpha", {}, *alpha, true, 1, 1, 1);
+    return LUMEN_OK;
+}
+
+// Row of a distance bias of `rows` rows for distance n: one row per distance in the lower half, a logarithmic scale up
+// to `most` above.  (Distances at which the scale meets a whole number belong to the row that starts there: the small
+// addend keeps the quotient of two logarithms from falling short of it.)
+static int bias_row(int n, int rows, int most) {
+    const int half = rows / 2;
+    if (n < half) return n;
+    if (n >= most || half < 1 || most <= half) return rows - 1;
+    return std::min(rows - 1, half + (int)std::floor(std::log((double)n / half) / std::log((double)most / half) * (rows - half) + 1e-9));
 }
 
 static int check_layer(const lumen_hybrid_layer &c, int i) {
@@ -153,6 +191,19 @@ static int check_layer(const lumen_hybrid_layer &c, int i) {
             if (c.kv_heads != c.heads || c.vdim != c.dim) LUMEN_FAIL(LUMEN_ERR_SHAPE, "hybrid_create: layer %d: WKV heads are square and unshared", i);
             if (c.rank_lo <= 0) LUMEN_FAIL(LUMEN_ERR_SHAPE, "hybrid_create: layer %d: decay rank %d", i, c.rank_lo);
             break;
+        case LUMEN_MIXER_GENERAL_DELTA:
+            if (c.kv_heads != c.heads || c.vdim != c.dim) LUMEN_FAIL(LUMEN_ERR_SHAPE, "hybrid_create: layer %d: general delta heads are square and unshared", i);
+            if (c.rank_lo <= 0) LUMEN_FAIL(LUMEN_ERR_SHAPE, "hybrid_create: layer %d: decay rank %d", i, c.rank_lo);
+            break;
+        case LUMEN_MIXER_PARALLEL:
+            if (c.mem_heads <= 0 || c.mem_dim <= 0 || c.mem_vdim <= 0 || c.bias_rows < 2 || c.bias_max <= 0 || !(c.gate_cap > 0.f))
+                LUMEN_FAIL(LUMEN_ERR_SHAPE, "hybrid_create: layer %d: matrix memory %d x %d x %d, gate cap %g, %d bias rows up to %d", i, c.mem_heads,
+                           c.mem_dim, c.mem_vdim, c.gate_cap, c.bias_rows, c.bias_max);
+            if (c.mem_dim > MIX_MAX_DIM || c.mem_vdim > MIX_MAX_DIM)
+                LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: heads wider than %d", i, MIX_MAX_DIM);
+            if (c.mem_heads * c.mem_vdim > 16384) LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: inner sizes above 16384", i);
+            break;
+            break;
         case LUMEN_MIXER_CHANNEL_DELTA:
             if (c.rank_lo <= 0 || c.rank_hi <= 0) LUMEN_FAIL(LUMEN_ERR_SHAPE, "hybrid_create: layer %d: ranks %d, %d", i, c.rank_lo, c.rank_hi);
             if (c.conv < 1 || c.conv > MIX_MAX_TAPS) LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: %d convolution taps", i, c.conv);
@@ -163,6 +214,25 @@ static int check_layer(const lumen_hybrid_layer &c, int i) {
         LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: ranks above %d", i, MIX_MAX_RANK);
     if (c.ff > 16384 || c.heads * c.vdim > 16384 || c.heads * c.dim > 16384)
         LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: inner sizes above 16384 do not fit the GEMV's LDS stage", i);
+    if (c.ff > 0 && c.ff_kind == LUMEN_FF_EXPERTS) {
+        if (c.experts <= 0 || c.groups <= 0 || c.experts % c.groups || c.keep <= 0 || c.keep > c.groups || c.top <= 0 ||
+            c.top > c.keep * (c.experts / c.groups))
+            LUMEN_FAIL(LUMEN_ERR_SHAPE, "hybrid_create: layer %d: %d of %d experts, %d of %d groups", i, c.top, c.experts, c.keep, c.groups);
+        if (c.experts > EXPERTS_MAX || c.top > EXPERTS_MAX_TOP || c.top * pad8(c.ff) > 16384)
+            LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: %d experts, %d at a time of %d", i, c.experts, c.top, c.ff);
+    } else if (c.ff > 0 && c.ff_kind != LUMEN_FF_POLYNORM && c.ff_kind != LUMEN_FF_GELU) {
+        LUMEN_FAIL(LUMEN_ERR_INVALID, "hybrid_create: layer %d: unknown feed-forward %d", i, c.ff_kind);
+    }
+    return LUMEN_OK;
+}
+
+// A design's layers fit together where its norm and residual have the products that take them.
+static int check_design(const lumen_hybrid_config &c, const lumen_hybrid_layer &y, int i) {
+    const bool dyt = c.norm_kind == LUMEN_NORM_DYT;
+    const bool later = y.mixer == LUMEN_MIXER_GENERAL_DELTA || y.mixer == LUMEN_MIXER_PARALLEL;
+    if (later != dyt || (y.ff > 0 && (y.ff_kind != LUMEN_FF_POLYNORM) != dyt) || (c.residual_gate != 0) != dyt)
+        LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: layer %d: Dynamic Tanh goes with gated residuals, general delta or parallel mixers and GELU or "
+                   "expert feed-forwards", i);
     return LUMEN_OK;
 }
 
@@ -174,8 +244,7 @@ static int create_layer(lumen_hybrid *m, Layer &L, int i) {
     L.od = pad8(H * Dv);
     L.lo_rank = pad8(c.rank_lo);
     L.hi_rank = pad8(c.rank_hi);
-    LUMEN_TRY(alloc_t(m, &L.norm1, m->W));
-    add_norm(m, p + "norm1", L.norm1);
+    LUMEN_TRY(create_norm(m, p + "norm1", &L.norm1, &L.norm1_b, &L.norm1_a));
     LUMEN_TRY(weight(&L.w_o, W, H * Dv));
     auto block = [&](int n) {  // the next block of the projection matrix
         const int off = L.n_proj;
@@ -225,6 +294,77 @@ static int create_layer(lumen_hybrid *m, Layer &L, int i) {
         add_vector(m, mp + "w0", L.bias, H * D);
         add_param(m, mp + "u", {H, D}, L.u, true, 1, (size_t)H * D, (size_t)H * D);
         add_vector(m, mp + "norm", L.gain, H * D);
+    } else if (c.mixer == LUMEN_MIXER_GENERAL_DELTA) {
+        L.off_q = block(H * D); L.off_k = block(H * D); L.off_v = block(H * D); L.off_g = block(H * D); L.off_a = block(H * D);
+        L.off_lo = block(c.rank_lo); L.off_rg = block(W);
+        LUMEN_TRY(weight(&L.w_proj, L.n_proj, W));
+        add_matrix(m, mp + "r", L.w_proj, L.off_q, H * D, W);
+        add_matrix(m, mp + "k", L.w_proj, L.off_k, H * D, W);
+        add_matrix(m, mp + "v", L.w_proj, L.off_v, H * D, W);
+        add_matrix(m, mp + "g", L.w_proj, L.off_g, H * D, W);
+        add_matrix(m, mp + "a", L.w_proj, L.off_a, H * D, W);
+        add_matrix(m, mp + "w1", L.w_proj, L.off_lo, c.rank_lo, W);
+        LUMEN_TRY(weight(&L.w_lo, H * D, c.rank_lo));
+        add_matrix(m, mp + "w2", L.w_lo, 0, H * D, c.rank_lo);
+        LUMEN_TRY(alloc_t(m, &L.bias, H * D));
+        LUMEN_TRY(alloc_t(m, &L.a_bias, H * D));
+        LUMEN_TRY(alloc_t(m, &L.gain, H * D));
+        add_vector(m, mp + "w0", L.bias, H * D);
+        add_vector(m, mp + "a.b", L.a_bias, H * D);
+        add_vector(m, mp + "norm", L.gain, H * D);
+    } else if (c.mixer == LUMEN_MIXER_PARALLEL) {
+        const int Hm = c.mem_heads, Dm = c.mem_dim, Vm = c.mem_vdim;
+        const std::string lp = mp + "left.", rp = mp + "right.";
+        L.off_q = block(H * D); L.off_k = block(G * D); L.off_v = block(G * Dv); L.off_g = block(H);
+        L.off_mq = block(Hm * Dm); L.off_mk = block(Hm * Dm); L.off_mv = block(Hm * Vm); L.off_mg = block(Hm * Vm);
+        L.off_mi = block(Hm); L.off_mf = block(Hm); L.off_rg = block(W);
+        LUMEN_TRY(weight(&L.w_proj, L.n_proj, W));
+        add_matrix(m, lp + "q", L.w_proj, L.off_q, H * D, W);
+        add_matrix(m, lp + "k", L.w_proj, L.off_k, G * D, W);
+        add_matrix(m, lp + "v", L.w_proj, L.off_v, G * Dv, W);
+        add_matrix(m, lp + "g", L.w_proj, L.off_g, H, W);
+        add_matrix(m, rp + "q", L.w_proj, L.off_mq, Hm * Dm, W);
+        add_matrix(m, rp + "k", L.w_proj, L.off_mk, Hm * Dm, W);
+        add_matrix(m, rp + "v", L.w_proj, L.off_mv, Hm * Vm, W);
+        add_matrix(m, rp + "g", L.w_proj, L.off_mg, Hm * Vm, W);
+        add_matrix(m, rp + "i", L.w_proj, L.off_mi, Hm, W);
+        add_matrix(m, rp + "f", L.w_proj, L.off_mf, Hm, W);
+        // attention
+        const int B = c.bias_rows, most = c.bias_max;
+        L.bias_n = 1;  // distances up to the first whose row is the last one, and to all further ones
+        while (bias_row(L.bias_n - 1, B, most) < B - 1 && L.bias_n < m->cfg.max_seq_len) ++L.bias_n;
+        LUMEN_TRY(alloc_t(m, &L.bias_tab, (size_t)H * L.bias_n));
+        LUMEN_TRY(alloc_t(m, &L.temp, H));
+        LUMEN_TRY(alloc_t(m, &L.sink, H));
+        const int n = L.bias_n;
+        add_param(m, lp + "rel", {B, H}, L.bias_tab, true, 1, (size_t)B * H, (size_t)B * H);
+        m->params.back().expand = [B, H, n, most](const std::vector<float> &rel) {
+            std::vector<float> tab((size_t)H * n);
+            for (int h = 0; h < H; ++h)
+                for (int d = 0; d < n; ++d) tab[(size_t)h * n + d] = rel[(size_t)bias_row(d, B, most) * H + h] * 1.44269504088896341f;
+            return tab;
+        };
+        add_vector(m, lp + "temp", L.temp, H);
+        add_vector(m, lp + "sink", L.sink, H);
+        L.window = L.cap = m->cfg.max_seq_len;
+        L.slices = window_attn_slices(L.window);
+        // matrix memory
+        L.od2 = pad8(Hm * Vm);
+        LUMEN_TRY(weight(&L.w_o2, W, Hm * Vm));
+        add_matrix(m, rp + "o", L.w_o2, 0, W, Hm * Vm);
+        LUMEN_TRY(alloc_t(m, &L.i_bias, Hm));
+        LUMEN_TRY(alloc_t(m, &L.f_bias, Hm));
+        LUMEN_TRY(alloc_t(m, &L.gain, Hm * Vm));
+        add_vector(m, rp + "i.b", L.i_bias, Hm);
+        add_vector(m, rp + "f.b", L.f_bias, Hm);
+        add_vector(m, rp + "norm", L.gain, Hm * Vm);
+        LUMEN_TRY(alloc_t(m, &L.out1, m->W));
+        LUMEN_TRY(alloc_t(m, &L.out2, m->W));
+        add_vector(m, lp + "out", L.out1, W);
+        add_vector(m, rp + "out", L.out2, W);
+        m->max_od2 = std::max(m->max_od2, L.od2);
+        m->max_raw = std::max(m->max_raw, (size_t)Hm * (Vm + 1));
+        m->max_heads = std::max(m->max_heads, Hm * std::max(Dm, Vm));
     } else {
         L.off_q = block(G * D); L.off_k = block(G * D); L.off_v = block(H * Dv); L.off_b = block(H);
         L.off_lo = block(c.rank_lo); L.off_hi = block(c.rank_hi);
@@ -254,20 +394,52 @@ static int create_layer(lumen_hybrid *m, Layer &L, int i) {
         add_vector(m, mp + "A_log", L.a_log, H);
         add_vector(m, mp + "norm", L.gain, Dv);
     }
-    add_matrix(m, mp + "o", L.w_o, 0, W, H * Dv);
+    add_matrix(m, mp + (c.mixer == LUMEN_MIXER_PARALLEL ? "left.o" : "o"), L.w_o, 0, W, H * Dv);
+    if (m->cfg.residual_gate) {
+        LUMEN_TRY(alloc_t(m, &L.rg1_b, m->W));
+        add_matrix(m, p + "rg1", L.w_proj, L.off_rg, W, W);
+        add_vector(m, p + "rg1.b", L.rg1_b, W);
+    }
     if (c.ff > 0) {
-        LUMEN_TRY(alloc_t(m, &L.norm2, m->W));
-        add_norm(m, p + "norm2", L.norm2);
-        LUMEN_TRY(weight(&L.w_up, c.ff, W));
-        LUMEN_TRY(weight(&L.w_down, W, c.ff));
-        LUMEN_TRY(alloc_t(m, &L.act, 4));
-        add_matrix(m, p + "mlp.up", L.w_up, 0, c.ff, W);
-        add_matrix(m, p + "mlp.down", L.w_down, 0, W, c.ff);
-        add_vector(m, p + "mlp.act", L.act, 4);
+        const bool experts = c.ff_kind == LUMEN_FF_EXPERTS;
+        LUMEN_TRY(create_norm(m, p + "norm2", &L.norm2, &L.norm2_b, &L.norm2_a));
+        // the up product: the feed-forward's gate, then the up matrix or the router
+        L.up_at = m->cfg.residual_gate ? m->W : 0;
+        L.n_up = L.up_at + pad8(experts ? c.experts : c.ff);
+        LUMEN_TRY(weight(&L.w_up, L.n_up, W));
+        if (m->cfg.residual_gate) {
+            LUMEN_TRY(alloc_t(m, &L.rg2_b, m->W));
+            add_matrix(m, p + "rg2", L.w_up, 0, W, W);
+            add_vector(m, p + "rg2.b", L.rg2_b, W);
+        }
+        if (experts) {
+            const size_t F = pad8(c.ff), K = m->W, E = c.experts;
+            add_matrix(m, p + "mlp.router", L.w_up, L.up_at, c.experts, W);
+            LUMEN_TRY(alloc_zero(m, &L.w_eup, E * 2 * F * K * m->esz));
+            LUMEN_TRY(alloc_zero(m, &L.w_edown, E * K * F * m->esz));
+            for (size_t e = 0; e < E; ++e) {  // gate and up rows in turn
+                const std::string ep = p + "mlp.e" + std::to_string(e) + ".";
+                char *up = (char *)L.w_eup + e * 2 * F * K * m->esz;
+                add_param(m, ep + "gate", {c.ff, W}, up, false, c.ff, W, 2 * K);
+                add_param(m, ep + "up", {c.ff, W}, up + K * m->esz, false, c.ff, W, 2 * K);
+                add_param(m, ep + "down", {W, c.ff}, (char *)L.w_edown + e * K * F * m->esz, false, W, c.ff, F);
+            }
+            m->max_top = std::max(m->max_top, c.top);
+            m->max_act = std::max(m->max_act, c.top * (int)F);
+            m->max_experts = std::max(m->max_experts, pad8(c.experts));
+        } else {
+            LUMEN_TRY(weight(&L.w_down, W, c.ff));
+            add_matrix(m, p + "mlp.up", L.w_up, L.up_at, c.ff, W);
+            add_matrix(m, p + "mlp.down", L.w_down, 0, W, c.ff);
+            if (c.ff_kind == LUMEN_FF_POLYNORM) {
+                LUMEN_TRY(alloc_t(m, &L.act, 4));
+                add_vector(m, p + "mlp.act", L.act, 4);
+            }
+        }
     }
     m->max_proj = std::max(m->max_proj, L.n_proj);
     m->max_od = std::max(m->max_od, L.od);
-    m->max_ff = std::max(m->max_ff, pad8(c.ff));
+    m->max_ff = std::max(m->max_ff, L.n_up);
     m->max_lo = std::max(m->max_lo, L.lo_rank);
     m->max_hi = std::max(m->max_hi, L.hi_rank);
     m->max_heads = std::max(m->max_heads, std::max(H * D, H * Dv));
@@ -281,22 +453,27 @@ static int create_impl(lumen_hybrid *m, const lumen_hybrid_layer *layers) {
     m->layers.resize(c.num_layers);
     LUMEN_TRY(alloc_t(m, &m->embed, (size_t)V * W));
     add_param(m, "embed", {V, c.width}, m->embed, true, V, c.width, W, 0.f, c.embed_scale);
+    if (c.max_positions > 0) {
+        LUMEN_TRY(alloc_t(m, &m->positions, (size_t)c.max_positions * W));
+        add_param(m, "pos", {c.max_positions, c.width}, m->positions, true, c.max_positions, c.width, W);
+    }
     if (c.loop_times > 0) {
-        LUMEN_TRY(alloc_zero(m, &m->loop_x, (size_t)W * W * m->esz));
-        LUMEN_TRY(alloc_zero(m, &m->loop_x0, (size_t)W * W * m->esz));
         LUMEN_TRY(alloc_t(m, &m->loop_step, (size_t)c.loop_times * W));
-        Param p;
-        p.name = "loop.in"; p.shape = {c.width, 2 * c.width}; p.dst = m->loop_x; p.dst2 = m->loop_x0; p.col_split = c.width;
-        p.rows = c.width; p.cols = 2 * (size_t)c.width; p.ld = W;
-        m->params.push_back(p);
+        if (c.loop_kind == LUMEN_LOOP_MIX) {
+            LUMEN_TRY(alloc_zero(m, &m->loop_x, (size_t)W * W * m->esz));
+            LUMEN_TRY(alloc_zero(m, &m->loop_x0, (size_t)W * W * m->esz));
+            Param p;
+            p.name = "loop.in"; p.shape = {c.width, 2 * c.width}; p.dst = m->loop_x; p.dst2 = m->loop_x0; p.col_split = c.width;
+            p.rows = c.width; p.cols = 2 * (size_t)c.width; p.ld = W;
+            m->params.push_back(p);
+        }
         add_param(m, "loop.step", {c.loop_times, c.width}, m->loop_step, true, c.loop_times, c.width, W);
     }
     for (int i = 0; i < c.num_layers; ++i) {
         m->layers[i].c = layers[i];
         LUMEN_TRY(create_layer(m, m->layers[i], i));
     }
-    LUMEN_TRY(alloc_t(m, &m->final_norm, W));
-    add_norm(m, "final.norm", m->final_norm);
+    LUMEN_TRY(create_norm(m, "final.norm", &m->final_norm, &m->final_b, &m->final_a));
     LUMEN_TRY(alloc_zero(m, &m->head, (size_t)V * W * m->esz));
     add_matrix(m, "head", m->head, 0, V, c.width);
 
@@ -305,9 +482,16 @@ static int create_impl(lumen_hybrid *m, const lumen_hybrid_layer *layers) {
         const Layer &L = m->layers[layer];
         r.layer = layer;
         r.pass = pass;
-        if (L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION) {
+        if (L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION || L.c.mixer == LUMEN_MIXER_PARALLEL) {
             r.st_k = m->state->reserve(SeqState::ROLLING, (size_t)L.c.kv_heads * L.cap * ((L.c.dim + 3) & ~3));
             r.st_v = m->state->reserve(SeqState::ROLLING, (size_t)L.c.kv_heads * L.cap * ((L.c.vdim + 3) & ~3));
+            if (L.c.mixer == LUMEN_MIXER_PARALLEL) {
+                r.st_matrix = m->state->reserve(SeqState::ZEROED, (size_t)L.c.mem_heads * recurrence_columns(REC_MEMORY, L.c.mem_vdim) *
+                                                                      recurrence_rows(L.c.mem_dim));
+                r.st_aux = m->state->reserve(SeqState::ZEROED, L.c.mem_heads);
+            }
+        } else if (L.c.mixer == LUMEN_MIXER_GENERAL_DELTA) {
+            r.st_matrix = m->state->reserve(SeqState::ZEROED, (size_t)L.c.heads * L.c.vdim * recurrence_rows(L.c.dim));
         } else {
             r.st_matrix = m->state->reserve(SeqState::ZEROED, (size_t)L.c.heads * L.c.vdim * recurrence_rows(L.c.dim));
             r.st_aux = m->state->reserve(SeqState::ZEROED, L.c.mixer == LUMEN_MIXER_WKV ? (size_t)2 * W
@@ -331,6 +515,10 @@ static int create_impl(lumen_hybrid *m, const lumen_hybrid_layer *layers) {
     LUMEN_TRY(alloc_t(m, &m->proj, m->max_proj));
     LUMEN_TRY(alloc_t(m, &m->mixed, m->max_od));
     LUMEN_TRY(alloc_t(m, &m->ff, m->max_ff));
+    LUMEN_TRY(alloc_t(m, &m->mixed2, m->max_od2));
+    LUMEN_TRY(alloc_t(m, &m->pair, (size_t)2 * W));
+    LUMEN_TRY(alloc_t(m, &m->act, m->max_act));
+    LUMEN_TRY(alloc_t(m, &m->d_sel, m->max_top));
     LUMEN_TRY(alloc_t(m, &m->logits, V));
     size_t part = 4;
     for (const Layer &L : m->layers)
@@ -359,7 +547,14 @@ extern "C" int lumen_hybrid_create(lumen_ctx *ctx, const lumen_hybrid_config *cf
                    cfg->num_layers);
     if (cfg->width > 16384) LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: width above 16384 does not fit the GEMV's LDS stage");
     if (cfg->vocab_size >= (1 << 24)) LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "hybrid_create: vocabulary of %d", cfg->vocab_size);
-    for (int i = 0; i < cfg->num_layers; ++i) LUMEN_TRY(check_layer(layers[i], i));
+    if (cfg->norm_kind != LUMEN_NORM_RMS && cfg->norm_kind != LUMEN_NORM_DYT) LUMEN_FAIL(LUMEN_ERR_INVALID, "hybrid_create: norm_kind %d", cfg->norm_kind);
+    if (cfg->loop_kind != LUMEN_LOOP_MIX && cfg->loop_kind != LUMEN_LOOP_ADD) LUMEN_FAIL(LUMEN_ERR_INVALID, "hybrid_create: loop_kind %d", cfg->loop_kind);
+    if (cfg->max_positions > 0 && cfg->max_seq_len > cfg->max_positions)
+        LUMEN_FAIL(LUMEN_ERR_SHAPE, "hybrid_create: sequences of %d with %d positions", cfg->max_seq_len, cfg->max_positions);
+    for (int i = 0; i < cfg->num_layers; ++i) {
+        LUMEN_TRY(check_layer(layers[i], i));
+        LUMEN_TRY(check_design(*cfg, layers[i], i));
+    }
     HIP_TRY(hipSetDevice(ctx->device));
     lumen_hybrid *m = new lumen_hybrid();
     m->ctx = ctx;
@@ -397,7 +592,7 @@ extern "C" int lumen_hybrid_param_info(const lumen_hybrid *m, int index, char *n
 }
 
 extern "C" int lumen_hybrid_set_param(lumen_hybrid *m, const char *name, const void *data, int dtype, const int64_t *shape, int ndim) {
-    if (!m || !name || !data || !shape) LUMEN_FAIL(LUMEN_ERR_INVALID, "hybrid_set_param: null argument");
+    if (!m || !name || !data || ndim < 0 || (!shape && ndim > 0)) LUMEN_FAIL(LUMEN_ERR_INVALID, "hybrid_set_param: null argument");
     if (dtype != LUMEN_DTYPE_F32 && dtype != LUMEN_DTYPE_BF16) LUMEN_FAIL(LUMEN_ERR_INVALID, "Unsupported dtype: %d for %s", dtype, name);
     for (const Param &p : m->params) {
         if (p.name != name) continue;
@@ -405,6 +600,15 @@ extern "C" int lumen_hybrid_set_param(lumen_hybrid *m, const char *name, const v
         HIP_TRY(hipSetDevice(m->ctx->device));
         const bool to_f32 = p.f32 || !m->bf16;
         const size_t esz = to_f32 ? 4 : 2, src_esz = dtype == LUMEN_DTYPE_BF16 ? 2 : 4;
+        if (p.expand) {
+            std::vector<float> in(p.rows * p.cols);
+            if (dtype == LUMEN_DTYPE_BF16) bf16_to_f32_host((const uint16_t *)data, in.data(), in.size());
+            else memcpy(in.data(), data, in.size() * 4);
+            const std::vector<float> out = p.expand(in);
+            HIP_TRY(hipMemcpyAsync(p.dst, out.data(), out.size() * 4, hipMemcpyHostToDevice, m->ctx->stream));
+            HIP_TRY(hipStreamSynchronize(m->ctx->stream));
+            return LUMEN_OK;
+        }
         const bool convert = p.add != 0.f || p.mul != 1.f || to_f32 != (dtype == LUMEN_DTYPE_F32);
         const size_t chunk = std::max<size_t>(1, ((size_t)16 << 20) / p.cols);
         std::vector<float> wide;
@@ -457,7 +661,8 @@ extern "C" int lumen_hybrid_load_safetensors(lumen_hybrid *m, const char *path, 
 
 // ------------------------------------------------------------------ decode
 // Launch classes of a decode step, for per-kernel timing.
-enum { HC_EMBED = 0, HC_LOOP, HC_PROJ_ATTN, HC_ATTN, HC_PROJ_WKV, HC_WKV, HC_PROJ_DELTA, HC_DELTA, HC_OUT, HC_UP, HC_DOWN, HC_HEAD, HC_COUNT };
+enum { HC_EMBED = 0, HC_LOOP, HC_PROJ_ATTN, HC_ATTN, HC_PROJ_WKV, HC_WKV, HC_PROJ_DELTA, HC_DELTA, HC_OUT, HC_UP, HC_DOWN, HC_HEAD,
+       HC_PROJ_GENERAL, HC_GENERAL, HC_PROJ_PARALLEL, HC_MEMORY, HC_PAIR, HC_EXPERT_UP, HC_EXPERT_DOWN, HC_COUNT };
 
 struct Probe {
     std::vector<hipEvent_t> ev;
@@ -482,6 +687,9 @@ static int timed(lumen_hybrid *m, int cls, int rc_launch(lumen_hybrid *, const v
 }
 static int do_gemv(lumen_hybrid *m, const void *a) { return launch_gemv(m->ctx, *(const GemvArgs *)a); }
 static int do_attn(lumen_hybrid *m, const void *a) { return launch_window_attn_decode(m->ctx, *(const WindowAttnArgs *)a); }
+static int do_pair(lumen_hybrid *m, const void *a) { return launch_gated_residual(m->ctx, *(const GatedResidualArgs *)a); }
+static int do_experts_up(lumen_hybrid *m, const void *a) { return launch_experts_up(m->ctx, *(const ExpertsArgs *)a); }
+static int do_experts_down(lumen_hybrid *m, const void *a) { return launch_experts_down(m->ctx, *(const ExpertsArgs *)a); }
 static int do_rec(lumen_hybrid *m, const void *a) { return launch_recurrence_decode(m->ctx, *(const RecurrenceDecodeArgs *)a); }
 
 static GemvArgs gemv_args(const lumen_hybrid *m, const void *w, int N, int K, const float *x, float *y) {
@@ -489,8 +697,9 @@ static GemvArgs gemv_args(const lumen_hybrid *m, const void *w, int N, int K, co
     g.W = w; g.N = N; g.K = K; g.x = x; g.y = y; g.w_bf16 = m->bf16; g.pro = PRO_NONE; g.epi = EPI_STORE;
     return g;
 }
-static void gemv_norm(const lumen_hybrid *m, GemvArgs &g, const float *gains) {
-    g.pro = PRO_RMSNORM; g.norm_w = gains; g.eps = m->eps_w;
+static void gemv_norm(const lumen_hybrid *m, GemvArgs &g, const float *gains, const float *shift, const float *alpha) {
+    g.pro = m->cfg.norm_kind == LUMEN_NORM_DYT ? PRO_DYT : PRO_RMSNORM;
+    g.norm_w = gains; g.norm_b = shift; g.norm_alpha = alpha; g.eps = m->eps_w;
 }
 static void gemv_residual(GemvArgs &g, const float *residual, float alpha) {
     g.epi = EPI_RESIDUAL; g.residual = residual; g.alpha = alpha;
@@ -504,6 +713,35 @@ static WindowAttnArgs attn_args(const lumen_hybrid *m, const Layer &L, const Run
     a.cap = L.cap; a.dpad = (L.c.dim + 3) & ~3; a.vpad = (L.c.vdim + 3) & ~3;
     a.heads = L.c.heads; a.kv_heads = L.c.kv_heads; a.dim = L.c.dim; a.vdim = L.c.vdim; a.window = L.window; a.gate_act = GATE_SIGMOID;
     a.scale = L.c.scale; a.softcap = L.c.softcap; a.r1 = L.r1; a.r2 = L.r2; a.slices = L.slices;
+    a.temp = L.temp; a.bias_tab = L.bias_tab; a.bias_n = L.bias_n; a.sink = L.sink; a.gate_heads = L.c.mixer == LUMEN_MIXER_PARALLEL;
+    return a;
+}
+
+#define MEMORY_DEN_EPS 1e-6f
+static const float GENERAL_DECAY = 0.60653065971263342f;  // e^{-1/2}
+
+// What the decode kernels of the general delta rule and of the matrix memory are told.
+static RecurrenceDecodeArgs later_decode_args(lumen_hybrid *m, const Layer &L, const Run &r) {
+    const lumen_hybrid_config &c = m->cfg;
+    RecurrenceDecodeArgs a = {};
+    a.w_bf16 = m->bf16; a.proj = m->proj; a.unit_eps = c.unit_eps; a.norm_eps = c.norm_eps; a.gain = L.gain; a.state = m->state->ptr(r.st_matrix);
+    if (L.c.mixer == LUMEN_MIXER_GENERAL_DELTA) {
+        a.kind = REC_GENERAL; a.heads = a.kv_heads = L.c.heads; a.dim = a.vdim = L.c.dim;
+        a.off_q = L.off_q; a.off_k = L.off_k; a.off_v = L.off_v; a.off_gate = L.off_g; a.off_a = L.off_a; a.off_lo = L.off_lo;
+        a.w_lo = L.w_lo; a.r_lo = L.lo_rank; a.bias = L.bias; a.a_bias = L.a_bias; a.z_scale = GENERAL_DECAY; a.out = m->mixed;
+    } else {
+        a.kind = REC_MEMORY; a.heads = a.kv_heads = L.c.mem_heads; a.dim = L.c.mem_dim; a.vdim = L.c.mem_vdim;
+        a.off_q = L.off_mq; a.off_k = L.off_mk; a.off_v = L.off_mv; a.off_gate = L.off_mg; a.off_i = L.off_mi; a.off_f = L.off_mf;
+        a.i_bias = L.i_bias; a.f_bias = L.f_bias; a.cap = L.c.gate_cap; a.den_eps = MEMORY_DEN_EPS; a.q_scale = 1.0f / sqrtf((float)L.c.mem_dim);
+        a.m = m->state->ptr(r.st_aux); a.out = m->mixed2;
+    }
+    return a;
+}
+
+static ExpertsArgs experts_args(const lumen_hybrid *m, const Layer &L) {
+    ExpertsArgs a = {};
+    a.r = RouterShape{L.c.experts, L.c.groups, L.c.keep, L.c.top, L.c.router_scale};
+    a.w_up = L.w_eup; a.w_down = L.w_edown; a.w_bf16 = m->bf16; a.dim = m->W; a.ff = pad8(L.c.ff); a.limit = L.c.limit;
     return a;
 }
 
@@ -521,12 +759,19 @@ static int tap_rows(lumen_hybrid *m, const Tap *tap, size_t run, const float *x,
     return LUMEN_OK;
 }
 
+static int embed_rows(lumen_hybrid *m, const int *ids, int n, const int *pos_dev, int pos, float *out) {
+    const lumen_hybrid_config &c = m->cfg;
+    if (!m->positions) return launch_embedding(m->ctx, m->embed, ids, n, m->W, c.vocab_size, out);
+    return launch_embedding_pos(m->ctx, m->embed, ids, m->positions, pos_dev, pos, n, m->W, c.vocab_size, c.max_positions, out);
+}
+
 static int enqueue_decode_step(lumen_hybrid *m, const Tap *tap = nullptr) {
     const lumen_hybrid_config &c = m->cfg;
     lumen_ctx *ctx = m->ctx;
     const int W = m->W;
-    LUMEN_TRY(launch_embedding(ctx, m->embed, m->d_tok, 1, W, c.vocab_size, m->x0));
-    if (c.loop_times > 0) {
+    LUMEN_TRY(embed_rows(m, m->d_tok, 1, m->d_pos, 0, m->x0));
+    const bool mix = c.loop_times > 0 && c.loop_kind == LUMEN_LOOP_MIX;
+    if (mix) {
         GemvArgs g = gemv_args(m, m->loop_x0, W, W, m->x0, m->c0);
         LUMEN_TRY(timed(m, HC_LOOP, do_gemv, &g));
         LUMEN_TRY(launch_add_steps(ctx, m->c0, m->loop_step, m->steps, c.loop_times, 1, W));
@@ -538,26 +783,41 @@ static int enqueue_decode_step(lumen_hybrid *m, const Tap *tap = nullptr) {
         const Layer &L = m->layers[r.layer];
         if (r.pass >= 0) {
             float *y = cur == m->xa ? m->xb : m->xa;
-            GemvArgs g = gemv_args(m, m->loop_x, W, W, cur, y);
-            gemv_residual(g, m->steps + (size_t)r.pass * W, 1.0f);
-            LUMEN_TRY(timed(m, HC_LOOP, do_gemv, &g));
+            if (mix) {
+                GemvArgs g = gemv_args(m, m->loop_x, W, W, cur, y);
+                gemv_residual(g, m->steps + (size_t)r.pass * W, 1.0f);
+                LUMEN_TRY(timed(m, HC_LOOP, do_gemv, &g));
+            } else {
+                LUMEN_TRY(launch_add_steps(ctx, cur, m->loop_step + (size_t)r.pass * W, y, 1, 1, W));
+            }
             cur = y;
         }
         if (L.c.mixer == LUMEN_MIXER_WKV) {
             GemvArgs g = gemv_args(m, L.w_proj, L.seg, W, cur, m->proj);
-            gemv_norm(m, g, L.norm1);
+            gemv_norm(m, g, L.norm1, nullptr, nullptr);
             g.pro = PRO_SHIFT; g.shift_mu = L.mu; g.shift_state = m->state->ptr(r.st_aux); g.shift_step = m->d_step;
             g.shift_segs = 5; g.shift_rows = L.seg; g.shift_last_rows = L.seg_last;
             LUMEN_TRY(timed(m, HC_PROJ_WKV, do_gemv, &g));
         } else {
             GemvArgs g = gemv_args(m, L.w_proj, L.n_proj, W, cur, m->proj);
-            gemv_norm(m, g, L.norm1);
-            LUMEN_TRY(timed(m, L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION ? HC_PROJ_ATTN : HC_PROJ_DELTA, do_gemv, &g));
+            gemv_norm(m, g, L.norm1, L.norm1_b, L.norm1_a);
+            const int cls = L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION ? HC_PROJ_ATTN
+                            : L.c.mixer == LUMEN_MIXER_CHANNEL_DELTA  ? HC_PROJ_DELTA
+                            : L.c.mixer == LUMEN_MIXER_GENERAL_DELTA  ? HC_PROJ_GENERAL
+                                                                      : HC_PROJ_PARALLEL;
+            LUMEN_TRY(timed(m, cls, do_gemv, &g));
         }
-        if (L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION) {
+        if (L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION || L.c.mixer == LUMEN_MIXER_PARALLEL) {
             WindowAttnArgs a = attn_args(m, L, r, m->proj, L.n_proj);
             a.out = m->mixed; a.pos_dev = m->d_pos; a.part = m->part; a.leave_slices = L.fold;
             LUMEN_TRY(timed(m, HC_ATTN, do_attn, &a));
+            if (L.c.mixer == LUMEN_MIXER_PARALLEL) {
+                const RecurrenceDecodeArgs rm = later_decode_args(m, L, r);
+                LUMEN_TRY(timed(m, HC_MEMORY, do_rec, &rm));
+            }
+        } else if (L.c.mixer == LUMEN_MIXER_GENERAL_DELTA) {
+            const RecurrenceDecodeArgs a = later_decode_args(m, L, r);
+            LUMEN_TRY(timed(m, HC_GENERAL, do_rec, &a));
         } else {
             const bool wkv = L.c.mixer == LUMEN_MIXER_WKV;
             RecurrenceDecodeArgs a = {};
@@ -572,9 +832,20 @@ static int enqueue_decode_step(lumen_hybrid *m, const Tap *tap = nullptr) {
             a.state = m->state->ptr(r.st_matrix); a.out = m->mixed;
             LUMEN_TRY(timed(m, wkv ? HC_WKV : HC_DELTA, do_rec, &a));
         }
-        {
+        if (L.c.mixer == LUMEN_MIXER_PARALLEL) {
+            GemvArgs g = gemv_args(m, L.w_o, W, L.od, m->mixed, m->pair);
+            LUMEN_TRY(timed(m, HC_OUT, do_gemv, &g));
+            g = gemv_args(m, L.w_o2, W, L.od2, m->mixed2, m->pair + W);
+            LUMEN_TRY(timed(m, HC_OUT, do_gemv, &g));
+            GatedResidualArgs p = {};
+            p.x = cur; p.y = m->pair; p.y2 = m->pair + W; p.w1 = L.out1; p.w2 = L.out2; p.pair_scale = 0.5f; p.eps = c.norm_eps;
+            p.gate = m->proj + L.off_rg; p.gate_b = L.rg1_b; p.out = out(); p.rows = 1; p.dim = W; p.width = c.width;
+            LUMEN_TRY(timed(m, HC_PAIR, do_pair, &p));
+            cur = p.out;
+        } else {
             GemvArgs g = gemv_args(m, L.w_o, W, L.od, m->mixed, out());
             gemv_residual(g, cur, c.residual_mult);
+            if (c.residual_gate) { g.res_gate = m->proj + L.off_rg; g.res_gate_b = L.rg1_b; }
             if (L.fold) {
                 g.pro = PRO_ATTN_FOLD; g.attn_part = m->part; g.attn_pos = m->d_pos; g.attn_nslices = L.slices; g.attn_d = L.c.vdim;
                 g.attn_trip = WINDOW_SLICE_KEYS; g.attn_short_rows = 0; g.attn_window = L.window; g.attn_gate = m->proj + L.off_g;
@@ -583,19 +854,31 @@ static int enqueue_decode_step(lumen_hybrid *m, const Tap *tap = nullptr) {
             cur = g.y;
         }
         if (L.c.ff > 0) {
-            GemvArgs g = gemv_args(m, L.w_up, pad8(L.c.ff), W, cur, m->ff);
-            gemv_norm(m, g, L.norm2);
+            GemvArgs g = gemv_args(m, L.w_up, L.n_up, W, cur, m->ff);
+            gemv_norm(m, g, L.norm2, L.norm2_b, L.norm2_a);
+            if (L.c.ff_kind == LUMEN_FF_GELU) g.gelu_from = L.up_at;
             LUMEN_TRY(timed(m, HC_UP, do_gemv, &g));
-            g = gemv_args(m, L.w_down, W, pad8(L.c.ff), m->ff, out());
-            gemv_residual(g, cur, c.residual_mult);
-            g.pro = PRO_POLYNORM; g.norm_w = L.act; g.eps = c.norm_eps; g.norm_dim = L.c.ff;
-            LUMEN_TRY(timed(m, HC_DOWN, do_gemv, &g));
-            cur = g.y;
+            if (L.c.ff_kind == LUMEN_FF_EXPERTS) {
+                ExpertsArgs e = experts_args(m, L);
+                e.z = m->ff + L.up_at; e.x = cur; e.norm_alpha = L.norm2_a; e.norm_w = L.norm2; e.norm_b = L.norm2_b; e.gate = m->ff; e.gate_b = L.rg2_b;
+                e.act = m->act; e.sel = m->d_sel; e.y = out();
+                LUMEN_TRY(timed(m, HC_EXPERT_UP, do_experts_up, &e));
+                LUMEN_TRY(timed(m, HC_EXPERT_DOWN, do_experts_down, &e));
+                cur = e.y;
+            } else {
+                g = gemv_args(m, L.w_down, W, pad8(L.c.ff), m->ff + L.up_at, out());
+                gemv_residual(g, cur, c.residual_mult);
+                if (c.residual_gate) { g.res_gate = m->ff; g.res_gate_b = L.rg2_b; }
+                if (L.c.ff_kind == LUMEN_FF_POLYNORM) { g.pro = PRO_POLYNORM; g.norm_w = L.act; g.eps = c.norm_eps; g.norm_dim = L.c.ff; }
+                LUMEN_TRY(timed(m, HC_DOWN, do_gemv, &g));
+                cur = g.y;
+            }
         }
         LUMEN_TRY(tap_rows(m, tap, ri, cur, 1));
     }
     GemvArgs g = gemv_args(m, m->head, c.vocab_size, W, cur, m->logits);
-    gemv_norm(m, g, m->final_norm);
+    gemv_norm(m, g, m->final_norm, m->final_b, m->final_a);
+    g.softcap = c.logit_softcap;
     g.epi = EPI_ARGMAX; g.amax_word = m->amax_word; g.amax_epoch = m->amax_epoch; g.err_dev = m->d_err; g.spin_limit = HANDOVER_MAX_SPINS;
     g.tok_out = m->d_tok; g.pos_inc = m->d_pos; g.tok_hist = m->tok_hist; g.step_inc = m->d_step;
     return timed(m, HC_HEAD, do_gemv, &g);
@@ -667,6 +950,28 @@ static int ensure_prompt_buffers(lumen_hybrid *m, int s) {
     LUMEN_TRY(get(&m->p_hi, S * m->max_hi));
     LUMEN_TRY(get(&m->p_z, S * pad8(m->max_heads)));
     LUMEN_TRY(get(&m->p_gate, S * pad8(m->max_heads)));
+    if (m->cfg.residual_gate) {
+        LUMEN_TRY(get(&m->p_y, S * W));
+        LUMEN_TRY(get(&m->p_rg, S * W));
+    }
+    if (m->max_od2) {
+        LUMEN_TRY(get(&m->p_y2, S * W));
+        LUMEN_TRY(get(&m->p_raw, S * m->max_raw));
+        LUMEN_TRY(get(&m->p_mixed2, S * m->max_od2));
+        size_t scan = 0;
+        for (const Layer &L : m->layers) scan = std::max(scan, memory_scan_floats(s, L.c.mem_heads));
+        LUMEN_TRY(get(&m->p_scan, scan));
+    }
+    if (m->max_top) {
+        size_t plan = 0;
+        for (const Layer &L : m->layers)
+            if (L.c.ff > 0 && L.c.ff_kind == LUMEN_FF_EXPERTS) plan = std::max(plan, experts_plan_ints(s, experts_args(m, L).r));
+        LUMEN_TRY(get(&m->p_route, S * m->max_experts));
+        LUMEN_TRY(get(&m->p_selw, S * m->max_top));
+        LUMEN_TRY(get(&m->p_act, S * m->max_act));
+        LUMEN_TRY(get(&m->p_eout, S * m->max_top * W));
+        LUMEN_TRY(alloc_t(m, &m->p_plan, plan, &m->pf_allocs));
+    }
     LUMEN_TRY(alloc_t(m, &m->p_ids, S, &m->pf_allocs));
     LUMEN_TRY(alloc_t(m, &m->p_idx, S, &m->pf_allocs));
     m->pf_cap = s;
@@ -736,6 +1041,83 @@ static int prompt_delta(lumen_hybrid *m, const Layer &L, const Run &r, int s) {
     return launch_head_norm_gate(ctx, m->p_mixed, L.od, L.gain, 1, m->p_gate, pad8(H * Dv), GATE_SIGMOID, s, H, Dv, m->cfg.norm_eps);
 }
 
+static int prompt_general(lumen_hybrid *m, const Layer &L, const Run &r, int s) {
+    lumen_ctx *ctx = m->ctx;
+    const int H = L.c.heads, D = L.c.dim, n = L.n_proj;
+    LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_n, L.w_proj, m->p_proj, s, n, m->W)));
+    LUMEN_TRY(launch_tanh_rows(ctx, m->p_proj + L.off_lo, n, m->p_lo, s, L.lo_rank));
+    LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_lo, L.w_lo, m->p_z, s, pad8(H * D), L.lo_rank)));
+    RecurrenceArgs a = {};
+    a.kind = REC_GENERAL; a.heads = H; a.rep = 1; a.dim = a.vdim = D; a.s = s;
+    a.q = m->p_proj + L.off_q; a.k = m->p_proj + L.off_k; a.v = m->p_proj + L.off_v; a.b = m->p_proj + L.off_a; a.z = m->p_z;
+    a.q_stride = a.k_stride = a.v_stride = a.b_stride = n; a.z_stride = pad8(H * D);
+    a.bias = L.bias; a.b_bias = L.a_bias; a.unit_eps = m->cfg.unit_eps; a.z_scale = GENERAL_DECAY;
+    a.state = m->state->ptr(r.st_matrix); a.out = m->p_mixed; a.out_stride = L.od;
+    LUMEN_TRY(launch_recurrence(ctx, a));
+    return launch_head_norm_gate(ctx, m->p_mixed, L.od, L.gain, 0, m->p_proj + L.off_g, n, GATE_SIGMOID, s, H, D, m->cfg.norm_eps);
+}
+
+static int prompt_memory(lumen_hybrid *m, const Layer &L, const Run &r, int s) {
+    const int H = L.c.mem_heads, D = L.c.mem_dim, V = L.c.mem_vdim, n = L.n_proj;
+    RecurrenceArgs a = {};
+    a.kind = REC_MEMORY; a.heads = H; a.rep = 1; a.dim = D; a.vdim = V; a.s = s;
+    a.q = m->p_proj + L.off_mq; a.k = m->p_proj + L.off_mk; a.v = m->p_proj + L.off_mv; a.gi = m->p_proj + L.off_mi; a.gf = m->p_proj + L.off_mf;
+    a.q_stride = a.k_stride = a.v_stride = a.g_stride = n;
+    a.gi_bias = L.i_bias; a.gf_bias = L.f_bias; a.cap = L.c.gate_cap; a.q_scale = 1.0f / sqrtf((float)D);
+    a.m = m->state->ptr(r.st_aux); a.m_out = m->p_scan; a.state = m->state->ptr(r.st_matrix); a.out = m->p_raw; a.out_stride = H * (V + 1);
+    LUMEN_TRY(launch_recurrence(m->ctx, a));
+    return launch_memory_read(m->ctx, m->p_raw, m->p_scan, m->p_mixed2, L.od2, L.gain, m->p_proj + L.off_mg, n, GATE_SIGMOID, s, H, V, m->cfg.norm_eps,
+                              MEMORY_DEN_EPS);
+}
+
+// Mixer and feed-forward of a layer whose residuals are gated, p_n holding norm1 of cur; the sums go to x.  next: the norm that
+// p_n is to hold afterwards (null gains: none).
+struct NormRef {
+    const float *w, *b, *alpha;
+};
+static int prompt_gated_layer(lumen_hybrid *m, const Layer &L, const Run &r, int s, const float *cur, float *x, NormRef next) {
+    lumen_ctx *ctx = m->ctx;
+    const lumen_hybrid_config &c = m->cfg;
+    const int W = m->W;
+    GatedResidualArgs p = {};
+    p.eps = c.norm_eps; p.rows = s; p.dim = W; p.width = c.width;
+    auto sum = [&](const float *from, const float *gate, int stride, const float *gate_b, NormRef n) {
+        p.x = from; p.gate = gate; p.gate_stride = stride; p.gate_b = gate_b; p.out = x;
+        p.norm_w = n.w; p.norm_b = n.b; p.norm_alpha = n.alpha; p.norm_out = n.w ? m->p_n : nullptr;
+        return launch_gated_residual(ctx, p);
+    };
+    const NormRef norm2 = {L.norm2, L.norm2_b, L.norm2_a};
+    if (L.c.mixer == LUMEN_MIXER_PARALLEL) {
+        LUMEN_TRY(prompt_attention(m, L, r, s));
+        LUMEN_TRY(prompt_memory(m, L, r, s));
+        LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_mixed2, L.w_o2, m->p_y2, s, W, L.od2)));
+        p.y2 = m->p_y2; p.w1 = L.out1; p.w2 = L.out2; p.pair_scale = 0.5f;
+    } else {
+        LUMEN_TRY(prompt_general(m, L, r, s));
+    }
+    LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_mixed, L.w_o, m->p_y, s, W, L.od)));
+    p.y = m->p_y;
+    LUMEN_TRY(sum(cur, m->p_proj + L.off_rg, L.n_proj, L.rg1_b, L.c.ff > 0 ? norm2 : next));
+    if (L.c.ff <= 0) return LUMEN_OK;
+    LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_n, L.w_up, m->p_rg, s, W, W)));
+    const void *up = (const char *)L.w_up + (size_t)L.up_at * W * m->esz;
+    p.y2 = nullptr;
+    if (L.c.ff_kind == LUMEN_FF_EXPERTS) {
+        const int E = pad8(L.c.experts);
+        LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_n, up, m->p_route, s, E, W)));
+        ExpertsArgs e = experts_args(m, L);
+        e.z = m->p_route; e.z_stride = E; e.rows = m->p_n; e.sel_w = m->p_selw; e.p_act = m->p_act; e.out = m->p_eout; e.plan = m->p_plan; e.s = s;
+        LUMEN_TRY(launch_experts_prefill(ctx, e));
+        p.y = m->p_eout; p.top = L.c.top; p.sel_w = m->p_selw;
+    } else {
+        const int F = pad8(L.c.ff);
+        LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_n, up, m->p_ff, s, F, W)));
+        LUMEN_TRY(launch_gelu(ctx, m->p_ff, m->p_ff, (size_t)s * F));
+        LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_ff, L.w_down, m->p_y, s, W, F)));
+    }
+    return sum(x, m->p_rg, W, L.rg2_b, next);
+}
+
 // s tokens (two or more) from the live state on; logits of the rows `want` [n_want] to logits_host.
 static int run_prompt(lumen_hybrid *m, const int32_t *ids, int s, const int *want, int n_want, float *logits_host, const Tap *tap) {
     const lumen_hybrid_config &c = m->cfg;
@@ -743,8 +1125,9 @@ static int run_prompt(lumen_hybrid *m, const int32_t *ids, int s, const int *wan
     const int W = m->W, V = c.vocab_size;
     LUMEN_TRY(ensure_prompt_buffers(m, s));
     HIP_TRY(hipMemcpyAsync(m->p_ids, ids, sizeof(int) * (size_t)s, hipMemcpyHostToDevice, ctx->stream));
-    LUMEN_TRY(launch_embedding(ctx, m->embed, m->p_ids, s, W, V, m->p_x0));
-    if (c.loop_times > 0) {
+    LUMEN_TRY(embed_rows(m, m->p_ids, s, nullptr, m->len, m->p_x0));
+    const bool mix = c.loop_times > 0 && c.loop_kind == LUMEN_LOOP_MIX, dyt = c.norm_kind == LUMEN_NORM_DYT;
+    if (mix) {
         LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_x0, m->loop_x0, m->p_n, s, W, W)));
         LUMEN_TRY(launch_add_steps(ctx, m->p_n, m->loop_step, m->p_steps, c.loop_times, s, W));
     }
@@ -762,11 +1145,26 @@ static int run_prompt(lumen_hybrid *m, const int32_t *ids, int s, const int *wan
         const Run &r = m->runs[ri];
         const Layer &L = m->layers[r.layer];
         const Run *next = ri + 1 < m->runs.size() ? &m->runs[ri + 1] : nullptr;
-        const float *next_norm = next && next->pass < 0 ? m->layers[next->layer].norm1 : nullptr;
-        if (r.pass >= 0)
+        const Layer *next_layer = next && next->pass < 0 ? &m->layers[next->layer] : nullptr;
+        const float *next_norm = next_layer ? next_layer->norm1 : nullptr;
+        if (r.pass >= 0 && !mix) {
+            float *y = cur == m->p_xa ? m->p_xb : m->p_xa;
+            LUMEN_TRY(launch_add_steps(ctx, cur, m->loop_step + (size_t)r.pass * W, y, 1, s, W));
+            cur = y;
+            normed = false;
+        } else if (r.pass >= 0)
             LUMEN_TRY(residual_gemm(gemm_args(m, cur, m->loop_x, cur == m->p_xa ? m->p_xb : m->p_xa, s, W, W),
                                     m->p_steps + (size_t)r.pass * s * W, 1.0f, L.norm1));
-        if (!normed) LUMEN_TRY(launch_rmsnorm(ctx, cur, L.norm1, m->p_n, s, W, m->eps_w));
+        if (!normed && dyt) LUMEN_TRY(launch_dyt(ctx, cur, L.norm1_a, L.norm1, L.norm1_b, m->p_n, s, W));
+        else if (!normed) LUMEN_TRY(launch_rmsnorm(ctx, cur, L.norm1, m->p_n, s, W, m->eps_w));
+        if (c.residual_gate) {
+            float *x = out();
+            LUMEN_TRY(prompt_gated_layer(m, L, r, s, cur, x, next_layer ? NormRef{next_layer->norm1, next_layer->norm1_b, next_layer->norm1_a} : NormRef{}));
+            cur = x;
+            normed = next_layer != nullptr;
+            LUMEN_TRY(tap_rows(m, tap, ri, cur, s));
+            continue;
+        }
         if (L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION) LUMEN_TRY(prompt_attention(m, L, r, s));
         else if (L.c.mixer == LUMEN_MIXER_WKV) LUMEN_TRY(prompt_wkv(m, L, r, s));
         else LUMEN_TRY(prompt_delta(m, L, r, s));
@@ -784,7 +1182,8 @@ static int run_prompt(lumen_hybrid *m, const int32_t *ids, int s, const int *wan
     LUMEN_TRY(sync_counters(m));
     if (n_want == 1) {
         GemvArgs g = gemv_args(m, m->head, V, W, cur + (size_t)want[0] * W, m->logits);
-        gemv_norm(m, g, m->final_norm);
+        gemv_norm(m, g, m->final_norm, m->final_b, m->final_a);
+        g.softcap = c.logit_softcap;
         LUMEN_TRY(launch_gemv(ctx, g));
         return lumen_download(ctx, logits_host, m->logits, sizeof(float) * (size_t)V);
     }
@@ -799,8 +1198,10 @@ static int run_prompt(lumen_hybrid *m, const int32_t *ids, int s, const int *wan
         }
         HIP_TRY(hipMemcpyAsync(m->p_idx, want, sizeof(int) * (size_t)n_want, hipMemcpyHostToDevice, ctx->stream));
         LUMEN_TRY(launch_gather_rows(ctx, cur, m->p_idx, m->p_rows, n_want, W));
-        LUMEN_TRY(launch_rmsnorm(ctx, m->p_rows, m->final_norm, m->p_n, n_want, W, m->eps_w));
+        if (dyt) LUMEN_TRY(launch_dyt(ctx, m->p_rows, m->final_a, m->final_norm, m->final_b, m->p_n, n_want, W));
+        else LUMEN_TRY(launch_rmsnorm(ctx, m->p_rows, m->final_norm, m->p_n, n_want, W, m->eps_w));
         LUMEN_TRY(launch_gemm(ctx, gemm_args(m, m->p_n, m->head, m->p_logits, n_want, V, W)));
+        if (c.logit_softcap > 0.f) LUMEN_TRY(launch_softcap(ctx, m->p_logits, c.logit_softcap, (size_t)n_want * V));
         return lumen_download(ctx, logits_host, m->p_logits, sizeof(float) * (size_t)n_want * V);
     }
     // (nothing to bring back: the ids' upload must still be done before the caller's array goes)
@@ -966,12 +1367,15 @@ extern "C" int lumen_hybrid_decode_bytes(const lumen_hybrid *m, int len, double 
     if (!m || !bytes_out) LUMEN_FAIL(LUMEN_ERR_INVALID, "hybrid_decode_bytes: null argument");
     const double W = m->W, e = (double)m->esz;
     double b = (double)m->cfg.vocab_size * W * e;
-    if (m->cfg.loop_times > 0) b += W * W * e * (1.0 + m->cfg.loop_times);
+    if (m->loop_x) b += W * W * e * (1.0 + m->cfg.loop_times);
     for (const Run &r : m->runs) {
         const Layer &L = m->layers[r.layer];
-        b += e * (W * L.n_proj + W * L.od + 2.0 * W * pad8(L.c.ff));
-        if (L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION) {
+        b += e * (W * L.n_proj + W * L.od + W * L.od2 + W * L.n_up);
+        if (L.c.ff_kind == LUMEN_FF_EXPERTS && L.c.ff > 0) b += e * 3.0 * W * pad8(L.c.ff) * L.c.top;
+        else b += e * W * pad8(L.c.ff);
+        if (L.c.mixer == LUMEN_MIXER_WINDOW_ATTENTION || L.c.mixer == LUMEN_MIXER_PARALLEL) {
             b += 4.0 * std::min(len, L.window) * L.c.kv_heads * (double)(L.c.dim + L.c.vdim);
+            if (r.st_matrix >= 0) b += 2.0 * 4.0 * (double)m->state->floats(r.st_matrix);
         } else {
             b += e * ((double)L.c.heads * L.c.dim * L.lo_rank + (double)L.c.heads * L.c.vdim * L.hi_rank);
             b += 2.0 * 4.0 * (double)m->state->floats(r.st_matrix);

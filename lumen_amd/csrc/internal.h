@@ -100,8 +100,9 @@ struct lumen_kv_cache {
 // element by element, N divides by the root mean square over norm_dim elements); norm_w = {a, b, c, e}.
 // PRO_SHIFT: RMSNorm, then the token-shift mix h + (h' - h) mu of h with the previous token's h'; gridDim.y products
 // at once, each with a mix of its own (GemvArgs::shift_*).
-enum GemvPro { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_ATTN_FOLD = 2, PRO_POLYNORM = 3, PRO_SHIFT = 4 };
-enum GemvEpi { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ARGMAX = 3, EPI_ROPE_QKV = 4 };
+// PRO_DYT: x enters as tanh(alpha x) norm_w + norm_b (Dynamic Tanh), alpha one float in device memory.
+enum GemvPro { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_ATTN_FOLD = 2, PRO_POLYNORM = 3, PRO_SHIFT = 4, PRO_DYT = 5 };
+enum GemvEpi { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ARGMAX = 3, EPI_ROPE_QKV = 4, EPI_EXPERT_ACT = 5 };
 
 struct GemvArgs {
     const void *W;        // [N, K] f32 or bf16 bits
@@ -110,10 +111,14 @@ struct GemvArgs {
     int N, K;
     int w_bf16;
     int pro, epi;
-    const float *norm_w;  // PRO_RMSNORM: gain [K]
+    const float *norm_w;  // PRO_RMSNORM, PRO_DYT: gain [K]
+    const float *norm_b, *norm_alpha;  // PRO_DYT: shift [K], one float
     float eps;
     const float *residual;  // EPI_RESIDUAL: [N]
     float alpha = 1.0f;     // EPI_RESIDUAL: y = residual + alpha * (W x)
+    const float *res_gate, *res_gate_b;  // EPI_RESIDUAL, or null: alpha is sigmoid(res_gate[row] + res_gate_b[row])
+    float softcap;          // EPI_STORE, EPI_ARGMAX, > 0: y = softcap tanh(W x / softcap) (the arg-max is taken before)
+    int gelu_from;          // EPI_STORE, > 0: rows from this one on are stored as their (erf) GELU
     int norm_dim;           // PRO_POLYNORM: elements the mean is taken over (0: K)
     // PRO_SHIFT: W holds shift_segs matrices one after the other, shift_rows rows each but shift_last_rows in the last;
     // segment s reads the mix of shift_mu [shift_segs][K].  h' is slot (*shift_step & 1) of shift_state [2][K]; the
@@ -150,6 +155,7 @@ struct GemvArgs {
     int attn_nslices, attn_d, attn_trip, attn_short_rows;
     int attn_window;         // > 0: at most that many rows are in use (a sliding window)
     const float *attn_gate;  // [K] or null: x is multiplied by the sigmoid of it
+    int attn_gate_heads;     // ... attn_gate holds one value per head
 };
 #define GEMV_FOLD_MAX_SLICES 16  // PRO_ATTN_FOLD reads this many slice states per element, whatever the count in use
 int launch_gemv(lumen_ctx *ctx, const GemvArgs &a);
@@ -186,12 +192,25 @@ struct GemmArgs {
     const float *norm_w;    // [N] or null
     float *norm_out;
     float norm_eps;
+    // products grouped by expert (launch_gemm_grouped): tile i of BM rows is {expert, first row, rows} of tiles, its weights the
+    // expert's of W [experts][N, K]; row r of the sorted rows reads row a_rows[r] of A (null: r) and is stored in row
+    // c_rows[r] of C (null: r).  Epilogues: store, or EPI_EXPERT_ACT: columns (2c, 2c + 1) = (gate, up) -> C [rows, N / 2]
+    const int *tiles, *a_rows, *c_rows;
+    float limit;
     // optional, with EPI_STORE: where K is split, leave the partial products [splits, M, N] in the workspace for a
     // consumer that adds them itself (in split order) and report how many there are; 1 = C holds the product
     int keep_splits;
     int *splits_used;
 };
 int launch_gemm(lumen_ctx *ctx, const GemmArgs &a);
+#define GEMM_GROUP_ROWS 128  // rows of a tile of a grouped product
+int launch_gemm_grouped(lumen_ctx *ctx, const GemmArgs &a, int max_tiles);  // M: total rows
+// act(gate, up) of a clamped expert
+__device__ __forceinline__ float expert_act(float g, float u, float limit) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
 int gemm_reserve_workspace(lumen_ctx *ctx, size_t bytes);  // grows the split-K workspace (synchronises the stream when it does)
 size_t gemm_workspace_bytes(const lumen_ctx *ctx, int M, int N, int K, int w_bf16);
 

@@ -21,17 +21,19 @@ __device__ __forceinline__ float tanh_w(float x) {
 
 // Scores are kept in log2 units (times log2 e), so that a weight is one base-2 exponential and the distance bias
 // r1 ln(1 + r2 d) is r1 log2(1 + r2 d).
+#define LOG2E 1.44269504088896341f
 struct ScoreShape {
     float in, out, r1, r2;  // score = out tanh(in dot), or in dot when out is 0
-    __device__ ScoreShape(float scale, float softcap, float r1_, float r2_) : r1(r1_), r2(r2_) {
-        const float log2e = 1.44269504088896341f;
+    bool log_bias;
+    __device__ ScoreShape(float scale, float softcap, float r1_, float r2_, bool log_bias_) : r1(r1_), r2(r2_), log_bias(log_bias_) {
+        const float log2e = LOG2E;
         in = softcap > 0.f ? scale / softcap : scale * log2e;
         out = softcap > 0.f ? softcap * log2e : 0.f;
     }
     __device__ float operator()(float dot, int dist) const {
         float s = in * dot;
         if (out > 0.f) s = out * tanh_w(s);
-        return less_bias(s, dist);
+        return log_bias ? less_bias(s, dist) : s;
     }
     // the same in steps, for a wavefront that looks at its scores together
     __device__ float capped_near(float x) const { return out * tanh_near(x); }
@@ -101,7 +103,9 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
     const int dq = min(tid, D - 1), dv = min(tid, Dv - 1);
     const float own_q = a.q[h * D + dq], own_k = a.k[hk * D + dq], own_v = a.v[hk * Dv + dv];
     const float gain_q = a.q_norm_w ? a.q_norm_w[h * D + dq] : 1.f, gain_k = a.k_norm_w ? a.k_norm_w[hk * D + dq] : 1.f;
-    const float gate = a.gate && a.slices == 1 ? a.gate[h * Dv + dv] : 0.f;
+    const float gate = a.gate && a.slices == 1 ? a.gate[a.gate_heads ? h : h * Dv + dv] : 0.f;
+    const float temp = a.temp ? a.temp[h] : 1.f, sink = a.sink ? a.sink[h] * LOG2E : -INFINITY;
+    const float tab = a.bias_tab ? a.bias_tab[(size_t)h * a.bias_n + min(max(pos - lo - tid, 0), a.bias_n - 1)] : 0.f;  // of key tid
     const float r1 = a.r1 ? a.r1[h] : 0.f, r2 = a.r1 ? a.r2[h] : 0.f;
     float sq = 0.f, sk = 0.f;
     if (a.q_norm_w) {
@@ -170,15 +174,16 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
         }
     }
     __syncthreads();
-    const ScoreShape shape(a.scale, a.softcap, r1, r2);
+    const ScoreShape shape(a.scale * temp, a.softcap, r1, r2, a.r1 != nullptr);
     float s = -INFINITY;
-    if (tid < n) s = shape(sc[tid], pos - lo - tid);
+    if (tid < n) s = shape(sc[tid], pos - lo - tid) + tab;
     float m = wave_max(s);
     if (lane == 0) red_m[wave] = m;
     __syncthreads();
     m = red_m[0];
 #pragma unroll
     for (int w = 1; w < WD_WAVES; ++w) m = fmaxf(m, red_m[w]);
+    if (slice == 0) m = fmaxf(m, sink);
     const float p = tid < n ? __builtin_amdgcn_exp2f(s - m) : 0.f;
     if (tid < WINDOW_SLICE_KEYS) sc[tid] = p;
     float l = wave_sum(p);
@@ -187,6 +192,7 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
     l = 0.f;
 #pragma unroll
     for (int w = 0; w < WD_WAVES; ++w) l += red_l[w];
+    if (slice == 0 && a.sink) l += __builtin_amdgcn_exp2f(sink - m);  // (once, whatever the number of slices)
 
     v4f acc = {0.f, 0.f, 0.f, 0.f};
     auto add = [&](int key, v4f v4) {
@@ -227,7 +233,7 @@ __global__ __launch_bounds__(256) void window_merge_kernel(WindowAttnArgs a) {
     for (int d = threadIdx.x; d < Dv; d += 256) {
         float o = 0.f;
         for (int s = 0; s < used; ++s) o = fmaf(part[(size_t)s * (Dv + 2) + d], __builtin_amdgcn_exp2f(part[(size_t)s * (Dv + 2) + Dv] - m), o);
-        a.out[h * Dv + d] = o / l * (a.gate ? gate_w(a.gate[h * Dv + d], a.gate_act) : 1.0f);
+        a.out[h * Dv + d] = o / l * (a.gate ? gate_w(a.gate[a.gate_heads ? h : h * Dv + d], a.gate_act) : 1.0f);
     }
 }
 
@@ -305,7 +311,9 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
     const int t0 = blockIdx.x * WP_Q, tw = t0 + wave * 16, t = tw + c;  // first token of the workgroup / wavefront, own token
     const int last = min(t0 + WP_Q, a.s) - 1;
     const int i = a.pos + t;  // own position
-    const ScoreShape shape(a.scale, a.softcap, a.r1 ? a.r1[h] : 0.f, a.r1 ? a.r2[h] : 0.f);
+    const ScoreShape shape(a.scale * (a.temp ? a.temp[h] : 1.f), a.softcap, a.r1 ? a.r1[h] : 0.f, a.r1 ? a.r2[h] : 0.f, a.r1 != nullptr);
+    const float *tab = a.bias_tab ? a.bias_tab + (size_t)h * a.bias_n : nullptr;
+    const float tab_far = tab ? tab[a.bias_n - 1] : 0.f;
     const float *kr = a.k_ring + (size_t)hk * a.cap * a.dpad, *vr = a.v_ring + (size_t)hk * a.cap * a.vpad;
 
     v4f qf[NB], acc[NB];
@@ -323,6 +331,10 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
         }
     }
     float m = -INFINITY, l = 0.f;
+    if (a.sink) {  // (the sums of the four lane groups of a query are added at the end: the sink counts in one of them)
+        m = a.sink[h] * LOG2E;
+        l = g == 0 ? 1.f : 0.f;
+    }
     const int j_first = max(0, a.pos + t0 - a.window + 1), j_last = a.pos + last;
     const int w_first = max(0, a.pos + tw - a.window + 1), w_last = a.pos + min(tw + 15, a.s - 1);  // of this wavefront
     // The tile in front travels in registers while this one is worked on.  Positions past the last key and channels past
@@ -398,10 +410,25 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
             sc[0] *= shape.in;
             sc[1] *= shape.in;
         }
+        if (shape.log_bias) {
 #pragma unroll
-        for (int u = 0; u < 2; ++u)
+            for (int u = 0; u < 2; ++u)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) sc[u][r] = shape.less_bias(sc[u][r], dist0 - (u * 16 + r));
+                for (int r = 0; r < 4; ++r) sc[u][r] = shape.less_bias(sc[u][r], dist0 - (u * 16 + r));
+        }
+        if (tab) {
+            if (a.pos + tw - (j0 + WP_K - 1) >= a.bias_n - 1) {  // (uniform: every distance of the tile is past the table)
+#pragma unroll
+                for (int u = 0; u < 2; ++u)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) sc[u][r] += tab_far;
+            } else {
+#pragma unroll
+                for (int u = 0; u < 2; ++u)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) sc[u][r] += tab[min(max(dist0 - (u * 16 + r), 0), a.bias_n - 1)];
+            }
+        }
         if (j0 + WP_K - 1 > a.pos + tw || j0 <= w_last - a.window) {  // (a tile every query of the wavefront sees whole needs no mask)
 #pragma unroll
             for (int u = 0; u < 2; ++u)
@@ -444,14 +471,14 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
     if (t >= a.s) return;
     const float inv = 1.0f / l;
     float *o = a.out + (size_t)t * a.out_stride + (size_t)h * Dv;
-    const float *gp = a.gate ? a.gate + (size_t)t * a.stride + (size_t)h * Dv : nullptr;
+    const float *gp = a.gate ? a.gate + (size_t)t * a.stride + (a.gate_heads ? (size_t)h : (size_t)h * Dv) : nullptr;
 #pragma unroll
     for (int b = 0; b < NB; ++b)
         if (b < nv) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int d = b * 16 + g * 4 + r;
-                if (d < Dv) o[d] = acc[b][r] * inv * (gp ? gate_w(gp[d], a.gate_act) : 1.0f);
+                if (d < Dv) o[d] = acc[b][r] * inv * (gp ? gate_w(gp[a.gate_heads ? 0 : d], a.gate_act) : 1.0f);
             }
         }
 }

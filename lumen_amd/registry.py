@@ -10,7 +10,7 @@ import os
 
 from . import _lib
 from ._lib import ERR_INVALID, LumenError, check, lib
-from .hybrid import HybridModel, pinavik_config
+from .hybrid import HybridModel, nufapel_config, pinavik_config
 from .models import LlamaConfig, LlamaModel
 
 ARCHITECTURES = {}
@@ -40,6 +40,11 @@ def _llama(cfg, shape_of, max_seq_len, weight_dtype):
 @register("Pinavik")
 def _pinavik(cfg, shape_of, max_seq_len, weight_dtype):
     return HybridModel(pinavik_config(cfg, shape_of, max_seq_len, weight_dtype))
+
+
+@register("Nufapel")
+def _nufapel(cfg, shape_of, max_seq_len, weight_dtype):
+    return HybridModel(nufapel_config(cfg, shape_of, max_seq_len, weight_dtype))
 
 
 def tensor_shape(path, name):

@@ -71,6 +71,19 @@ static inline T __shfl_xor(T v, int off, int width = 64) {
     (void)width;
     return emu_bits_to<T>(emu::wave_exchange(emu_bits_of(v), (int)((threadIdx.x & 63) ^ (unsigned)off)));
 }
+template <typename T>
+static inline T __shfl_up(T v, unsigned off, int width = 64) {
+    (void)width;
+    const int lane = (int)(threadIdx.x & 63);
+    return emu_bits_to<T>(emu::wave_exchange(emu_bits_of(v), lane >= (int)off ? lane - (int)off : lane));
+}
+template <typename T>
+static inline T __shfl(T v, int from, int width = 64) {
+    (void)width;
+    return emu_bits_to<T>(emu::wave_exchange(emu_bits_of(v), from));
+}
+static inline unsigned __umulhi(unsigned a, unsigned b) { return (unsigned)(((uint64_t)a * b) >> 32); }
+static inline int atomicAdd(int *p, int v) { return __atomic_fetch_add(p, v, __ATOMIC_SEQ_CST); }
 // DPP row_ror:n (control 0x121 .. 0x12f): lane i of a row of 16 lanes receives the value of lane (i - n) mod 16
 static inline int emu_update_dpp(int src, int ctrl) {
     if (ctrl < 0x121 || ctrl > 0x12f) emu::not_emulated("DPP control other than row_ror");
