@@ -508,6 +508,34 @@ int lumen_channel_delta_f32(lumen_ctx *ctx, const float *q_dev, const float *k_d
  * unit q and k; prev / next [taps - 1, channels]: inputs before the first / up to the last token, oldest first */
 int lumen_conv_unit_f32(lumen_ctx *ctx, const float *qkv_dev, const float *taps_dev, const float *prev_dev, float *next_dev, float *q_dev,
                         float *k_dev, float *v_dev, int s, int taps, int heads, int kv_heads, int dim, int vdim, float unit_eps, float q_scale);
+/* tanh(*alpha x) w + b, rows of dim */
+int lumen_dynamic_tanh_f32(lumen_ctx *ctx, const float *x_dev, const float *alpha_dev, const float *w_dev, const float *b_dev, float *out_dev,
+                           int rows, int dim);
+/* out = x + sigmoid(gate + gate_b) v, v being y, or with y2 pair_scale (N(y) w1 + N(y2) w2), N an RMS norm over the first `width` of the rows'
+ * dim elements (a multiple of 4; the others zero) */
+int lumen_gated_residual_f32(lumen_ctx *ctx, const float *x_dev, const float *y_dev, const float *y2_dev, const float *w1_dev, const float *w2_dev,
+                             const float *gate_dev, const float *gate_b_dev, float *out_dev, int rows, int dim, int width, float pair_scale, float eps);
+/* generalised delta rule: r, k, z, a [s, heads, dim], v [s, heads, vdim]; decay exp(-e^{-1/2} sigmoid(z + z_bias)), removal rate sigmoid(a + a_bias),
+ * both biases [heads, dim]; state [heads, vdim, rows] */
+int lumen_general_delta_f32(lumen_ctx *ctx, const float *r_dev, const float *k_dev, const float *v_dev, const float *z_dev, const float *a_dev,
+                            const float *z_bias_dev, const float *a_bias_dev, float *state_dev, float *out_dev, int s, int heads, int dim, int vdim,
+                            float unit_eps);
+/* matrix memory: q, k [s, heads, dim], v [s, heads, vdim], gates i, f [s, heads] before bias and cap; state [heads, vdim + 1, rows], its last column the
+ * normaliser; m [heads] the running maxima (0 at the start).  out [s, heads, vdim]: read, RMS norm per head, times gain [heads, vdim] */
+int lumen_matrix_memory_f32(lumen_ctx *ctx, const float *q_dev, const float *k_dev, const float *v_dev, const float *i_dev, const float *f_dev,
+                            const float *i_bias_dev, const float *f_bias_dev, const float *gain_dev, float *state_dev, float *m_dev, float *out_dev,
+                            int s, int heads, int dim, int vdim, float cap, float eps);
+/* lumen_window_attn_f32 without norms, cap and logarithmic bias, with: temp [heads] times the scale, bias_tab [heads, bias_n] times log2 e (distances past
+ * its end take the last entry), sink [heads] in the softmax's denominator, gate [s, heads] (before the sigmoid); each may be NULL */
+int lumen_biased_attn_f32(lumen_ctx *ctx, const float *q_dev, const float *k_dev, const float *v_dev, const float *gate_dev, const float *temp_dev,
+                          const float *bias_tab_dev, int bias_n, const float *sink_dev, float *k_ring_dev, float *v_ring_dev, int cap, float *out_dev,
+                          int s, int pos, int heads, int kv_heads, int dim, int vdim, int window, float scale);
+/* router logits z [rows, experts] -> sel [rows, top] (device ints), w [rows, top]; groups, keep, scale as in lumen_hybrid_layer */
+int lumen_route_f32(lumen_ctx *ctx, const float *z_dev, int *sel_dev, float *w_dev, int rows, int experts, int groups, int keep, int top, float scale);
+/* h [s, dim], z [s, experts]; w_up [experts, 2 ff, dim] (gate and up rows in turn), w_down [experts, dim, ff], f32 or bf16, sizes multiples of 8;
+ * out [s, top, dim] not weighted yet, w [s, top] */
+int lumen_experts_f32(lumen_ctx *ctx, const float *h_dev, const float *z_dev, const void *w_up_dev, const void *w_down_dev, int w_bf16, float *out_dev,
+                      float *w_dev, int s, int dim, int ff, int experts, int groups, int keep, int top, float scale, float limit);
 /* o [rows, heads, vdim] in place: RMS norm per head, times gain, times act(gate) (0 none, 1 sigmoid, 2 silu) */
 int lumen_head_norm_gate_f32(lumen_ctx *ctx, float *o_dev, const float *gain_dev, int gain_shared, const float *gate_dev, int gate_act, int rows,
                              int heads, int vdim, float eps);

@@ -160,6 +160,13 @@ SIGNATURES = {
     "lumen_channel_delta_f32": (_i, [_vp] * 10 + [_i] * 5),
     "lumen_conv_unit_f32": (_i, [_vp] * 8 + [_i] * 6 + [_f] * 2),
     "lumen_head_norm_gate_f32": (_i, [_vp, _vp, _vp, _i, _vp, _i, _i, _i, _i, _f]),
+    "lumen_dynamic_tanh_f32": (_i, [_vp] * 6 + [_i] * 2),
+    "lumen_gated_residual_f32": (_i, [_vp] * 9 + [_i] * 3 + [_f] * 2),
+    "lumen_general_delta_f32": (_i, [_vp] * 10 + [_i] * 4 + [_f]),
+    "lumen_matrix_memory_f32": (_i, [_vp] * 12 + [_i] * 4 + [_f] * 2),
+    "lumen_biased_attn_f32": (_i, [_vp] * 7 + [_i] + [_vp] * 3 + [_i, _vp] + [_i] * 7 + [_f]),
+    "lumen_route_f32": (_i, [_vp] * 4 + [_i] * 5 + [_f]),
+    "lumen_experts_f32": (_i, [_vp] * 5 + [_i] + [_vp] * 2 + [_i] * 7 + [_f] * 2),
     "lumen_window_attn_f32": (_i, [_vp] * 11 + [_i, _vp] + [_i] * 7 + [_f] * 3),
 }
 

@@ -1449,18 +1449,108 @@ extern "C" int lumen_head_norm_gate_f32(lumen_ctx *ctx, float *o, const float *g
     return launch_head_norm_gate(ctx, o, heads * vdim, gain, gain_shared, gate, heads * vdim, gate_act, rows, heads, vdim, eps);
 }
 
-extern "C" int lumen_window_attn_f32(lumen_ctx *ctx, const float *q, const float *k, const float *v, const float *gate, const float *q_norm,
-                                     const float *k_norm, const float *r1, const float *r2, float *k_ring, float *v_ring, int cap, float *out,
-                                     int s, int pos, int heads, int kv_heads, int dim, int vdim, int window, float scale, float softcap,
-                                     float norm_eps) {
+extern "C" int lumen_dynamic_tanh_f32(lumen_ctx *ctx, const float *x, const float *alpha, const float *w, const float *b, float *out, int rows, int dim) {
+    if (!ctx || !x || !alpha || !w || !b || !out) LUMEN_FAIL(LUMEN_ERR_INVALID, "dynamic_tanh: null argument");
+    if (rows < 0 || dim <= 0) LUMEN_FAIL(LUMEN_ERR_SHAPE, "dynamic_tanh: rows=%d dim=%d", rows, dim);
+    return launch_dyt(ctx, x, alpha, w, b, out, rows, dim);
+}
+
+extern "C" int lumen_gated_residual_f32(lumen_ctx *ctx, const float *x, const float *y, const float *y2, const float *w1, const float *w2,
+                                        const float *gate, const float *gate_b, float *out, int rows, int dim, int width, float pair_scale, float eps) {
+    if (!ctx || !x || !y || !gate || !gate_b || !out || (y2 && (!w1 || !w2))) LUMEN_FAIL(LUMEN_ERR_INVALID, "gated_residual: null argument");
+    if (rows < 0 || dim <= 0 || dim % 4 || width <= 0 || width > dim) LUMEN_FAIL(LUMEN_ERR_SHAPE, "gated_residual: rows=%d dim=%d width=%d", rows, dim, width);
+    GatedResidualArgs a = {};
+    a.x = x; a.y = y; a.y2 = y2; a.w1 = w1; a.w2 = w2; a.gate = gate; a.gate_stride = dim; a.gate_b = gate_b; a.out = out;
+    a.rows = rows; a.dim = dim; a.width = width; a.pair_scale = pair_scale; a.eps = eps;
+    return launch_gated_residual(ctx, a);
+}
+
+extern "C" int lumen_general_delta_f32(lumen_ctx *ctx, const float *r, const float *k, const float *v, const float *z, const float *a_raw,
+                                       const float *z_bias, const float *a_bias, float *state, float *out, int s, int heads, int dim, int vdim,
+                                       float unit_eps) {
+    if (!ctx || !r || !k || !v || !z || !a_raw || !z_bias || !a_bias || !state || !out) LUMEN_FAIL(LUMEN_ERR_INVALID, "general_delta: null argument");
+    if (s < 0 || heads <= 0 || dim <= 0 || vdim <= 0 || dim > MIX_MAX_DIM || vdim > MIX_MAX_DIM)
+        LUMEN_FAIL(LUMEN_ERR_SHAPE, "general_delta: s=%d heads=%d dim=%d vdim=%d", s, heads, dim, vdim);
+    RecurrenceArgs a = {};
+    a.kind = REC_GENERAL; a.heads = heads; a.rep = 1; a.dim = dim; a.vdim = vdim; a.s = s;
+    a.q = r; a.k = k; a.v = v; a.z = z; a.b = a_raw; a.bias = z_bias; a.b_bias = a_bias; a.unit_eps = unit_eps; a.z_scale = GENERAL_DECAY;
+    a.q_stride = a.k_stride = a.z_stride = a.b_stride = heads * dim; a.v_stride = a.out_stride = heads * vdim;
+    a.state = state; a.out = out;
+    return launch_recurrence(ctx, a);
+}
+
+extern "C" int lumen_matrix_memory_f32(lumen_ctx *ctx, const float *q, const float *k, const float *v, const float *gi, const float *gf,
+                                       const float *i_bias, const float *f_bias, const float *gain, float *state, float *m, float *out, int s, int heads,
+                                       int dim, int vdim, float cap, float eps) {
+    if (!ctx || !q || !k || !v || !gi || !gf || !i_bias || !f_bias || !gain || !state || !m || !out)
+        LUMEN_FAIL(LUMEN_ERR_INVALID, "matrix_memory: null argument");
+    if (s <= 0 || heads <= 0 || dim <= 0 || vdim <= 0 || dim > MIX_MAX_DIM || vdim > MIX_MAX_DIM || !(cap > 0.f))
+        LUMEN_FAIL(LUMEN_ERR_SHAPE, "matrix_memory: s=%d heads=%d dim=%d vdim=%d cap=%g", s, heads, dim, vdim, cap);
+    float *raw = nullptr, *scan = nullptr;
+    auto run = [&]() {
+        HIP_TRY(hipMalloc((void **)&raw, sizeof(float) * (size_t)s * heads * (vdim + 1)));
+        HIP_TRY(hipMalloc((void **)&scan, sizeof(float) * memory_scan_floats(s, heads)));
+        RecurrenceArgs a = {};
+        a.kind = REC_MEMORY; a.heads = heads; a.rep = 1; a.dim = dim; a.vdim = vdim; a.s = s;
+        a.q = q; a.k = k; a.v = v; a.gi = gi; a.gf = gf; a.gi_bias = i_bias; a.gf_bias = f_bias; a.g_stride = heads; a.cap = cap;
+        a.q_stride = a.k_stride = heads * dim; a.v_stride = heads * vdim; a.q_scale = 1.0f / sqrtf((float)dim);
+        a.m = m; a.m_out = scan; a.state = state; a.out = raw; a.out_stride = heads * (vdim + 1);
+        LUMEN_TRY(launch_recurrence(ctx, a));
+        return launch_memory_read(ctx, raw, scan, out, heads * vdim, gain, nullptr, 0, GATE_NONE, s, heads, vdim, eps, MEMORY_DEN_EPS);
+    };
+    const int rc = run();
+    hipStreamSynchronize(ctx->stream);
+    hipFree(raw);
+    hipFree(scan);
+    return rc;
+}
+
+static int check_router(const char *what, int rows, int experts, int groups, int keep, int top) {
+    if (rows < 0 || experts <= 0 || groups <= 0 || experts % groups || keep <= 0 || keep > groups || top <= 0 || top > keep * (experts / groups))
+        LUMEN_FAIL(LUMEN_ERR_SHAPE, "%s: %d rows, %d of %d experts, %d of %d groups", what, rows, top, experts, keep, groups);
+    if (experts > EXPERTS_MAX || top > EXPERTS_MAX_TOP) LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "%s: %d experts, %d at a time", what, experts, top);
+    return LUMEN_OK;
+}
+
+extern "C" int lumen_route_f32(lumen_ctx *ctx, const float *z, int *sel, float *w, int rows, int experts, int groups, int keep, int top, float scale) {
+    if (!ctx || !z || !sel || !w) LUMEN_FAIL(LUMEN_ERR_INVALID, "route: null argument");
+    LUMEN_TRY(check_router("route", rows, experts, groups, keep, top));
+    return launch_route(ctx, RouterShape{experts, groups, keep, top, scale}, z, experts, rows, sel, w);
+}
+
+extern "C" int lumen_experts_f32(lumen_ctx *ctx, const float *h, const float *z, const void *w_up, const void *w_down, int w_bf16, float *out, float *w,
+                                 int s, int dim, int ff, int experts, int groups, int keep, int top, float scale, float limit) {
+    if (!ctx || !h || !z || !w_up || !w_down || !out || !w) LUMEN_FAIL(LUMEN_ERR_INVALID, "experts: null argument");
+    LUMEN_TRY(check_router("experts", s, experts, groups, keep, top));
+    if (dim <= 0 || ff <= 0 || dim % 8 || ff % 8) LUMEN_FAIL(LUMEN_ERR_SHAPE, "experts: dim=%d ff=%d", dim, ff);
+    float *act = nullptr;
+    int *plan = nullptr;
+    ExpertsArgs e = {};
+    e.r = RouterShape{experts, groups, keep, top, scale};
+    auto run = [&]() {
+        HIP_TRY(hipMalloc((void **)&act, sizeof(float) * (size_t)s * top * ff + 16));
+        HIP_TRY(hipMalloc((void **)&plan, sizeof(int) * experts_plan_ints(s, e.r) + 16));
+        e.w_up = w_up; e.w_down = w_down; e.w_bf16 = w_bf16; e.dim = dim; e.ff = ff; e.limit = limit; e.z = z; e.z_stride = experts;
+        e.rows = h; e.sel_w = w; e.p_act = act; e.out = out; e.plan = plan; e.s = s;
+        return launch_experts_prefill(ctx, e);
+    };
+    const int rc = run();
+    hipStreamSynchronize(ctx->stream);
+    hipFree(act);
+    hipFree(plan);
+    return rc;
+}
+
+// One operator call of the window attention; `shape` holds what differs from caller to caller.
+static int window_attn_operator(lumen_ctx *ctx, const float *q, const float *k, const float *v, const float *gate, float *k_ring, float *v_ring, int cap,
+                                float *out, int s, int pos, int heads, int kv_heads, int dim, int vdim, int window, const WindowAttnArgs &shape) {
     if (!ctx || !q || !k || !v || !k_ring || !v_ring || !out) LUMEN_FAIL(LUMEN_ERR_INVALID, "window_attn: null argument");
     if (s <= 0 || pos < 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads || dim <= 0 || vdim <= 0 || window <= 0)
         LUMEN_FAIL(LUMEN_ERR_SHAPE, "window_attn: s=%d pos=%d heads=%d/%d dim=%d vdim=%d window=%d", s, pos, heads, kv_heads, dim, vdim, window);
     if (dim > MIX_MAX_DIM || vdim > MIX_MAX_DIM) LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "window_attn: heads wider than %d", MIX_MAX_DIM);
     if (cap < window - 1 + s) LUMEN_FAIL(LUMEN_ERR_KV_OVERFLOW, "window_attn: ring of %d positions for a window of %d and %d tokens", cap, window, s);
-    if ((r1 == nullptr) != (r2 == nullptr)) LUMEN_FAIL(LUMEN_ERR_INVALID, "window_attn: one of the two bias vectors");
     // the projections as the model lays them out: one row of q | k | v | gate blocks per token
-    const int nq = heads * dim, nk = kv_heads * dim, nv = kv_heads * vdim, no = heads * vdim, stride = nq + nk + nv + (gate ? no : 0);
+    const int nq = heads * dim, nk = kv_heads * dim, nv = kv_heads * vdim, ng = shape.gate_heads ? heads : heads * vdim, stride = nq + nk + nv + (gate ? ng : 0);
     float *rows = nullptr, *qn = nullptr, *part = nullptr;
     int *d_pos = nullptr;
     const int slices = window_attn_slices(window);
@@ -1470,7 +1560,7 @@ extern "C" int lumen_window_attn_f32(lumen_ctx *ctx, const float *q, const float
         HIP_TRY(hipMalloc((void **)&part, sizeof(float) * (size_t)heads * slices * (vdim + 2)));
         HIP_TRY(hipMalloc((void **)&d_pos, sizeof(int)));
         const float *src[4] = {q, k, v, gate};
-        const int n[4] = {nq, nk, nv, no};
+        const int n[4] = {nq, nk, nv, ng};
         size_t off[4] = {0, 0, 0, 0}, at = 0;
         for (int i = 0; i < (gate ? 4 : 3); ++i) {
             off[i] = at;
@@ -1478,12 +1568,12 @@ extern "C" int lumen_window_attn_f32(lumen_ctx *ctx, const float *q, const float
             at += n[i];
         }
         HIP_TRY(hipMemcpyAsync(d_pos, &pos, sizeof(int), hipMemcpyHostToDevice, ctx->stream));
-        WindowAttnArgs a = {};
+        WindowAttnArgs a = shape;
         a.q = rows; a.k = rows + off[1]; a.v = rows + off[2]; a.gate = gate ? rows + off[3] : nullptr; a.stride = stride;
-        a.out = out; a.out_stride = no; a.q_norm_w = q_norm; a.k_norm_w = k_norm; a.norm_eps = norm_eps;
+        a.out = out; a.out_stride = heads * vdim;
         a.k_ring = k_ring; a.v_ring = v_ring; a.cap = cap; a.dpad = (dim + 3) & ~3; a.vpad = (vdim + 3) & ~3;
         a.heads = heads; a.kv_heads = kv_heads; a.dim = dim; a.vdim = vdim; a.window = window; a.gate_act = gate ? GATE_SIGMOID : GATE_NONE;
-        a.scale = scale; a.softcap = softcap; a.r1 = r1; a.r2 = r2; a.pos_dev = d_pos; a.pos = pos; a.s = s; a.qn = qn; a.part = part; a.slices = slices;
+        a.pos_dev = d_pos; a.pos = pos; a.s = s; a.qn = qn; a.part = part; a.slices = slices;
         return s == 1 ? launch_window_attn_decode(ctx, a) : launch_window_attn_prefill(ctx, a);
     };
     const int rc = run();
@@ -1493,4 +1583,23 @@ extern "C" int lumen_window_attn_f32(lumen_ctx *ctx, const float *q, const float
     hipFree(part);
     hipFree(d_pos);
     return rc;
+}
+
+extern "C" int lumen_window_attn_f32(lumen_ctx *ctx, const float *q, const float *k, const float *v, const float *gate, const float *q_norm,
+                                     const float *k_norm, const float *r1, const float *r2, float *k_ring, float *v_ring, int cap, float *out,
+                                     int s, int pos, int heads, int kv_heads, int dim, int vdim, int window, float scale, float softcap,
+                                     float norm_eps) {
+    if ((r1 == nullptr) != (r2 == nullptr)) LUMEN_FAIL(LUMEN_ERR_INVALID, "window_attn: one of the two bias vectors");
+    WindowAttnArgs a = {};
+    a.q_norm_w = q_norm; a.k_norm_w = k_norm; a.norm_eps = norm_eps; a.scale = scale; a.softcap = softcap; a.r1 = r1; a.r2 = r2;
+    return window_attn_operator(ctx, q, k, v, gate, k_ring, v_ring, cap, out, s, pos, heads, kv_heads, dim, vdim, window, a);
+}
+
+extern "C" int lumen_biased_attn_f32(lumen_ctx *ctx, const float *q, const float *k, const float *v, const float *gate, const float *temp,
+                                     const float *bias_tab, int bias_n, const float *sink, float *k_ring, float *v_ring, int cap, float *out, int s, int pos,
+                                     int heads, int kv_heads, int dim, int vdim, int window, float scale) {
+    if (bias_tab && bias_n < 1) LUMEN_FAIL(LUMEN_ERR_SHAPE, "biased_attn: a bias table of %d", bias_n);
+    WindowAttnArgs a = {};
+    a.scale = scale; a.temp = temp; a.bias_tab = bias_tab; a.bias_n = bias_n; a.sink = sink; a.gate_heads = 1;
+    return window_attn_operator(ctx, q, k, v, gate, k_ring, v_ring, cap, out, s, pos, heads, kv_heads, dim, vdim, window, a);
 }

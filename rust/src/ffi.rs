@@ -27,6 +27,11 @@ pub struct lumen_hybrid_config {
     pub max_seq_len: c_int,
     pub max_chunk: c_int,
     pub weight_dtype: c_int,
+    pub norm_kind: c_int,
+    pub loop_kind: c_int,
+    pub residual_gate: c_int,
+    pub max_positions: c_int,
+    pub logit_softcap: c_float,
 }
 
 #[repr(C)]
@@ -44,6 +49,19 @@ pub struct lumen_hybrid_layer {
     pub rank_lo: c_int,
     pub rank_hi: c_int,
     pub ff: c_int,
+    pub ff_kind: c_int,
+    pub bias_rows: c_int,
+    pub bias_max: c_int,
+    pub mem_heads: c_int,
+    pub mem_dim: c_int,
+    pub mem_vdim: c_int,
+    pub gate_cap: c_float,
+    pub experts: c_int,
+    pub top: c_int,
+    pub groups: c_int,
+    pub keep: c_int,
+    pub router_scale: c_float,
+    pub limit: c_float,
 }
 
 #[repr(C)]
@@ -98,6 +116,15 @@ pub const LUMEN_DECODE_PERSISTENT: c_int = 2;
 pub const LUMEN_MIXER_WINDOW_ATTENTION: c_int = 0;
 pub const LUMEN_MIXER_WKV: c_int = 1;
 pub const LUMEN_MIXER_CHANNEL_DELTA: c_int = 2;
+pub const LUMEN_MIXER_GENERAL_DELTA: c_int = 3;
+pub const LUMEN_MIXER_PARALLEL: c_int = 4;
+pub const LUMEN_FF_POLYNORM: c_int = 0;
+pub const LUMEN_FF_GELU: c_int = 1;
+pub const LUMEN_FF_EXPERTS: c_int = 2;
+pub const LUMEN_NORM_RMS: c_int = 0;
+pub const LUMEN_NORM_DYT: c_int = 1;
+pub const LUMEN_LOOP_MIX: c_int = 0;
+pub const LUMEN_LOOP_ADD: c_int = 1;
 
 extern "C" {
     pub fn lumen_last_error() -> *const c_char;
@@ -195,6 +222,13 @@ extern "C" {
     pub fn lumen_wkv_f32(ctx: *mut lumen_ctx, r_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, z_dev: *const c_float, bias_dev: *const c_float, u_dev: *const c_float, state_dev: *mut c_float, out_dev: *mut c_float, s: c_int, heads: c_int, dim: c_int) -> c_int;
     pub fn lumen_channel_delta_f32(ctx: *mut lumen_ctx, q_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, z_dev: *const c_float, b_dev: *const c_float, bias_dev: *const c_float, a_log_dev: *const c_float, state_dev: *mut c_float, out_dev: *mut c_float, s: c_int, heads: c_int, kv_heads: c_int, dim: c_int, vdim: c_int) -> c_int;
     pub fn lumen_conv_unit_f32(ctx: *mut lumen_ctx, qkv_dev: *const c_float, taps_dev: *const c_float, prev_dev: *const c_float, next_dev: *mut c_float, q_dev: *mut c_float, k_dev: *mut c_float, v_dev: *mut c_float, s: c_int, taps: c_int, heads: c_int, kv_heads: c_int, dim: c_int, vdim: c_int, unit_eps: c_float, q_scale: c_float) -> c_int;
+    pub fn lumen_dynamic_tanh_f32(ctx: *mut lumen_ctx, x_dev: *const c_float, alpha_dev: *const c_float, w_dev: *const c_float, b_dev: *const c_float, out_dev: *mut c_float, rows: c_int, dim: c_int) -> c_int;
+    pub fn lumen_gated_residual_f32(ctx: *mut lumen_ctx, x_dev: *const c_float, y_dev: *const c_float, y2_dev: *const c_float, w1_dev: *const c_float, w2_dev: *const c_float, gate_dev: *const c_float, gate_b_dev: *const c_float, out_dev: *mut c_float, rows: c_int, dim: c_int, width: c_int, pair_scale: c_float, eps: c_float) -> c_int;
+    pub fn lumen_general_delta_f32(ctx: *mut lumen_ctx, r_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, z_dev: *const c_float, a_dev: *const c_float, z_bias_dev: *const c_float, a_bias_dev: *const c_float, state_dev: *mut c_float, out_dev: *mut c_float, s: c_int, heads: c_int, dim: c_int, vdim: c_int, unit_eps: c_float) -> c_int;
+    pub fn lumen_matrix_memory_f32(ctx: *mut lumen_ctx, q_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, i_dev: *const c_float, f_dev: *const c_float, i_bias_dev: *const c_float, f_bias_dev: *const c_float, gain_dev: *const c_float, state_dev: *mut c_float, m_dev: *mut c_float, out_dev: *mut c_float, s: c_int, heads: c_int, dim: c_int, vdim: c_int, cap: c_float, eps: c_float) -> c_int;
+    pub fn lumen_biased_attn_f32(ctx: *mut lumen_ctx, q_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, gate_dev: *const c_float, temp_dev: *const c_float, bias_tab_dev: *const c_float, bias_n: c_int, sink_dev: *const c_float, k_ring_dev: *mut c_float, v_ring_dev: *mut c_float, cap: c_int, out_dev: *mut c_float, s: c_int, pos: c_int, heads: c_int, kv_heads: c_int, dim: c_int, vdim: c_int, window: c_int, scale: c_float) -> c_int;
+    pub fn lumen_route_f32(ctx: *mut lumen_ctx, z_dev: *const c_float, sel_dev: *mut c_int, w_dev: *mut c_float, rows: c_int, experts: c_int, groups: c_int, keep: c_int, top: c_int, scale: c_float) -> c_int;
+    pub fn lumen_experts_f32(ctx: *mut lumen_ctx, h_dev: *const c_float, z_dev: *const c_float, w_up_dev: *const c_void, w_down_dev: *const c_void, w_bf16: c_int, out_dev: *mut c_float, w_dev: *mut c_float, s: c_int, dim: c_int, ff: c_int, experts: c_int, groups: c_int, keep: c_int, top: c_int, scale: c_float, limit: c_float) -> c_int;
     pub fn lumen_head_norm_gate_f32(ctx: *mut lumen_ctx, o_dev: *mut c_float, gain_dev: *const c_float, gain_shared: c_int, gate_dev: *const c_float, gate_act: c_int, rows: c_int, heads: c_int, vdim: c_int, eps: c_float) -> c_int;
     pub fn lumen_window_attn_f32(ctx: *mut lumen_ctx, q_dev: *const c_float, k_dev: *const c_float, v_dev: *const c_float, gate_dev: *const c_float, q_norm_dev: *const c_float, k_norm_dev: *const c_float, r1_dev: *const c_float, r2_dev: *const c_float, k_ring_dev: *mut c_float, v_ring_dev: *mut c_float, cap: c_int, out_dev: *mut c_float, s: c_int, pos: c_int, heads: c_int, kv_heads: c_int, dim: c_int, vdim: c_int, window: c_int, scale: c_float, softcap: c_float, norm_eps: c_float) -> c_int;
 }
