@@ -54,17 +54,18 @@ def main():
     ap.add_argument("--resident", action="store_true",
                     help="--workload gemv: every launch reads the SAME copy of W (what the caches hold counts: the "
                          "figure is no longer HBM bandwidth); default: >= 1.2 GB of copies in rotation")
-    ap.add_argument("--workload", choices=["decode", "gemv", "gemm", "prefill", "copy", "hybrid"], default="decode",
+    ap.add_argument("--workload", choices=["decode", "gemv", "gemm", "prefill", "copy", "hybrid", "nufapel"], default="decode",
                     help="decode: the headline batch-1 decode benchmark; gemv: the isolated M=1 GEMV shapes; "
                          "gemm: the prompt-pass GEMM shapes against the fp32 matrix-core peak; prefill: one long "
                          "prompt pass (3968 tokens, TinyLlama shape with a 4096-row cache); "
                          "copy: a plain 1 GiB copy kernel (calibrates the FETCH_SIZE / WRITE_SIZE counters); "
                          "hybrid: prompt passes and decode of the layered hybrid decoder (Pinavik) beside a Llama of "
-                         "equal size (--hybrid-width, --hybrid-dtype)")
+                         "equal size (--hybrid-width, --hybrid-dtype); nufapel: the same of the Nufapel design, beside the "
+                         "hybrid decoder")
     ap.add_argument("--hybrid-width", type=int, default=2048, help="--workload hybrid: width of both models (a multiple of 256)")
     ap.add_argument("--hybrid-dtype", choices=["bf16", "f32"], default="bf16", help="--workload hybrid: storage of the matrices")
-    ap.add_argument("--hybrid-only", choices=["hybrid", "llama"], default=None,
-                    help="--workload hybrid: one of the two models (for a kernel trace)")
+    ap.add_argument("--hybrid-only", choices=["hybrid", "llama", "nufapel"], default=None,
+                    help="--workload hybrid, nufapel: one of the two models (for a kernel trace)")
     args = ap.parse_args()
     if args.gpus != 1:
         sys.exit("bench.py: this build runs the batch-1 decode path on ONE GPU; --gpus %d is not supported "
@@ -78,7 +79,7 @@ def main():
         return gemm_microbench(args)
     if args.workload == "prefill":
         return prefill_bench(args)
-    if args.workload == "hybrid":
+    if args.workload in ("hybrid", "nufapel"):
         return hybrid_bench(args)
 
     import numpy as np
@@ -466,15 +467,23 @@ def hybrid_bench(args):
     W, dt = args.hybrid_width, args.hybrid_dtype
     steps, warmup = args.steps, args.warmup
     rows = {}
-    for name in ("hybrid", "llama"):
+    for name in ("hybrid", "llama") if args.workload == "hybrid" else ("nufapel", "hybrid"):
         if args.hybrid_only not in (None, name):
             continue
         t0 = time.time()
-        if name == "hybrid":
-            cfg = synth.hybrid_shape(W, dt)
+        if name in ("hybrid", "nufapel"):
+            cfg = synth.hybrid_shape(W, dt) if name == "hybrid" else synth.nufapel_shape(W, dt)
+            make, same = synth.hybrid_param if name == "hybrid" else synth.nufapel_param, {}
             model = HybridModel(cfg)
             shapes = model.named_parameter_shapes()
-            one = lambda n: synth.hybrid_param(n, shapes[n], 0)  # noqa: E731
+
+            def one(n):  # (the experts of a model share their values: there are gigabytes of them)
+                if ".mlp.e" not in n:
+                    return make(n, shapes[n], 0)
+                key = n.split(".")[-1]
+                if key not in same:
+                    same[key] = make(n, shapes[n], 0)
+                return same[key]
             length = lambda: model.length  # noqa: E731
             vocab = cfg.vocab_size
         else:
@@ -533,7 +542,14 @@ def hybrid_bench(args):
                                   "middle group twice = 16 layer runs, feed-forward 4 x width; Llama of 16 layers beside it; "
                                   "width %d, vocabulary 32000, random weights" % W}}
     out.update(rows)
-    if "hybrid" in rows:
+    if args.workload == "nufapel":
+        out["metric"] = "nufapel decoder tokens/s"
+        out["config"]["workload"] = ("Nufapel: (parallel: attention over all positions beside a matrix memory, general delta rule) x 6, the "
+                                     "middle four layers twice = 16 layer runs, 8 of 32 experts of width / 4; the layered hybrid decoder of "
+                                     "equal width and layer runs beside it; width %d, vocabulary 32000, random weights" % W)
+        if "nufapel" in rows:
+            out["value"] = rows["nufapel"]["decode"]["tokens_per_s"]
+    elif "hybrid" in rows:
         out["value"] = rows["hybrid"]["decode"]["tokens_per_s"]
     print(json.dumps(out))
 

@@ -62,7 +62,7 @@ class DecoderModel:
     # -- weights ------------------------------------------------------------
     def set_param(self, name, array):
         """One tensor by its name; f32 arrays or bf16 bits as uint16 (loader.rs:32-68)."""
-        a = np.ascontiguousarray(array)
+        a = np.asarray(array, order="C")  # (ascontiguousarray would give a scalar a dimension)
         dtype = _lib.DTYPE_BF16 if a.dtype == np.uint16 else _lib.DTYPE_F32
         if dtype == _lib.DTYPE_F32 and a.dtype != np.float32:
             a = a.astype(np.float32)

@@ -145,6 +145,22 @@ def llama_beside(width, weight_dtype="bf16", layers=16, max_seq_len=8192):
                 rms_norm_eps=1e-6, max_seq_len=max_seq_len, rope_theta=10000.0, weight_dtype=weight_dtype)
 
 
+def nufapel_shape(width, weight_dtype="bf16", groups=3, max_seq_len=8192):
+    """A Nufapel HybridConfig of hybrid_shape's width, layer runs and loop: parallel mixers (attention as there but over all
+    positions, a matrix memory of half the width beside it) and general delta rules in turn, a dense feed-forward in the
+    first layer and 32 experts of width / 4, 8 at a time, in the others."""
+    from .hybrid import HybridConfig, HybridLayer
+    moe = dict(ff=width // 4, ff_kind="experts", experts=32, top=8, groups=8, keep=4, router_scale=1.0, limit=7.0)
+    par = dict(heads=width // 64, kv_heads=max(width // 256, 1), dim=64, vdim=64, scale=0.125, bias_rows=32, bias_max=128,
+               mem_heads=max(width // 256, 1), mem_dim=128, mem_vdim=128, gate_cap=15.0)
+    gen = dict(heads=width // 64, kv_heads=width // 64, dim=64, vdim=64, rank_lo=64)
+    layers = [HybridLayer("parallel" if i % 2 == 0 else "general_delta", **(gen if i % 2 else par),
+                          **(moe if i else dict(ff=4 * width, ff_kind="gelu"))) for i in range(4 * groups)]
+    mid = groups // 2 * 4
+    return HybridConfig(32000, width, layers, mid, mid + 4, 2, max_seq_len=max_seq_len, weight_dtype=weight_dtype, norm_kind="dyt",
+                        loop_kind="add", residual_gate=True, max_positions=max_seq_len, logit_softcap=30.0)
+
+
 def hybrid_param(name, shape, seed):
     """A tensor of a hybrid model: N(0, fan_in^-1/2) matrices, decays that let the state live for tens of tokens."""
     rng = _rng(seed, name)
@@ -166,4 +182,29 @@ def hybrid_param(name, shape, seed):
         return np.abs(a) * np.float32(0.3)
     if leaf in ("w0", "dt_bias"):
         return a * np.float32(0.5) - np.float32(2.5)
+    return a * np.float32(0.3)
+
+
+def nufapel_param(name, shape, seed):
+    """A tensor of a Nufapel model: N(0, fan_in^-1/2) matrices; norms whose tanh bends, gates that remember for tens of
+    tokens, sinks and distance biases of the size of a score."""
+    rng = _rng(seed, name)
+    a = rng.standard_normal(shape, dtype=np.float32)
+    leaf = name.split(".")[-1]
+    if leaf == "alpha":
+        return np.float32(0.6) + np.float32(0.1) * np.asarray(a, np.float32)
+    if name.endswith(".b") and "norm" in name or name in ("pos", "loop.step"):
+        return a * np.float32(0.3)
+    if leaf in ("norm1", "norm2", "norm", "out", "temp"):
+        return 1 + a * np.float32(0.2)
+    if leaf in ("rel", "sink"):
+        return a
+    if name.endswith(".f.b"):
+        return 3 + a
+    if name.endswith(".b") or leaf == "w0":
+        return a
+    if name == "embed":
+        return a
+    if len(shape) == 2:
+        return a * np.float32(shape[-1] ** -0.5 * (2.0 if name.endswith(("mlp.router", "head", "left.q")) else 1.0))
     return a * np.float32(0.3)
