@@ -8,8 +8,10 @@
 typedef float v4f __attribute__((ext_vector_type(4)));
 typedef unsigned int v4u __attribute__((ext_vector_type(4)));
 
-// A workgroup's choice for one token.  An expert's place is the number of better ones (ties: the lower index first), so no
-// step waits for the one before; every index in `sel` is valid whatever the logits are.
+// One wavefront's choice for one token: its LDS accesses execute in order, so its phases need no workgroup barrier (the wave
+// barrier emits no instruction; it keeps the compiler from moving LDS accesses across it).  An expert's place is the number of
+// better ones (ties: the lower index first), so no choice waits for the one before; every index in `sel` is valid
+// whatever the logits are.
 struct RouteLds {
     float s[EXPERTS_MAX], group[EXPERTS_MAX];
     int kept[EXPERTS_MAX];
@@ -17,52 +19,50 @@ struct RouteLds {
     float w[EXPERTS_MAX_TOP];
 };
 __device__ __forceinline__ void route_token(RouteLds &l, const RouterShape &r, const float *__restrict__ z) {
-    const int tid = threadIdx.x, nt = blockDim.x, size = r.experts / r.groups;
-    for (int e = tid; e < r.experts; e += nt) l.s[e] = 1.0f / (1.0f + expf(-z[e]));
-    for (int j = tid; j < r.top; j += nt) {
-        l.sel[j] = 0;
-        l.w[j] = 0.f;
+    const int lane = threadIdx.x & 63, size = r.experts / r.groups;
+    for (int e = lane; e < r.experts; e += 64) l.s[e] = 1.0f / (1.0f + expf(-z[e]));
+    if (lane < r.top) {
+        l.sel[lane] = 0;
+        l.w[lane] = 0.f;
     }
-    __syncthreads();
-    for (int g = tid; g < r.groups; g += nt) {
-        float a = -INFINITY, b = 0.f;  // the two largest (a group of one counts its one)
-        for (int i = 0; i < size; ++i) {
-            const float v = l.s[g * size + i];
-            if (v > a) {
-                b = i ? a : 0.f;
-                a = v;
-            } else if (v > b) {
-                b = v;
+    __builtin_amdgcn_wave_barrier();
+    if (r.groups > r.keep) {
+        for (int g = lane; g < r.groups; g += 64) {
+            float a = -INFINITY, b = 0.f;  // the two largest (a group of one counts its one)
+            for (int i = 0; i < size; ++i) {
+                const float v = l.s[g * size + i];
+                b = v > a ? (i ? a : 0.f) : fmaxf(v, b);
+                a = fmaxf(v, a);
             }
+            l.group[g] = a + b;
         }
-        l.group[g] = a + b;
+        __builtin_amdgcn_wave_barrier();
+        for (int g = lane; g < r.groups; g += 64) {
+            int better = 0;
+            for (int o = 0; o < r.groups; ++o) better += l.group[o] > l.group[g] || (l.group[o] == l.group[g] && o < g);
+            l.kept[g] = better < r.keep;
+        }
+        __builtin_amdgcn_wave_barrier();
+        // (an expert that cannot be chosen: below every score)
+        for (int e = lane; e < r.experts; e += 64)
+            if (!l.kept[e / size]) l.s[e] = -1.f;
+        __builtin_amdgcn_wave_barrier();
     }
-    __syncthreads();
-    for (int g = tid; g < r.groups; g += nt) {
-        int better = 0;
-        for (int o = 0; o < r.groups; ++o) better += l.group[o] > l.group[g] || (l.group[o] == l.group[g] && o < g);
-        l.kept[g] = better < r.keep;
-    }
-    __syncthreads();
-    for (int e = tid; e < r.experts; e += nt) {
-        if (!l.kept[e / size]) continue;
+    for (int e = lane; e < r.experts; e += 64) {
         const float mine = l.s[e];
         int better = 0;
-        for (int g = 0; g < r.groups; ++g) {
-            if (!l.kept[g]) continue;
-            for (int o = g * size; o < (g + 1) * size; ++o) better += l.s[o] > mine || (l.s[o] == mine && o < e);
-        }
-        if (better < r.top) {
+#pragma unroll 8
+        for (int o = 0; o < r.experts; ++o) better += l.s[o] > mine || (l.s[o] == mine && o < e);
+        if (better < r.top && mine >= 0.f) {
             l.sel[better] = e;
             l.w[better] = mine;
         }
     }
-    __syncthreads();
-    float sum = 0.f;
-    for (int j = 0; j < r.top; ++j) sum += l.w[j];
-    __syncthreads();
-    for (int j = tid; j < r.top; j += nt) l.w[j] = l.w[j] / (sum + 1e-20f) * r.scale;
-    __syncthreads();
+    __builtin_amdgcn_wave_barrier();
+    const float w = lane < r.top ? l.w[lane] : 0.f;
+    const float sum = wave_sum(w);
+    if (lane < r.top) l.w[lane] = w / (sum + 1e-20f) * r.scale;
+    __builtin_amdgcn_wave_barrier();
 }
 
 __global__ __launch_bounds__(64) void route_kernel(RouterShape r, const float *__restrict__ z, int z_stride, int *__restrict__ sel,
@@ -107,7 +107,7 @@ __device__ __forceinline__ float dot16_e(const v4u raw, const float *xs) {
 }
 
 // A wavefront takes one (expert, channel) at a time: its gate and up rows, ED_LOADS / 2 pieces of each in flight.  Every
-// workgroup routes and normalises for itself; the first one leaves the choice for the down product.
+// workgroup routes (one wavefront) and normalises (the others) for itself; the first one leaves the choice for the down product.
 template <bool BF16>
 __global__ __launch_bounds__(ED_THREADS) void experts_up_kernel(ExpertsArgs a) {
     constexpr int VEC = BF16 ? 8 : 4, ESZ = BF16 ? 2 : 4, SWEEP = 64 * VEC, U = ED_LOADS / 2;
@@ -115,7 +115,8 @@ __global__ __launch_bounds__(ED_THREADS) void experts_up_kernel(ExpertsArgs a) {
     LUMEN_DYNAMIC_LDS(float, xs);
     const int tid = threadIdx.x, lane = tid & 63, K = a.dim, F = a.ff, kpad = (K + SWEEP * U - 1) / (SWEEP * U) * (SWEEP * U);
     const float alpha = *a.norm_alpha;
-    for (int k = tid * 4; k < kpad; k += ED_THREADS * 4) {
+    if (tid < 64) route_token(l, a.r, a.z);  // the first wavefront routes, the others normalise
+    for (int k = (tid - 64) * 4; k < kpad && tid >= 64; k += (ED_THREADS - 64) * 4) {
         v4f v = {0.f, 0.f, 0.f, 0.f};
         if (k < K) {
             const v4f x = *(const v4f *)(a.x + k), g = *(const v4f *)(a.norm_w + k), b = *(const v4f *)(a.norm_b + k);
@@ -124,7 +125,7 @@ __global__ __launch_bounds__(ED_THREADS) void experts_up_kernel(ExpertsArgs a) {
         }
         *(v4f *)(xs + k) = v;
     }
-    route_token(l, a.r, a.z);  // (ends with a barrier: xs is complete too)
+    __syncthreads();
     if (blockIdx.x == 0 && tid < a.r.top) a.sel[tid] = l.sel[tid];
     const int units = a.r.top * F, nw = gridDim.x * ED_WAVES;
     const size_t row_bytes = (size_t)K * ESZ;

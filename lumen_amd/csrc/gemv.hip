@@ -396,7 +396,8 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
     constexpr int ESZ = BF16 ? 2 : 4;
     // (several products in one launch: this workgroup's rows)
     const int seg = PRO == PRO_SHIFT ? (int)blockIdx.y : 0;
-    const int K = K_hot, D = D_hot;
+    const bool other = PRO == PRO_PAIR && blockIdx.y > 0;  // (the second product of a pair)
+    const int K = other ? a.K2 : K_hot, D = D_hot;
     const int N = PRO == PRO_SHIFT ? (seg == a.shift_segs - 1 ? a.shift_last_rows : a.shift_rows) : N_hot;
     const int kpad = (K + PIECE - 1) / PIECE * PIECE;  // xs is zero from K to kpad
 
@@ -406,8 +407,9 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
     const int nw = nblocks * nwaves;
     const int nunits = (N + R - 1) / R;
     const size_t row_bytes = (size_t)K * ESZ;
-    const char *Wb = (const char *)W_hot + (PRO == PRO_SHIFT ? (size_t)seg * a.shift_rows * row_bytes : 0);
-    float *y_out = a.y + (PRO == PRO_SHIFT ? (size_t)seg * a.shift_rows : 0);
+    const char *Wb = (const char *)(other ? a.W2 : W_hot) + (PRO == PRO_SHIFT ? (size_t)seg * a.shift_rows * row_bytes : 0);
+    float *y_out = (other ? a.y2 : a.y) + (PRO == PRO_SHIFT ? (size_t)seg * a.shift_rows : 0);
+    const float *x_in = other ? a.x2 : x_hot;
     if (PRO == PRO_SHIFT && (int)blockIdx.x * nwaves >= (N + R - 1) / R) return;  // (no unit of a short segment here)
     const int half_d = D >> 1;
 
@@ -448,12 +450,12 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
         }
     };
 
-    constexpr bool EARLY = XB == 0 && (PRO == PRO_NONE || PRO == PRO_RMSNORM || PRO == PRO_DYT);
+    constexpr bool EARLY = XB == 0 && (PRO == PRO_NONE || PRO == PRO_RMSNORM || PRO == PRO_DYT || PRO == PRO_PAIR);
     v4f xe[GEMV_EARLY], ge[GEMV_EARLY], be[GEMV_EARLY];
     const float dyt_alpha = PRO == PRO_DYT ? *a.norm_alpha : 0.f;
     // (with a row selector -- the first layer's gather -- the address of x needs a trip to memory itself:
     // then the weights go first)
-    if (EARLY && !row_sel_hot) request_early<PRO>(xe, ge, be, x_hot, norm_w_hot, a.norm_b, K, nwaves * 64);
+    if (EARLY && !row_sel_hot) request_early<PRO>(xe, ge, be, x_in, norm_w_hot, a.norm_b, K, nwaves * 64);
 
     // the first weights of this wavefront start streaming before x is staged: they do not depend on it
     v4u rawA[R][U], rawB[R][U];
@@ -469,7 +471,7 @@ __global__ __launch_bounds__(GEMV_MAX_WAVES * 64) void gemv_kernel(const void *W
     const int T = my_units * np;
 
     long sel_off = 0;
-    const float *xin = x_hot;
+    const float *xin = x_in;
     if (row_sel_hot) {
         sel_off = (long)(*row_sel_hot) * a.row_stride;
         if (a.x_sel) xin += sel_off;
@@ -753,6 +755,8 @@ static void launch_pro(const GemvArgs &a, dim3 grid, int threads, size_t lds, hi
         hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_POLYNORM, EPI_RESIDUAL, (XB == 0 ? 1 : XB), KA>), grid, dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
     else if (a.pro == PRO_SHIFT)  // token-shift products (launch_gemv checks): plain store
         hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_SHIFT, EPI_STORE, (XB == 0 ? 1 : XB), KA>), dim3(grid.x, a.shift_segs), dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
+    else if (a.pro == PRO_PAIR)  // two output projections (launch_gemv checks)
+        hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_PAIR, EPI_STORE, XB, KA>), dim3(grid.x, 2), dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
     else if (a.pro == PRO_DYT) {  // projections and the head (launch_gemv checks)
         if (a.epi == EPI_ARGMAX)
             hipLaunchKernelGGL((gemv_kernel<BF16, R, PRO_DYT, EPI_ARGMAX, XB, KA>), grid, dim3(threads), lds, s, a.W, a.x, a.norm_w, a.row_sel, a.N, a.K, a.D, (int)grid.x, threads >> 6, a);
@@ -828,7 +832,7 @@ GemvPick gemv_pick(int num_cus, int N, int K, int w_bf16, int pro, int epi, bool
     // at a time from three pieces per thread on.
     const int x_pieces = (kpad + p.threads * 4 - 1) / (p.threads * 4);
     const int nunits = (N + p.R - 1) / p.R;
-    const bool early_x = (pro == PRO_NONE || pro == PRO_RMSNORM || pro == PRO_DYT) && x_pieces <= GEMV_EARLY && kpad / piece <= 2 &&
+    const bool early_x = (pro == PRO_NONE || pro == PRO_RMSNORM || pro == PRO_DYT || pro == PRO_PAIR) && x_pieces <= GEMV_EARLY && kpad / piece <= 2 &&
                          nunits <= p.blocks * (p.threads / 64);
     p.xb = early_x ? 0 : x_pieces > 2 ? 4 : 1;
     p.ka = K % piece == 0;  // whole pieces: no clamped load positions
@@ -867,6 +871,9 @@ int launch_gemv(lumen_ctx *ctx, const GemvArgs &a) {
             LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over attention partials: one row per unit, residual epilogue, at most %d slices (got %d)",
                        GEMV_FOLD_MAX_SLICES, a.attn_nslices);
     }
+    if (a.pro == PRO_PAIR && (a.epi != EPI_STORE || !a.W2 || !a.x2 || !a.y2 || a.K2 < 1 || a.K2 > a.K || a.K2 % vec || a.row_sel ||
+                             (((uintptr_t)a.W2 | (uintptr_t)a.x2) & 15)))
+        LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV of a pair: a second product of no more columns (K=%d, K2=%d), store epilogue", a.K, a.K2);
     if (a.pro == PRO_DYT && (!a.norm_w || !a.norm_b || !a.norm_alpha || (a.epi != EPI_STORE && a.epi != EPI_ARGMAX)))
         LUMEN_FAIL(LUMEN_ERR_INVALID, "GEMV over a Dynamic Tanh input: gain, shift and alpha, store or arg-max epilogue");
     if (a.epi == EPI_RESIDUAL && a.res_gate && !a.res_gate_b) LUMEN_FAIL(LUMEN_ERR_INVALID, "gated residual: no gate bias");
@@ -900,6 +907,8 @@ int launch_gemv(lumen_ctx *ctx, const GemvArgs &a) {
     const int threads = p.threads;
     const size_t lds = p.lds;
     dim3 grid(blocks);
+    const int pieces_of = 64 * vec * (8 / p.R);
+    const bool whole = p.ka && (a.pro != PRO_PAIR || a.K2 % pieces_of == 0);  // no clamped load positions in either product
 #define LAUNCH_GEMV_K(BF, RR, KAV)                                                       \
     do {                                                                                 \
         if (p.xb == 0) launch_pro<BF, RR, 0, KAV>(a, grid, threads, lds, ctx->stream);      \
@@ -908,7 +917,7 @@ int launch_gemv(lumen_ctx *ctx, const GemvArgs &a) {
     } while (0)
 #define LAUNCH_GEMV(BF, RR)                  \
     do {                                     \
-        if (p.ka) LAUNCH_GEMV_K(BF, RR, true); \
+        if (whole) LAUNCH_GEMV_K(BF, RR, true); \
         else LAUNCH_GEMV_K(BF, RR, false);   \
     } while (0)
     if (a.w_bf16) {

@@ -833,9 +833,10 @@ static int enqueue_decode_step(lumen_hybrid *m, const Tap *tap = nullptr) {
             LUMEN_TRY(timed(m, wkv ? HC_WKV : HC_DELTA, do_rec, &a));
         }
         if (L.c.mixer == LUMEN_MIXER_PARALLEL) {
+            // both output projections in one launch, the one of more columns first
             GemvArgs g = gemv_args(m, L.w_o, W, L.od, m->mixed, m->pair);
-            LUMEN_TRY(timed(m, HC_OUT, do_gemv, &g));
-            g = gemv_args(m, L.w_o2, W, L.od2, m->mixed2, m->pair + W);
+            g.pro = PRO_PAIR; g.W2 = L.w_o2; g.x2 = m->mixed2; g.y2 = m->pair + W; g.K2 = L.od2;
+            if (L.od2 > L.od) { std::swap(g.W, g.W2); std::swap(g.x, g.x2); std::swap(g.y, g.y2); std::swap(g.K, g.K2); }
             LUMEN_TRY(timed(m, HC_OUT, do_gemv, &g));
             GatedResidualArgs p = {};
             p.x = cur; p.y = m->pair; p.y2 = m->pair + W; p.w1 = L.out1; p.w2 = L.out2; p.pair_scale = 0.5f; p.eps = c.norm_eps;

@@ -100,8 +100,9 @@ struct lumen_kv_cache {
 // element by element, N divides by the root mean square over norm_dim elements); norm_w = {a, b, c, e}.
 // PRO_SHIFT: RMSNorm, then the token-shift mix h + (h' - h) mu of h with the previous token's h'; gridDim.y products
 // at once, each with a mix of its own (GemvArgs::shift_*).
+// PRO_PAIR: two products of N rows in one launch, y [N] = W x and y2 [N] = W2 x2 (GemvArgs::W2, x2, y2, K2), plain stores.
 // PRO_DYT: x enters as tanh(alpha x) norm_w + norm_b (Dynamic Tanh), alpha one float in device memory.
-enum GemvPro { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_ATTN_FOLD = 2, PRO_POLYNORM = 3, PRO_SHIFT = 4, PRO_DYT = 5 };
+enum GemvPro { PRO_NONE = 0, PRO_RMSNORM = 1, PRO_ATTN_FOLD = 2, PRO_POLYNORM = 3, PRO_SHIFT = 4, PRO_DYT = 5, PRO_PAIR = 6 };
 enum GemvEpi { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ARGMAX = 3, EPI_ROPE_QKV = 4, EPI_EXPERT_ACT = 5 };
 
 struct GemvArgs {
@@ -112,6 +113,10 @@ struct GemvArgs {
     int w_bf16;
     int pro, epi;
     const float *norm_w;  // PRO_RMSNORM, PRO_DYT: gain [K]
+    const void *W2;         // PRO_PAIR
+    const float *x2;
+    float *y2;
+    int K2;
     const float *norm_b, *norm_alpha;  // PRO_DYT: shift [K], one float
     float eps;
     const float *residual;  // EPI_RESIDUAL: [N]

@@ -221,20 +221,47 @@ __global__ __launch_bounds__(WD_THREADS) void window_decode_kernel(WindowAttnArg
     }
 }
 
-// Adds the slices of a head in slice order: one workgroup per head.
+// Adds the slices of a head in slice order: one workgroup per head, a thread per channel.  The slices' maxima and sums
+// are looked at by one wavefront, 64 at a time; a channel's values are requested WM_AHEAD slices at a time, the first of them
+// before the weights are known.
+#define WM_AHEAD 16
+#define WM_SLICES 1024
 __global__ __launch_bounds__(256) void window_merge_kernel(WindowAttnArgs a) {
-    const int h = blockIdx.x, Dv = a.vdim, pos = *a.pos_dev;
-    const int used = (min(a.window, pos + 1) + WINDOW_SLICE_KEYS - 1) / WINDOW_SLICE_KEYS;
+    __shared__ float ws[WM_SLICES];
+    __shared__ float total;
+    const int h = blockIdx.x, tid = threadIdx.x, Dv = a.vdim, d = min(tid, Dv - 1);
     const float *part = a.part + (size_t)h * a.slices * (Dv + 2);
-    float m = -INFINITY;
-    for (int s = 0; s < used; ++s) m = fmaxf(m, part[(size_t)s * (Dv + 2) + Dv]);
-    float l = 0.f;
-    for (int s = 0; s < used; ++s) l = fmaf(part[(size_t)s * (Dv + 2) + Dv + 1], __builtin_amdgcn_exp2f(part[(size_t)s * (Dv + 2) + Dv] - m), l);
-    for (int d = threadIdx.x; d < Dv; d += 256) {
-        float o = 0.f;
-        for (int s = 0; s < used; ++s) o = fmaf(part[(size_t)s * (Dv + 2) + d], __builtin_amdgcn_exp2f(part[(size_t)s * (Dv + 2) + Dv] - m), o);
-        a.out[h * Dv + d] = o / l * (a.gate ? gate_w(a.gate[a.gate_heads ? h : h * Dv + d], a.gate_act) : 1.0f);
+    const float gate = a.gate ? a.gate[a.gate_heads ? h : h * Dv + d] : 0.f;
+    const int used = min(a.slices, (min(a.window, *a.pos_dev + 1) + WINDOW_SLICE_KEYS - 1) / WINDOW_SLICE_KEYS);
+    float v[WM_AHEAD];
+    auto fetch = [&](int s0) {
+#pragma unroll
+        for (int i = 0; i < WM_AHEAD; ++i) v[i] = part[(size_t)min(s0 + i, used - 1) * (Dv + 2) + d];
+    };
+    fetch(0);
+    if (tid < 64) {
+        const int mine = min(tid, used - 1);
+        const float m0 = part[(size_t)mine * (Dv + 2) + Dv], l0 = part[(size_t)mine * (Dv + 2) + Dv + 1];
+        float m = m0;
+        for (int s = tid + 64; s < used; s += 64) m = fmaxf(m, part[(size_t)s * (Dv + 2) + Dv]);
+        m = wave_max(m);
+        float l = 0.f;
+        for (int s = tid; s < used; s += 64) {
+            const float w = __builtin_amdgcn_exp2f((s == tid ? m0 : part[(size_t)s * (Dv + 2) + Dv]) - m);
+            ws[s] = w;
+            l = fmaf(s == tid ? l0 : part[(size_t)s * (Dv + 2) + Dv + 1], w, l);
+        }
+        l = wave_sum(l);
+        if (tid == 0) total = l;
     }
+    __syncthreads();
+    float o = 0.f;
+    for (int s0 = 0; s0 < used; s0 += WM_AHEAD) {
+        if (s0) fetch(s0);
+#pragma unroll
+        for (int i = 0; i < WM_AHEAD; ++i) o = s0 + i < used ? fmaf(v[i], ws[s0 + i], o) : o;
+    }
+    if (tid < Dv) a.out[h * Dv + tid] = o / total * (a.gate ? gate_w(gate, a.gate_act) : 1.0f);
 }
 
 int launch_window_attn_decode(lumen_ctx *ctx, const WindowAttnArgs &a) {
@@ -251,6 +278,7 @@ int launch_window_attn_decode(lumen_ctx *ctx, const WindowAttnArgs &a) {
     else if (db == 2) WD_LAUNCH(2);
     else WD_LAUNCH(4);
 #undef WD_LAUNCH
+    if (a.slices > WM_SLICES) LUMEN_FAIL(LUMEN_ERR_UNSUPPORTED, "window attention: %d slices of a decode step (at most %d)", a.slices, WM_SLICES);
     if (a.slices > 1 && !a.leave_slices) hipLaunchKernelGGL(window_merge_kernel, dim3(a.heads), dim3(256), 0, ctx->stream, a);
     LUMEN_CHECK_LAUNCH();
     return LUMEN_OK;
@@ -308,7 +336,8 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
     float *ks = lds, *vs = lds + WP_K * kld;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
     const int h = blockIdx.y, hk = h / (a.heads / a.kv_heads), D = a.dim, Dv = a.vdim;
-    const int t0 = blockIdx.x * WP_Q, tw = t0 + wave * 16, t = tw + c;  // first token of the workgroup / wavefront, own token
+    // (the last queries see the most keys: their workgroups start first)
+    const int t0 = (int)(gridDim.x - 1 - blockIdx.x) * WP_Q, tw = t0 + wave * 16, t = tw + c;  // first token of the workgroup / wavefront, own token
     const int last = min(t0 + WP_Q, a.s) - 1;
     const int i = a.pos + t;  // own position
     const ScoreShape shape(a.scale * (a.temp ? a.temp[h] : 1.f), a.softcap, a.r1 ? a.r1[h] : 0.f, a.r1 ? a.r2[h] : 0.f, a.r1 != nullptr);

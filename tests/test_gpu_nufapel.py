@@ -437,3 +437,13 @@ def test_trace_runner(tmp_path):
     assert max_rel(read(0), la[[24, 3]]) < 5e-5
     assert max_rel(read(2), la[[26, 29]]) < 5e-5
     assert max_rel(read(3), lb[[16]]) < 5e-5
+
+
+def test_tiny_model(tmp_path):
+    """Every mechanism once at the smallest sizes: a prompt, a portion of two, decoding."""
+    cfg = nu.config(8, 11, [nu.parallel((2, 1, 4, 4), (1, 4, 3), nu.moe(8, 4, 2, (2, 1)), bias_max=20), nu.general(1, 4, nu.dense(8))], loop=(0, 1, 2),
+                    positions=16)
+    params = nu.make_params(cfg, seed=11, rank=2, bias_rows=4)
+    model = hu.load(tmp_path, cfg, params, max_seq_len=16)
+    toks = tokens_of(cfg, 6)
+    assert max_rel(hu.run(model, toks, [3, 2, 1]), npn.forward(cfg, params, toks)) < 5e-5
