@@ -482,7 +482,8 @@ def hybrid_bench(args):
                     return make(n, shapes[n], 0)
                 key = n.split(".")[-1]
                 if key not in same:
-                    same[key] = make(n, shapes[n], 0)
+                    a = make(n, shapes[n], 0)
+                    same[key] = synth.bf16_round(a).reshape(shapes[n]) if dt == "bf16" else a
                 return same[key]
             length = lambda: model.length  # noqa: E731
             vocab = cfg.vocab_size
