@@ -269,13 +269,20 @@ int launch_experts_down(lumen_ctx *ctx, const ExpertsArgs &a) {
 
 // ------------------------------------------------------------------ prompt
 // plan: sel [s * top] | a_rows [s * top] | c_rows [s * top] | tiles [max_tiles][3]
-static int plan_tiles(int s, const RouterShape &r) { return (int)(((long)s * r.top + GEMM_GROUP_ROWS - 1) / GEMM_GROUP_ROWS) + std::min(r.experts, s * r.top); }
-size_t experts_plan_ints(int s, const RouterShape &r) { return (size_t)3 * s * r.top + (size_t)3 * plan_tiles(s, r); }
+// Rows of a tile by the mean number of tokens an expert gets: a few and the products are a matter of reading the experts'
+// weights (the streaming kernel's 16 rows), more and the matrix cores' 128-row tiles take them (8 of 32 experts of width
+// 512 on rows of 2048, prompt passes of 16 / 64 / 96 tokens: 2.8 / 3.9 / 4.5 ms with the former, 3.5 / 4.1 / 4.3 with the latter;
+// 32 streamed rows are never the best).
+#define EXPERTS_STREAM_ROWS 16
+static int group_rows(int s, const RouterShape &r) { return (long)s * r.top <= (long)EXPERTS_STREAM_ROWS * r.experts ? 16 : 128; }
+static int plan_tiles(int s, const RouterShape &r, int rows) { return (int)(((long)s * r.top + rows - 1) / rows) + std::min(r.experts, s * r.top); }
+// (for up to s tokens)
+size_t experts_plan_ints(int s, const RouterShape &r) { return (size_t)3 * s * r.top + (size_t)3 * plan_tiles(s, r, 16); }
 
 // One workgroup: counts per expert, where each expert's rows start, the tiles, and every (token, choice)'s row.  The order
 // of an expert's rows is whatever the counters give out; no row's values depend on it.
 #define PLAN_THREADS 1024
-__global__ __launch_bounds__(PLAN_THREADS) void experts_plan_kernel(int *plan, int n, int top, int experts, int max_tiles) {
+__global__ __launch_bounds__(PLAN_THREADS) void experts_plan_kernel(int *plan, int n, int top, int experts, int max_tiles, int tile_rows) {
     __shared__ int count[EXPERTS_MAX], start[EXPERTS_MAX + 1], tile0[EXPERTS_MAX + 1];
     const int tid = threadIdx.x;
     const int *sel = plan;
@@ -287,7 +294,7 @@ __global__ __launch_bounds__(PLAN_THREADS) void experts_plan_kernel(int *plan, i
     if (tid < 64) {  // prefix sums over the experts, 64 at a time
         int rows = 0, tl = 0;
         for (int e0 = 0; e0 < experts; e0 += 64) {
-            const int e = e0 + tid, c = e < experts ? count[e] : 0, t = (c + GEMM_GROUP_ROWS - 1) / GEMM_GROUP_ROWS;
+            const int e = e0 + tid, c = e < experts ? count[e] : 0, t = (c + tile_rows - 1) / tile_rows;
             int sc = c, st = t;
 #pragma unroll
             for (int d = 1; d < 64; d <<= 1) {
@@ -308,10 +315,10 @@ __global__ __launch_bounds__(PLAN_THREADS) void experts_plan_kernel(int *plan, i
     }
     __syncthreads();
     for (int e = tid; e < experts; e += PLAN_THREADS)
-        for (int r = 0, t = tile0[e]; r < count[e] && t < max_tiles; r += GEMM_GROUP_ROWS, ++t) {
+        for (int r = 0, t = tile0[e]; r < count[e] && t < max_tiles; r += tile_rows, ++t) {
             tiles[3 * t] = e;
             tiles[3 * t + 1] = start[e] + r;
-            tiles[3 * t + 2] = min(GEMM_GROUP_ROWS, count[e] - r);
+            tiles[3 * t + 2] = min(tile_rows, count[e] - r);
         }
     for (int t = tile0[experts] + tid; t < max_tiles; t += PLAN_THREADS) tiles[3 * t] = tiles[3 * t + 1] = tiles[3 * t + 2] = 0;
     __syncthreads();
@@ -324,12 +331,12 @@ __global__ __launch_bounds__(PLAN_THREADS) void experts_plan_kernel(int *plan, i
 
 int launch_experts_prefill(lumen_ctx *ctx, const ExpertsArgs &a) {
     if (a.s <= 0) return LUMEN_OK;
-    const int n = a.s * a.r.top, max_tiles = plan_tiles(a.s, a.r);
+    const int n = a.s * a.r.top, rows = group_rows(a.s, a.r), max_tiles = plan_tiles(a.s, a.r, rows);
     LUMEN_TRY(launch_route(ctx, a.r, a.z, a.z_stride, a.s, a.plan, a.sel_w));
-    hipLaunchKernelGGL(experts_plan_kernel, dim3(1), dim3(PLAN_THREADS), 0, ctx->stream, a.plan, n, a.r.top, a.r.experts, max_tiles);
+    hipLaunchKernelGGL(experts_plan_kernel, dim3(1), dim3(PLAN_THREADS), 0, ctx->stream, a.plan, n, a.r.top, a.r.experts, max_tiles, rows);
     LUMEN_CHECK_LAUNCH();
     GemmArgs g = {};
-    g.w_bf16 = a.w_bf16; g.M = n; g.tiles = a.plan + 3 * (size_t)n;
+    g.w_bf16 = a.w_bf16; g.group_rows = rows; g.M = n; g.tiles = a.plan + 3 * (size_t)n;
     g.A = a.rows; g.a_rows = a.plan + n; g.W = a.w_up; g.C = a.p_act; g.N = 2 * a.ff; g.K = a.dim; g.epi = EPI_EXPERT_ACT; g.limit = a.limit;
     LUMEN_TRY(launch_gemm_grouped(ctx, g, max_tiles));
     g.A = a.p_act; g.a_rows = nullptr; g.c_rows = a.plan + 2 * (size_t)n; g.W = a.w_down; g.C = a.out; g.N = a.dim; g.K = a.ff; g.epi = EPI_STORE;

@@ -589,8 +589,16 @@ __global__ __launch_bounds__(SK_THREADS) void gemm_skinny_kernel(GemmArgs a, int
 typedef float v4acc __attribute__((ext_vector_type(4)));
 // BF16: W holds bf16 bits; widened by a shift on the way into the operand registers like src/loader.rs:58 widens them at
 // load time, so the products are those of f32 weights with the same values.
-template <int MT, bool BF16, int EPI, bool PARTIAL>
+template <int MT, bool BF16, int EPI, bool PARTIAL, bool GROUPED = false>
 __global__ __launch_bounds__(256) void gemm_stream_kernel(GemmArgs a) {
+    int row0 = 0;  // of the sorted rows
+    if (GROUPED) {  // (uniform)
+        const int *tile = a.tiles + 3 * blockIdx.y;
+        if (tile[2] <= 0) return;
+        row0 = tile[1];
+        a.M = tile[2];
+        a.W = (const char *)a.W + (size_t)tile[0] * a.N * a.K * (BF16 ? 2 : 4);
+    }
     constexpr int DW = BF16 ? 16 : 8;  // blocks of W in flight per wavefront (16 KB)
     constexpr int WP = BF16 ? 1 : 2;   // 16-byte pieces of a W block per lane
     __shared__ __align__(16) float stage_w[4][16 * GS_LD];
@@ -627,7 +635,10 @@ __global__ __launch_bounds__(256) void gemm_stream_kernel(GemmArgs a) {
 #pragma unroll
     for (int t = 0; t < MT; ++t)
 #pragma unroll
-        for (int i = 0; i < 2; ++i) ap[t][i] = A + (size_t)min(t * 16 + arow + 8 * i, M - 1) * K + ak;
+        for (int i = 0; i < 2; ++i) {
+            const int r = row0 + min(t * 16 + arow + 8 * i, M - 1);
+            ap[t][i] = A + (size_t)(GROUPED && a.a_rows ? a.a_rows[r] : r) * K + ak;
+        }
     v4u vw[DW][WP];
     v4f va[GS_DA][MT][2];
     auto fetch_w = [&](int slot, int d) {
@@ -741,8 +752,11 @@ __global__ __launch_bounds__(256) void gemm_stream_kernel(GemmArgs a) {
             } else if (EPI == EPI_SWIGLU) {
                 const float up = __shfl_xor(v, 1, 64);
                 if (!(col & 1) && row < M && col < N) a.C[(size_t)row * (N >> 1) + (col >> 1)] = silu_g(v) * up;
+            } else if (EPI == EPI_EXPERT_ACT) {
+                const float up = __shfl_xor(v, 1, 64);
+                if (!(col & 1) && row < M && col < N) a.C[(size_t)(row0 + row) * (N >> 1) + (col >> 1)] = expert_act(v, up, a.limit);
             } else if (row < M && col < N) {
-                const size_t o = (size_t)row * N + col;
+                const size_t o = (GROUPED && a.c_rows ? (size_t)a.c_rows[row0 + row] : (size_t)(row0 + row)) * N + col;
                 a.C[o] = (EPI == EPI_RESIDUAL) ? fmaf(a.alpha, v, a.residual[o]) : v;
             }
         }
@@ -1166,11 +1180,23 @@ int launch_gemm(lumen_ctx *ctx, const GemmArgs &a) {
 }
 
 int launch_gemm_grouped(lumen_ctx *ctx, const GemmArgs &a, int max_tiles) {
-    static_assert(GEMM_GROUP_ROWS == BM, "tiles of the plain kernel");
     if (a.M <= 0 || a.N <= 0 || max_tiles <= 0) return LUMEN_OK;
     if ((((uintptr_t)a.A | (uintptr_t)a.W) & 15) || a.K % (a.w_bf16 ? 8 : 4) || !a.tiles || (a.epi != EPI_STORE && a.epi != EPI_EXPERT_ACT) ||
         (a.epi == EPI_EXPERT_ACT && (a.N & 1)))
         LUMEN_FAIL(LUMEN_ERR_INVALID, "grouped GEMM: K=%d N=%d epilogue %d", a.K, a.N, a.epi);
+    if (a.group_rows == 16) {
+        const dim3 sgrid((a.N + 15) / 16, max_tiles);
+        if (a.w_bf16) {
+            if (a.epi == EPI_STORE) hipLaunchKernelGGL((gemm_stream_kernel<1, true, EPI_STORE, false, true>), sgrid, dim3(256), 0, ctx->stream, a);
+            else hipLaunchKernelGGL((gemm_stream_kernel<1, true, EPI_EXPERT_ACT, false, true>), sgrid, dim3(256), 0, ctx->stream, a);
+        } else {
+            if (a.epi == EPI_STORE) hipLaunchKernelGGL((gemm_stream_kernel<1, false, EPI_STORE, false, true>), sgrid, dim3(256), 0, ctx->stream, a);
+            else hipLaunchKernelGGL((gemm_stream_kernel<1, false, EPI_EXPERT_ACT, false, true>), sgrid, dim3(256), 0, ctx->stream, a);
+        }
+        LUMEN_CHECK_LAUNCH();
+        return LUMEN_OK;
+    }
+    if (a.group_rows != BM) LUMEN_FAIL(LUMEN_ERR_INVALID, "grouped GEMM: tiles of %d rows", a.group_rows);
     const dim3 grid((a.N + BN - 1) / BN, max_tiles);
     if (a.w_bf16) {
         if (a.epi == EPI_STORE) hipLaunchKernelGGL((gemm_bf16x3_kernel<true, EPI_STORE, false, true>), grid, dim3(256), 0, ctx->stream, a);

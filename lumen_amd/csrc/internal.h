@@ -197,10 +197,12 @@ struct GemmArgs {
     const float *norm_w;    // [N] or null
     float *norm_out;
     float norm_eps;
-    // products grouped by expert (launch_gemm_grouped): tile i of BM rows is {expert, first row, rows} of tiles, its weights the
-    // expert's of W [experts][N, K]; row r of the sorted rows reads row a_rows[r] of A (null: r) and is stored in row
-    // c_rows[r] of C (null: r).  Epilogues: store, or EPI_EXPERT_ACT: columns (2c, 2c + 1) = (gate, up) -> C [rows, N / 2]
+    // products grouped by expert (launch_gemm_grouped): tile i, of up to group_rows rows (16: the weight-streaming kernel; 128),
+    // is {expert, first row, rows} of tiles, its weights the expert's of W [experts][N, K]; row r of the sorted rows reads
+    // row a_rows[r] of A (null: r) and is stored in row c_rows[r] of C (null: r).  Epilogues: store, or EPI_EXPERT_ACT: columns
+    // (2c, 2c + 1) = (gate, up) -> C [rows, N / 2]
     const int *tiles, *a_rows, *c_rows;
+    int group_rows;
     float limit;
     // optional, with EPI_STORE: where K is split, leave the partial products [splits, M, N] in the workspace for a
     // consumer that adds them itself (in split order) and report how many there are; 1 = C holds the product
@@ -208,7 +210,6 @@ struct GemmArgs {
     int *splits_used;
 };
 int launch_gemm(lumen_ctx *ctx, const GemmArgs &a);
-#define GEMM_GROUP_ROWS 128  // rows of a tile of a grouped product
 int launch_gemm_grouped(lumen_ctx *ctx, const GemmArgs &a, int max_tiles);  // M: total rows
 // act(gate, up) of a clamped expert
 __device__ __forceinline__ float expert_act(float g, float u, float limit) {

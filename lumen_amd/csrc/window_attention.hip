@@ -328,6 +328,17 @@ __global__ __launch_bounds__(256) void window_append_kernel(WindowAttnArgs a) {
 // are laid out for.
 #define WP_Q 64
 #define WP_K 32
+// Which head and which block of queries a workgroup takes.  Later queries see more keys, and workgroup n runs where
+// workgroups n + 256, n + 512, ... run (round robin over 8 XCDs of 32 compute units): blocks are handed out from the last
+// queries to the first, every other round of 256 in the opposite order, so that a compute unit's workgroups add up to
+// about the same number of keys; neighbouring heads, which share keys, go to one XCD.
+__device__ __forceinline__ void window_prefill_place(int n, int blocks, int heads, int &h, int &tb) {
+    const int round = n >> 8;
+    if ((round & 1) && (round + 1) * 256 <= blocks * heads) n = (round << 8) + ((31 - ((n & 255) >> 3)) << 3) + (n & 7);
+    tb = blocks - 1 - n / heads;
+    h = n % heads;
+    if (heads % 8 == 0) h = (h & 7) * (heads >> 3) + (h >> 3);
+}
 template <int NB, bool FULL>
 __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, int nd_, int nv_) {
     const int nd = FULL ? NB : nd_, nv = FULL ? NB : nv_;
@@ -335,9 +346,10 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(WindowAttnArgs a, i
     const int kld = nd * 16 + 4, vld = nv * 16 + 4;
     float *ks = lds, *vs = lds + WP_K * kld;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
-    const int h = blockIdx.y, hk = h / (a.heads / a.kv_heads), D = a.dim, Dv = a.vdim;
-    // (the last queries see the most keys: their workgroups start first)
-    const int t0 = (int)(gridDim.x - 1 - blockIdx.x) * WP_Q, tw = t0 + wave * 16, t = tw + c;  // first token of the workgroup / wavefront, own token
+    int h, tb;
+    window_prefill_place((int)(blockIdx.y * gridDim.x + blockIdx.x), (int)gridDim.x, a.heads, h, tb);
+    const int hk = h / (a.heads / a.kv_heads), D = a.dim, Dv = a.vdim;
+    const int t0 = tb * WP_Q, tw = t0 + wave * 16, t = tw + c;  // first token of the workgroup / wavefront, own token
     const int last = min(t0 + WP_Q, a.s) - 1;
     const int i = a.pos + t;  // own position
     const ScoreShape shape(a.scale * (a.temp ? a.temp[h] : 1.f), a.softcap, a.r1 ? a.r1[h] : 0.f, a.r1 ? a.r2[h] : 0.f, a.r1 != nullptr);

@@ -242,7 +242,8 @@ def test_router(L, experts, groups, keep, top):  # noqa: F811
         assert len(set(got[t].tolist())) == top and got[t].min() >= 0 and got[t].max() < experts
 
 
-@pytest.mark.parametrize("s,dim,ff,experts,top", [(1, 8, 8, 3, 2), (5, 40, 24, 7, 3), (70, 64, 48, 4, 2), (300, 32, 16, 2, 2), (33, 136, 200, 40, 5)])
+@pytest.mark.parametrize("s,dim,ff,experts,top", [(1, 8, 8, 3, 2), (5, 40, 24, 7, 3), (70, 64, 48, 4, 2), (300, 32, 16, 2, 2), (33, 136, 200, 40, 5),
+                                                    (20, 72, 40, 3, 1), (30, 64, 24, 5, 2), (200, 40, 48, 20, 2)])
 def test_experts_of_a_prompt(L, s, dim, ff, experts, top):  # noqa: F811
     """More tokens than a tile, experts nobody chose, experts everybody chose; the clamps bite."""
     r = rng(s, dim, experts)
