@@ -22,7 +22,7 @@ def test_help_names_the_workloads():
     r = run("--help")
     assert r.returncode == 0
     for word in ("--steps", "--warmup", "--gpus", "decode", "gemv", "prefill", "--max-seq", "--model", "qwen3-0.6b",
-                 "llama2-7b-bf16", "hybrid", "--hybrid-width"):
+                 "llama2-7b-bf16", "hybrid", "nufapel", "--hybrid-width"):
         assert word in r.stdout
 
 
